@@ -1,7 +1,9 @@
-"""Builds libe2h_quant.so (the C-ABI library declared in include/e2h_quant.h) with hipcc for gfx950.
+"""Builds the C-ABI libraries with hipcc for gfx950: libe2h_quant.so (include/e2h_quant.h, the quantized linears and the
+Llama decode step) and libe2h_seq.so (include/e2h_seq.h, the layers with per-sequence state).
 
-The library is built in-tree, next to this file, so that it travels with the source tree; nothing is
-installed into site-packages and no JIT cache is involved.
+The libraries are built in-tree, next to this file, so that they travel with the source tree; nothing is
+installed into site-packages and no JIT cache is involved.  They are separate so that a model that needs one of them
+compiles only that one.
 """
 
 import os
@@ -12,10 +14,12 @@ from pathlib import Path
 
 PKG_DIR = Path(__file__).resolve().parent
 CSRC = PKG_DIR / "csrc"
-LIB_NAME = "libe2h_quant.so"
-LIB_PATH = PKG_DIR / LIB_NAME
+LIB_PATH = PKG_DIR / "libe2h_quant.so"
+SEQ_LIB_PATH = PKG_DIR / "libe2h_seq.so"
 
 SOURCES = ["e2h_abi.hip", "e2h_quantize.hip", "e2h_int4_mm.hip", "e2h_int4_staged.hip", "e2h_int4_rows64.hip", "e2h_int8_mm.hip", "e2h_int8_stream.hip", "e2h_int4_gemm.hip", "e2h_int4_gemm128.hip", "e2h_int8_gemm.hip", "e2h_attention.hip", "e2h_sample.hip", "e2h_probe.hip"]
+
+SEQ_SOURCES = ["e2h_seq_norm.hip", "e2h_seq_attention.hip", "e2h_seq_hgrn2.hip", "e2h_seq_delta.hip"]
 
 # -ffp-contract=off: the quantizers are bit-exact restatements of separate torch ops; an FMA formed
 # across two of them would change codes.  packed-fp32-ops is switched off because some packed float32
@@ -53,12 +57,11 @@ def _run(cmd):
     return proc.stdout
 
 
-def build_library(verbose=False):
-    """Compile every HIP source for gfx950 and link libe2h_quant.so.  Always recompiles."""
+def _compile_and_link(names, lib_path, verbose):
     hipcc = _hipcc()
     obj_dir = PKG_DIR / "build"
     obj_dir.mkdir(exist_ok=True)
-    sources = [s for s in SOURCES if (CSRC / s).exists()]
+    sources = [s for s in names if (CSRC / s).exists()]
 
     def compile_one(src):
         obj = obj_dir / (Path(src).stem + ".o")
@@ -69,11 +72,22 @@ def build_library(verbose=False):
 
     with ThreadPoolExecutor(max_workers=min(len(sources), 6)) as pool:
         objs = list(pool.map(compile_one, sources))
-    tmp = PKG_DIR / (LIB_NAME + ".tmp")
+    tmp = lib_path.with_name(lib_path.name + ".tmp")
     _run([hipcc, "--offload-arch=gfx950", "-shared", "-fPIC", "-o", str(tmp), *map(str, objs)])
-    os.replace(tmp, LIB_PATH)
-    return LIB_PATH
+    os.replace(tmp, lib_path)
+    return lib_path
+
+
+def build_library(verbose=False):
+    """Compile every HIP source of libe2h_quant.so for gfx950 and link it.  Always recompiles."""
+    return _compile_and_link(SOURCES, LIB_PATH, verbose)
+
+
+def build_seq_library(verbose=False):
+    """The same for libe2h_seq.so."""
+    return _compile_and_link(SEQ_SOURCES, SEQ_LIB_PATH, verbose)
 
 
 if __name__ == "__main__":
     print(build_library(verbose=True))
+    print(build_seq_library(verbose=True))

@@ -1,13 +1,13 @@
-"""ctypes binding of libe2h_quant.so (C ABI: include/e2h_quant.h).
+"""ctypes bindings of libe2h_quant.so (C ABI: include/e2h_quant.h) and libe2h_seq.so (include/e2h_seq.h).
 
-The library is loaded from the package directory.  If it has not been built, loading raises: there is
+The libraries are loaded from the package directory.  If one has not been built, loading it raises: there is
 no fallback implementation behind these entry points.
 """
 
 import ctypes
-from ctypes import c_char_p, c_float, c_int, c_int64, c_void_p
+from ctypes import c_char_p, c_float, c_int, c_int32, c_int64, c_void_p
 
-from ._build import LIB_PATH, build_library
+from ._build import LIB_PATH, SEQ_LIB_PATH, build_library, build_seq_library
 
 _P = c_void_p
 _SIGNATURES = {
@@ -63,34 +63,110 @@ _SIGNATURES = {
 
 EXPORTED_SYMBOLS = tuple(_SIGNATURES)
 
+# e2h_dtype values of include/e2h_seq.h
+SEQ_BF16, SEQ_F32 = 0, 1
+
+
+class NormConvArgs(ctypes.Structure):
+    _fields_ = [("dtype", c_int32), ("taps", c_int32), ("batch", c_int64), ("seqlen", c_int64), ("width", c_int64), ("eps", c_float),
+                ("delta_offset", c_float), ("norm_offset", c_float), ("pad_", c_int32), ("x", _P), ("delta", _P), ("delta_weight", _P),
+                ("x_out", _P), ("norm_weight", _P), ("conv", _P), ("tail_in", _P), ("tail_out", _P), ("out", _P), ("input_pos", _P), ("first", _P)]
+
+
+class WindowAttentionArgs(ctypes.Structure):
+    _fields_ = [("dtype", c_int32), ("pad_", c_int32), ("batch", c_int64), ("seqlen", c_int64), ("heads", c_int64), ("kv_heads", c_int64),
+                ("dim", c_int64), ("vdim", c_int64), ("cache_len", c_int64), ("proj", _P), ("ld", c_int64), ("q_off", c_int64),
+                ("k_off", c_int64), ("v_off", c_int64), ("g_off", c_int64), ("q_bias", _P), ("k_bias", _P), ("v_bias", _P), ("k_cache", _P),
+                ("v_cache", _P), ("input_pos", _P), ("first", _P), ("window", c_int64), ("keep_first", c_int64), ("scale", c_float),
+                ("out_scale", c_float), ("out", _P), ("ld_out", c_int64), ("out_off", c_int64)]
+
+
+class Hgrn2Args(ctypes.Structure):
+    _fields_ = [("dtype", c_int32), ("eps", c_float), ("batch", c_int64), ("seqlen", c_int64), ("heads", c_int64), ("dim", c_int64),
+                ("vdim", c_int64), ("proj", _P), ("ld", c_int64), ("q_off", c_int64), ("f_off", c_int64), ("v_off", c_int64), ("f_bias", _P),
+                ("lower", _P), ("norm_weight", _P), ("state", _P), ("input_pos", _P), ("first", _P), ("scratch", _P), ("scratch_bytes", c_int64),
+                ("out_scale", c_float), ("pad_", c_int32), ("out", _P), ("ld_out", c_int64), ("out_off", c_int64)]
+
+
+class DeltaArgs(ctypes.Structure):
+    _fields_ = [("dtype", c_int32), ("taps", c_int32), ("batch", c_int64), ("seqlen", c_int64), ("heads", c_int64), ("kv_heads", c_int64),
+                ("dim", c_int64), ("vdim", c_int64), ("proj", _P), ("ld", c_int64), ("q_off", c_int64), ("k_off", c_int64), ("v_off", c_int64),
+                ("b_off", c_int64), ("a_off", c_int64), ("g_off", c_int64), ("conv", _P), ("tail_in", _P), ("tail_out", _P), ("a_log", _P),
+                ("dt_bias", _P), ("norm_weight", _P), ("state", _P), ("input_pos", _P), ("first", _P), ("scratch", _P), ("scratch_bytes", c_int64),
+                ("eps", c_float), ("out_scale", c_float), ("out", _P), ("ld_out", c_int64), ("out_off", c_int64)]
+
+
+_A = ctypes.POINTER
+_SEQ_SIGNATURES = {
+    "e2h_seq_abi_version": (c_int, []),
+    "e2h_seq_set_option": (c_int, [c_char_p, c_int]),
+    "e2h_seq_norm_conv": (c_int, [_A(NormConvArgs), _P]),
+    "e2h_seq_square_relu": (c_int, [c_int, _P, _P, c_int64, _P]),
+    "e2h_seq_softcap": (c_int, [c_int, _P, _P, c_int64, c_float, _P]),
+    "e2h_seq_gelu_gate_rows": (c_int, [c_int, _P, _P, _P, _P, c_int64, c_int64, c_int64, c_int64, c_int64, _P]),
+    "e2h_seq_window_attention": (c_int, [_A(WindowAttentionArgs), _P]),
+    "e2h_seq_hgrn2_scratch_bytes": (c_int64, [_A(Hgrn2Args)]),
+    "e2h_seq_hgrn2": (c_int, [_A(Hgrn2Args), _P]),
+    "e2h_seq_delta_scratch_bytes": (c_int64, [_A(DeltaArgs)]),
+    "e2h_seq_delta": (c_int, [_A(DeltaArgs), _P]),
+}
+
+SEQ_EXPORTED_SYMBOLS = tuple(_SEQ_SIGNATURES)
+
 _lib = None
+_seq_lib = None
 
 
 class E2HLibraryError(RuntimeError):
     pass
 
 
-def load(build_if_missing=False):
-    """Return the loaded library.  `build_if_missing` compiles it first when the .so is absent."""
-    global _lib
-    if _lib is not None:
-        return _lib
-    if not LIB_PATH.exists():
+def _open(path, build, build_if_missing, signatures, version_symbol):
+    if not path.exists():
         if not build_if_missing:
             raise E2HLibraryError(
-                f"{LIB_PATH} is missing: build it with `python -c 'import __graft_entry__ as g; g.build()'` "
-                "(there is no fallback path for the quantized-linear kernels)"
+                f"{path} is missing: build it with `python -c 'import __graft_entry__ as g; g.build()'` "
+                "(there is no fallback path for its kernels)"
             )
-        build_library()
-    lib = ctypes.CDLL(str(LIB_PATH))
-    for name, (restype, argtypes) in _SIGNATURES.items():
+        build()
+    lib = ctypes.CDLL(str(path))
+    for name, (restype, argtypes) in signatures.items():
         fn = getattr(lib, name)  # AttributeError if the symbol is not exported
         fn.restype = restype
         fn.argtypes = argtypes
-    if lib.e2h_abi_version() != 1:
-        raise E2HLibraryError(f"{LIB_PATH}: ABI version {lib.e2h_abi_version()} != 1; rebuild the library")
-    _lib = lib
+    version = getattr(lib, version_symbol)()
+    if version != 1:
+        raise E2HLibraryError(f"{path}: ABI version {version} != 1; rebuild the library")
     return lib
+
+
+def load(build_if_missing=False):
+    """Return the loaded libe2h_quant.so.  `build_if_missing` compiles it first when the .so is absent."""
+    global _lib
+    if _lib is None:
+        _lib = _open(LIB_PATH, build_library, build_if_missing, _SIGNATURES, "e2h_abi_version")
+    return _lib
+
+
+def load_seq(build_if_missing=False):
+    """Return the loaded libe2h_seq.so.  `build_if_missing` compiles it first when the .so is absent."""
+    global _seq_lib
+    if _seq_lib is None:
+        _seq_lib = _open(SEQ_LIB_PATH, build_seq_library, build_if_missing, _SEQ_SIGNATURES, "e2h_seq_abi_version")
+    return _seq_lib
+
+
+_STATUS_TEXT = {-1: "a required pointer is NULL", -2: "unsupported shape", -5: "pointer not aligned as required", -6: "HIP kernel launch failed",
+                -8: "unknown option or value out of range", -9: "scratch memory too small"}
+
+
+def check_seq(code, what):
+    if code != 0:
+        raise RuntimeError(f"{what}: {_STATUS_TEXT.get(code, 'unknown status')} (status {code})")
+
+
+def set_seq_option(name, value):
+    check_seq(load_seq().e2h_seq_set_option(name.encode(), int(value)), f"e2h_seq_set_option({name})")
 
 
 def status_string(code):

@@ -1,0 +1,609 @@
+// Windowed softmax attention with kept first tokens over a per-sequence key/value cache (e2h_seq_window_attention).
+//
+// A query at position i sees the keys first .. min(i, first + keep_first - 1) and max(first, i - window + 1) .. i.  The keys a
+// group of queries needs are walked as one list: the kept ones first, then the window, so both ends cost only what they hold.
+//
+// bfloat16: both products on v_mfma_f32_16x16x32_bf16 in transposed form.  S^T = K Q^T puts one query into each lane column
+// (lane 16 b + c holds keys 4 b .. 4 b + 3 of query c), so the softmax statistics of a query are in-lane sums plus two
+// shuffles, and the weights are, without moving, the B operand of O^T = V^T P^T over a key order that the V operand follows.
+// Weights enter that product as two bfloat16 terms (value and remainder), which keeps them at float32 accuracy against
+// bfloat16 values.
+// float32: one wave per query and head on the vector units.
+#include "e2h_seq_common.h"
+
+namespace e2h {
+namespace {
+
+constexpr float kLog2e = 1.4426950408889634f;
+constexpr float kMasked = -1e30f;
+
+struct KeyList {  // virtual index n -> key position
+  int first, kept, start, count;
+  __device__ int at(int n) const { return n < kept ? first + n : start + (n - kept); }
+};
+
+// keys of the queries at positions pa .. pb of one sequence
+__device__ __forceinline__ KeyList key_list(int pa, int pb, int first, int64_t window, int64_t keep_first) {
+  KeyList k;
+  k.first = first;
+  if (pb < first) {
+    k.kept = k.count = 0;
+    k.start = first;
+    return k;
+  }
+  const int64_t live = static_cast<int64_t>(pb) - first + 1;
+  k.kept = static_cast<int>(keep_first < live ? keep_first : live);
+  int64_t lo = window > 0 ? static_cast<int64_t>(pa) - window + 1 : 0;
+  if (lo < first + k.kept) lo = first + k.kept;
+  k.start = static_cast<int>(lo);
+  k.count = k.kept + (lo <= pb ? static_cast<int>(pb - lo) + 1 : 0);
+  return k;
+}
+
+__device__ __forceinline__ bool sees(int i, int j, int first, int64_t window, int64_t keep_first) {
+  return j <= i && j >= first && (window <= 0 || static_cast<int64_t>(i) - j < window || static_cast<int64_t>(j) - first < keep_first);
+}
+
+// eight consecutive bfloat16 values starting at p, of which `valid` exist; VEC: 16-byte accesses are aligned and valid is 8 or <= 0
+template <bool VEC>
+__device__ __forceinline__ u32x4_t load8(const bf16_t *p, int valid) {
+  u32x4_t r = {0u, 0u, 0u, 0u};
+  if (VEC) {
+    if (valid > 0) r = *reinterpret_cast<const u32x4_t *>(p);
+  } else {
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+      if (i < valid) r[i >> 1] |= static_cast<uint32_t>(p[i]) << (16 * (i & 1));
+  }
+  return r;
+}
+
+__device__ __forceinline__ u32x4_t add_bias8(u32x4_t r, const float *bias, int valid) {
+  if (!bias) return r;
+  u32x4_t o = {0u, 0u, 0u, 0u};
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    if (i < valid) {
+      const float v = __builtin_bit_cast(float, (i & 1) ? (r[i >> 1] & 0xFFFF0000u) : (r[i >> 1] << 16)) + bias[i];
+      o[i >> 1] |= static_cast<uint32_t>(f32_to_bf16_rne(v)) << (16 * (i & 1));
+    }
+  }
+  return o;
+}
+
+// ---- new keys and values into the caches ---------------------------------------------------------------------------------
+template <typename T>
+__global__ __launch_bounds__(256) void kv_append_kernel(const e2h_window_attention_args a) {
+  const int per_row = static_cast<int>(a.kv_heads * (a.dim + a.vdim));
+  const int64_t idx = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
+  if (idx >= a.batch * a.seqlen * per_row) return;
+  const int64_t row = idx / per_row;
+  int c = static_cast<int>(idx % per_row);
+  const int64_t b = row / a.seqlen, pos = a.input_pos[0] + row % a.seqlen;
+  if (pos < 0 || pos >= a.cache_len) return;
+  const T *src = static_cast<const T *>(a.proj) + row * a.ld;
+  const int kw = static_cast<int>(a.kv_heads * a.dim);
+  const bool is_k = c < kw;
+  if (!is_k) c -= kw;
+  const int d = static_cast<int>(is_k ? a.dim : a.vdim);
+  float v = to_f32(src[(is_k ? a.k_off : a.v_off) + c]);
+  const float *bias = is_k ? a.k_bias : a.v_bias;
+  if (bias) v += bias[c];
+  T *dst = static_cast<T *>(is_k ? a.k_cache : a.v_cache);
+  dst[((b * a.kv_heads + c / d) * a.cache_len + pos) * d + c % d] = from_f32<T>(v);
+}
+
+// ---- float32: one wave per (row, head) ------------------------------------------------------------------------------------
+constexpr int kMaxHeadDim = 256;
+
+template <typename T>
+__global__ __launch_bounds__(256) void attention_rows_kernel(const e2h_window_attention_args a) {
+  __shared__ float sh_q[4][kMaxHeadDim], sh_p[4][64];
+  __shared__ int sh_j[4][64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int64_t item = static_cast<int64_t>(blockIdx.x) * 4 + wave;
+  const bool active = item < a.batch * a.seqlen * a.heads;  // every wave reaches the end; idle ones hold no keys
+  const int64_t row = active ? item / a.heads : 0;
+  const int h = active ? static_cast<int>(item % a.heads) : 0;
+  const int64_t b = row / a.seqlen;
+  const int g = h / static_cast<int>(a.heads / a.kv_heads);
+  const int pos = static_cast<int>(a.input_pos[0] + row % a.seqlen);
+  const int first = a.first ? static_cast<int>(a.first[b]) : 0;
+  const int D = static_cast<int>(a.dim), DV = static_cast<int>(a.vdim);
+  const T *src = static_cast<const T *>(a.proj) + row * a.ld;
+  for (int d = lane; d < D; d += 64) sh_q[wave][d] = to_f32(src[a.q_off + static_cast<int64_t>(h) * D + d]) + (a.q_bias ? a.q_bias[h * D + d] : 0.f);
+  const int last = pos < a.cache_len ? pos : static_cast<int>(a.cache_len) - 1;
+  const KeyList kl = key_list(pos, last, first, a.window, a.keep_first);
+  const int count = active ? kl.count : 0;
+  const T *kc = static_cast<const T *>(a.k_cache) + (b * a.kv_heads + g) * a.cache_len * D;
+  const T *vc = static_cast<const T *>(a.v_cache) + (b * a.kv_heads + g) * a.cache_len * DV;
+  float m = kMasked, l = 0.f, acc[kMaxHeadDim / 64] = {0.f, 0.f, 0.f, 0.f};
+  for (int n0 = 0; n0 < count; n0 += 64) {
+    const int n = n0 + lane;
+    float s = kMasked;
+    int j = first;
+    if (n < count) {
+      j = kl.at(n);
+      const T *kr = kc + static_cast<size_t>(j) * D;
+      float dot = 0.f;
+      for (int d = 0; d < D; ++d) dot = __builtin_fmaf(sh_q[wave][d], to_f32(kr[d]), dot);
+      if (sees(pos, j, first, a.window, a.keep_first)) s = dot * a.scale;
+    }
+    float mx = s;
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off));
+    const float m_new = fmaxf(m, mx);
+    const float corr = expf(m - m_new);
+    const float p = s > 0.5f * kMasked ? expf(s - m_new) : 0.f;
+    m = m_new;
+    l = l * corr + wave_add(p);
+    sh_p[wave][lane] = p;
+    sh_j[wave][lane] = j;
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // wave-private LDS
+    const int live = count - n0 < 64 ? count - n0 : 64;
+#pragma unroll
+    for (int i = 0; i < kMaxHeadDim / 64; ++i) {
+      const int d = i * 64 + lane;
+      if (d < DV) {
+        float o = acc[i] * corr;
+        for (int n2 = 0; n2 < live; ++n2) o = __builtin_fmaf(sh_p[wave][n2], to_f32(vc[static_cast<size_t>(sh_j[wave][n2]) * DV + d]), o);
+        acc[i] = o;
+      }
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  }
+  if (!active) return;
+#pragma unroll
+  for (int i = 0; i < kMaxHeadDim / 64; ++i) {
+    const int d = i * 64 + lane;
+    if (d < DV) {
+      float o = l > 0.f ? acc[i] / l : 0.f;
+      if (a.g_off >= 0) o *= sigmoid_f32(to_f32(src[a.g_off + static_cast<int64_t>(h) * DV + d]));
+      static_cast<T *>(a.out)[row * a.ld_out + a.out_off + static_cast<int64_t>(h) * DV + d] = from_f32<T>(o * a.out_scale);
+    }
+  }
+}
+
+// weights of two key tiles (keys 4b .. 4b+3 and 16+4b .. 16+4b+3 of this lane's query) as value + remainder operands
+__device__ __forceinline__ void split_weights(const float (&p)[8], bf16x8_t &hi, bf16x8_t &lo) {
+  u32x4_t h, l;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const uint32_t a = __builtin_bit_cast(uint32_t, p[2 * i]) & 0xFFFF0000u, b = __builtin_bit_cast(uint32_t, p[2 * i + 1]) & 0xFFFF0000u;
+    h[i] = (a >> 16) | b;
+    l[i] = static_cast<uint32_t>(f32_to_bf16_rne(p[2 * i] - __builtin_bit_cast(float, a))) |
+           (static_cast<uint32_t>(f32_to_bf16_rne(p[2 * i + 1] - __builtin_bit_cast(float, b))) << 16);
+  }
+  hi = __builtin_bit_cast(bf16x8_t, h);
+  lo = __builtin_bit_cast(bf16x8_t, l);
+}
+
+// ---- bfloat16, many tokens: 4 waves x NQ x 16 queries of one head, key tiles of 64 shared through LDS ----------------------
+// KS: head dimension in steps of 32 (zero padded), VT: value dimension in tiles of 16.
+template <int KS, int VT, int NQ, bool VEC>
+__global__ __launch_bounds__(256) void attention_prefill_kernel(const e2h_window_attention_args a, int q_blocks) {
+  constexpr int kKeys = 64;
+  constexpr int kKRow = KS * 64 + 16;   // bytes per key row (padding spreads the rows over the banks)
+  constexpr int kVRow = kKeys * 2 + 8;  // bytes per row of V^T (one value column, 64 keys)
+  __shared__ __attribute__((aligned(16))) uint8_t sh_k[kKeys * kKRow];
+  __shared__ __attribute__((aligned(16))) uint8_t sh_v[VT * 16 * kVRow];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = lane & 15, b4 = lane >> 4;
+  const int D = static_cast<int>(a.dim), DV = static_cast<int>(a.vdim), seqlen = static_cast<int>(a.seqlen);
+  // consecutive workgroups share a key/value head: query heads of one group first, then query blocks
+  int w = blockIdx.x;
+  const int rep = static_cast<int>(a.heads / a.kv_heads);
+  const int r = w % rep;
+  w /= rep;
+  const int qb = q_blocks - 1 - w % q_blocks;  // blocks with the most keys start first
+  w /= q_blocks;
+  const int g = w % static_cast<int>(a.kv_heads);
+  const int bi = w / static_cast<int>(a.kv_heads);
+  const int h = g * rep + r;
+  const int pos0 = static_cast<int>(a.input_pos[0]);
+  const int first = a.first ? static_cast<int>(a.first[bi]) : 0;
+  const int t0 = qb * (64 * NQ);
+  const int t_last = t0 + 64 * NQ - 1 < seqlen - 1 ? t0 + 64 * NQ - 1 : seqlen - 1;
+  const int cache_last = static_cast<int>(a.cache_len) - 1;
+  const int pb = pos0 + t_last < cache_last ? pos0 + t_last : cache_last;
+  const KeyList kl = key_list(pos0 + t0, pb, first, a.window, a.keep_first);
+  const bf16_t *proj = static_cast<const bf16_t *>(a.proj);
+  const bf16_t *kc = static_cast<const bf16_t *>(a.k_cache) + (static_cast<size_t>(bi) * a.kv_heads + g) * a.cache_len * D;
+  const bf16_t *vc = static_cast<const bf16_t *>(a.v_cache) + (static_cast<size_t>(bi) * a.kv_heads + g) * a.cache_len * DV;
+  const size_t row0 = static_cast<size_t>(bi) * seqlen;
+
+  int tq[NQ];
+  bf16x8_t qf[NQ][KS];
+#pragma unroll
+  for (int n = 0; n < NQ; ++n) {
+    tq[n] = t0 + (wave * NQ + n) * 16 + c;
+    const int tc = tq[n] < seqlen ? tq[n] : seqlen - 1;
+#pragma unroll
+    for (int s = 0; s < KS; ++s) {
+      const int d = 32 * s + 8 * b4;
+      u32x4_t raw = load8<VEC>(proj + (row0 + tc) * a.ld + a.q_off + static_cast<int64_t>(h) * D + d, D - d);
+      if (a.q_bias) raw = add_bias8(raw, a.q_bias + static_cast<int64_t>(h) * D + d, D - d);
+      qf[n][s] = __builtin_bit_cast(bf16x8_t, raw);
+    }
+  }
+  f32x4_t oacc[NQ][VT];
+  float m_run[NQ], l_run[NQ];
+#pragma unroll
+  for (int n = 0; n < NQ; ++n) {
+    m_run[n] = kMasked;
+    l_run[n] = 0.f;
+#pragma unroll
+    for (int v = 0; v < VT; ++v) oacc[n][v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  }
+  const float sc = a.scale * kLog2e;
+
+  constexpr int kKPieces = kKeys * KS * 4, kVPieces = kKeys * VT * 2;  // 16-byte pieces per tile
+  constexpr int kKPer = kKPieces / 256, kVPer = (kVPieces + 255) / 256;
+  u32x4_t kr[kKPer], vr[kVPer];
+  auto fetch = [&](int n0) {
+#pragma unroll
+    for (int i = 0; i < kKPer; ++i) {
+      const int piece = i * 256 + threadIdx.x, n = n0 + piece / (KS * 4), d = (piece % (KS * 4)) * 8;
+      kr[i] = u32x4_t{0u, 0u, 0u, 0u};
+      if (n < kl.count) kr[i] = load8<VEC>(kc + static_cast<size_t>(kl.at(n)) * D + d, D - d);
+    }
+    // V pieces: consecutive threads take consecutive keys of one column group, so the transposed 2-byte LDS writes of a wave
+    // fill whole rows
+#pragma unroll
+    for (int i = 0; i < kVPer; ++i) {
+      const int piece = i * 256 + threadIdx.x, n = n0 + piece % kKeys, d = (piece / kKeys) * 8;
+      vr[i] = u32x4_t{0u, 0u, 0u, 0u};
+      if (piece < kVPieces && n < kl.count) vr[i] = load8<VEC>(vc + static_cast<size_t>(kl.at(n)) * DV + d, DV - d);
+    }
+  };
+  if (kl.count > 0) fetch(0);
+  for (int n0 = 0; n0 < kl.count; n0 += kKeys) {
+    __syncthreads();  // the previous tile has been read
+#pragma unroll
+    for (int i = 0; i < kKPer; ++i) {
+      const int piece = i * 256 + threadIdx.x;
+      *reinterpret_cast<u32x4_t *>(sh_k + (piece / (KS * 4)) * kKRow + (piece % (KS * 4)) * 16) = kr[i];
+    }
+#pragma unroll
+    for (int i = 0; i < kVPer; ++i) {
+      const int piece = i * 256 + threadIdx.x, n = piece % kKeys, d = (piece / kKeys) * 8;
+      if (piece < kVPieces) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          *reinterpret_cast<uint16_t *>(sh_v + (d + e) * kVRow + n * 2) = static_cast<uint16_t>(vr[i][e >> 1] >> (16 * (e & 1)));
+      }
+    }
+    __syncthreads();
+    if (n0 + kKeys < kl.count) fetch(n0 + kKeys);
+
+    f32x4_t st[NQ][4];
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt) {
+#pragma unroll
+      for (int n = 0; n < NQ; ++n) st[n][kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < KS; ++s) {
+        const bf16x8_t kf = *reinterpret_cast<const bf16x8_t *>(sh_k + (16 * kt + c) * kKRow + s * 64 + b4 * 16);
+#pragma unroll
+        for (int n = 0; n < NQ; ++n) st[n][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[n][s], st[n][kt], 0, 0, 0);
+      }
+    }
+    // positions of this lane's keys
+    int j[4][4];
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int n = n0 + 16 * kt + 4 * b4 + e;
+        j[kt][e] = n < kl.count ? kl.at(n) : INT32_MAX;
+      }
+#pragma unroll
+    for (int n = 0; n < NQ; ++n) {
+      const int pq = pos0 + tq[n];
+      float mx = kMasked;
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float v = sees(pq, j[kt][e], first, a.window, a.keep_first) ? st[n][kt][e] * sc : kMasked;
+          st[n][kt][e] = v;
+          mx = fmaxf(mx, v);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16));
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      const float m_new = fmaxf(m_run[n], mx);
+      const float corr = __builtin_amdgcn_exp2f(m_run[n] - m_new);
+      m_run[n] = m_new;
+      float ls = 0.f;
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float p = st[n][kt][e] > 0.5f * kMasked ? __builtin_amdgcn_exp2f(st[n][kt][e] - m_new) : 0.f;
+          st[n][kt][e] = p;
+          ls += p;
+        }
+      l_run[n] = l_run[n] * corr + ls;
+#pragma unroll
+      for (int v = 0; v < VT; ++v)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) oacc[n][v][e] *= corr;
+    }
+#pragma unroll
+    for (int half = 0; half < 2; ++half) {
+      bf16x8_t hi[NQ], lo[NQ];
+#pragma unroll
+      for (int n = 0; n < NQ; ++n) {
+        float p[8];
+#pragma unroll
+        for (int e = 0; e < 8; ++e) p[e] = st[n][2 * half + (e >> 2)][e & 3];
+        split_weights(p, hi[n], lo[n]);
+      }
+#pragma unroll
+      for (int v = 0; v < VT; ++v) {
+        const uint8_t *vp = sh_v + (16 * v + c) * kVRow + half * 64 + b4 * 8;
+        const u32x2_t v0 = *reinterpret_cast<const u32x2_t *>(vp), v1 = *reinterpret_cast<const u32x2_t *>(vp + 32);
+        const bf16x8_t vf = __builtin_bit_cast(bf16x8_t, u32x4_t{v0[0], v0[1], v1[0], v1[1]});
+#pragma unroll
+        for (int n = 0; n < NQ; ++n) {
+          oacc[n][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[n], oacc[n][v], 0, 0, 0);
+          oacc[n][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[n], oacc[n][v], 0, 0, 0);
+        }
+      }
+    }
+  }
+  // lane (b, c): value columns 16 v + 4 b .. + 3 of query c
+#pragma unroll
+  for (int n = 0; n < NQ; ++n) {
+    float l = l_run[n];
+    l += __shfl_xor(l, 16);
+    l += __shfl_xor(l, 32);
+    const float inv = l > 0.f ? a.out_scale / l : 0.f;
+    if (tq[n] >= seqlen) continue;
+    const size_t row = row0 + tq[n];
+#pragma unroll
+    for (int v = 0; v < VT; ++v)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int d = 16 * v + 4 * b4 + e;
+        if (d < DV) {
+          float o = oacc[n][v][e] * inv;
+          if (a.g_off >= 0) o *= sigmoid_f32(to_f32(proj[row * a.ld + a.g_off + static_cast<int64_t>(h) * DV + d]));
+          static_cast<bf16_t *>(a.out)[row * a.ld_out + a.out_off + static_cast<int64_t>(h) * DV + d] = f32_to_bf16_rne(o);
+        }
+      }
+  }
+}
+
+// ---- bfloat16, one token per sequence: one workgroup per (sequence, key/value head) ------------------------------------------
+// The lane columns are the query heads of the group (up to 16); the waves take key tiles of 32 round robin and are combined at
+// the end.  The workgroup appends its own new key and value row first.
+template <int KS, int VT, int NW, bool VEC>
+__global__ __launch_bounds__(64 * NW) void attention_step_kernel(const e2h_window_attention_args a) {
+  constexpr int kVRow = VT * 32 + 8;  // bytes per value row in LDS
+  constexpr int kWaveLds = 32 * kVRow;
+  constexpr int kEndLds = NW * (16 * VT * 16 + 32) * 4;
+  constexpr int kLds = NW * kWaveLds > kEndLds ? NW * kWaveLds : kEndLds;
+  __shared__ __attribute__((aligned(16))) uint8_t lds[kLds];
+  const int lane = threadIdx.x & 63, c = lane & 15, b4 = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int D = static_cast<int>(a.dim), DV = static_cast<int>(a.vdim);
+  const int bi = blockIdx.x / static_cast<int>(a.kv_heads), g = blockIdx.x % static_cast<int>(a.kv_heads);
+  const int rep = static_cast<int>(a.heads / a.kv_heads);
+  const int pos = static_cast<int>(a.input_pos[0]);
+  const int first = a.first ? static_cast<int>(a.first[bi]) : 0;
+  const bf16_t *proj = static_cast<const bf16_t *>(a.proj) + static_cast<size_t>(bi) * a.ld;
+  bf16_t *kc = static_cast<bf16_t *>(a.k_cache) + (static_cast<size_t>(bi) * a.kv_heads + g) * a.cache_len * D;
+  bf16_t *vc = static_cast<bf16_t *>(a.v_cache) + (static_cast<size_t>(bi) * a.kv_heads + g) * a.cache_len * DV;
+  if (pos >= 0 && pos < a.cache_len) {
+    for (int i = threadIdx.x; i < D + DV; i += 64 * NW) {
+      const bool is_k = i < D;
+      const int d = is_k ? i : i - D;
+      const int col = g * (is_k ? D : DV) + d;
+      float v = to_f32(proj[(is_k ? a.k_off : a.v_off) + col]);
+      const float *bias = is_k ? a.k_bias : a.v_bias;
+      if (bias) v += bias[col];
+      (is_k ? kc + static_cast<size_t>(pos) * D : vc + static_cast<size_t>(pos) * DV)[d] = f32_to_bf16_rne(v);
+    }
+  }
+  __threadfence_block();
+  __syncthreads();  // the new row is visible to the workgroup
+
+  const int last = pos < a.cache_len ? pos : static_cast<int>(a.cache_len) - 1;
+  const KeyList kl = key_list(pos, last, first, a.window, a.keep_first);
+  bf16x8_t qf[KS];
+#pragma unroll
+  for (int s = 0; s < KS; ++s) {
+    const int d = 32 * s + 8 * b4;
+    u32x4_t raw = {0u, 0u, 0u, 0u};
+    if (c < rep) {
+      raw = load8<VEC>(proj + a.q_off + static_cast<int64_t>(g * rep + c) * D + d, D - d);
+      if (a.q_bias) raw = add_bias8(raw, a.q_bias + static_cast<int64_t>(g * rep + c) * D + d, D - d);
+    }
+    qf[s] = __builtin_bit_cast(bf16x8_t, raw);
+  }
+  f32x4_t oacc[VT];
+  float m_run = kMasked, l_run = 0.f;
+#pragma unroll
+  for (int v = 0; v < VT; ++v) oacc[v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const float sc = a.scale * kLog2e;
+  uint8_t *v_lds = lds + wave * kWaveLds;
+  constexpr int kVPer = (32 * VT * 2 + 63) / 64;
+
+  for (int n0 = wave * 32; n0 < kl.count; n0 += NW * 32) {
+    u32x4_t kf[2][KS], vr[kVPer];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+      const int n = n0 + 16 * t + c;
+      const int j = kl.at(n < kl.count ? n : kl.count - 1);
+#pragma unroll
+      for (int s = 0; s < KS; ++s) {
+        const int d = 32 * s + 8 * b4;
+        kf[t][s] = load8<VEC>(kc + static_cast<size_t>(j) * D + d, D - d);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < kVPer; ++i) {
+      const int piece = i * 64 + lane, n = n0 + piece / (VT * 2), d = (piece % (VT * 2)) * 8;
+      const int j = kl.at(n < kl.count ? n : kl.count - 1);
+      vr[i] = load8<VEC>(vc + static_cast<size_t>(j) * DV + d, DV - d);
+    }
+    f32x4_t st[2];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+      st[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < KS; ++s)
+        st[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kf[t][s]), qf[s], st[t], 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < kVPer; ++i) {
+      const int piece = i * 64 + lane;
+      uint8_t *dst = v_lds + (piece / (VT * 2)) * kVRow + (piece % (VT * 2)) * 16;
+      *reinterpret_cast<u32x2_t *>(dst) = u32x2_t{vr[i][0], vr[i][1]};
+      *reinterpret_cast<u32x2_t *>(dst + 8) = u32x2_t{vr[i][2], vr[i][3]};
+    }
+    float p[8], mx = kMasked;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const int n = n0 + 16 * (e >> 2) + 4 * b4 + (e & 3);
+      p[e] = n < kl.count ? st[e >> 2][e & 3] * sc : kMasked;  // every listed key is visible to the one query position
+      mx = fmaxf(mx, p[e]);
+    }
+    mx = fmaxf(mx, __shfl_xor(mx, 16));
+    mx = fmaxf(mx, __shfl_xor(mx, 32));
+    const float m_new = fmaxf(m_run, mx);
+    const float corr = __builtin_amdgcn_exp2f(m_run - m_new);
+    m_run = m_new;
+    float ls = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      p[e] = p[e] > 0.5f * kMasked ? __builtin_amdgcn_exp2f(p[e] - m_new) : 0.f;
+      ls += p[e];
+    }
+    l_run = l_run * corr + ls;
+    bf16x8_t hi, lo;
+    split_weights(p, hi, lo);
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // wave-private tile: the wave's own writes have landed
+#pragma unroll
+    for (int v = 0; v < VT; ++v) {
+      uint32_t vw[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int k0 = 16 * (i >> 1) + 4 * b4 + 2 * (i & 1);
+        const uint32_t x0 = *reinterpret_cast<const uint16_t *>(v_lds + k0 * kVRow + (16 * v + c) * 2);
+        const uint32_t x1 = *reinterpret_cast<const uint16_t *>(v_lds + (k0 + 1) * kVRow + (16 * v + c) * 2);
+        vw[i] = x0 | (x1 << 16);
+      }
+      const bf16x8_t vf = __builtin_bit_cast(bf16x8_t, u32x4_t{vw[0], vw[1], vw[2], vw[3]});
+#pragma unroll
+      for (int e = 0; e < 4; ++e) oacc[v][e] *= corr;
+      oacc[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi, oacc[v], 0, 0, 0);
+      oacc[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo, oacc[v], 0, 0, 0);
+    }
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // reads done before the next tile overwrites the wave's LDS
+  }
+  __syncthreads();  // every wave is done with its tiles: the LDS is reused
+  float *const sh_o = reinterpret_cast<float *>(lds);  // [NW][16 heads][VT * 16]
+  float *const sh_m = sh_o + NW * 16 * VT * 16;        // [NW][16]
+  float *const sh_l = sh_m + NW * 16;                  // [NW][16]
+  l_run += __shfl_xor(l_run, 16);
+  l_run += __shfl_xor(l_run, 32);
+#pragma unroll
+  for (int v = 0; v < VT; ++v) *reinterpret_cast<f32x4_t *>(sh_o + (wave * 16 + c) * VT * 16 + 16 * v + 4 * b4) = oacc[v];
+  if (b4 == 0) {
+    sh_m[wave * 16 + c] = m_run;
+    sh_l[wave * 16 + c] = l_run;
+  }
+  __syncthreads();
+  for (int e = threadIdx.x; e < rep * DV; e += 64 * NW) {
+    const int r = e / DV, d = e % DV;
+    float m = sh_m[r];
+#pragma unroll
+    for (int w = 1; w < NW; ++w) m = fmaxf(m, sh_m[w * 16 + r]);
+    float l = 0.f, o = 0.f;
+#pragma unroll
+    for (int w = 0; w < NW; ++w) {
+      const float cw = __builtin_amdgcn_exp2f(sh_m[w * 16 + r] - m);
+      l += sh_l[w * 16 + r] * cw;
+      o += sh_o[(w * 16 + r) * VT * 16 + d] * cw;
+    }
+    const int col = (g * rep + r) * DV + d;
+    o = l > 0.f ? o / l * a.out_scale : 0.f;
+    if (a.g_off >= 0) o *= sigmoid_f32(to_f32(proj[a.g_off + col]));
+    static_cast<bf16_t *>(a.out)[static_cast<size_t>(bi) * a.ld_out + a.out_off + col] = f32_to_bf16_rne(o);
+  }
+}
+
+void launch_append(const e2h_window_attention_args &a, hipStream_t s) {
+  const int64_t n = a.batch * a.seqlen * a.kv_heads * (a.dim + a.vdim);
+  const dim3 grid(static_cast<unsigned>((n + 255) / 256)), block(256);
+  if (a.dtype == E2H_SEQ_BF16) hipLaunchKernelGGL(kv_append_kernel<bf16_t>, grid, block, 0, s, a);
+  else hipLaunchKernelGGL(kv_append_kernel<float>, grid, block, 0, s, a);
+}
+
+template <int KS, int VT, bool VEC>
+void launch_mfma(const e2h_window_attention_args &a, hipStream_t s) {
+  if (a.seqlen == 1) {
+    const dim3 grid(static_cast<unsigned>(a.batch * a.kv_heads));
+    // one wave walks 32 keys at a time; more waves pay once there are enough keys to share
+    const int64_t span = a.window > 0 && a.window + a.keep_first < a.cache_len ? a.window + a.keep_first : a.cache_len;
+    const int nw = seq_options().attention_decode_waves ? seq_options().attention_decode_waves : (span > 256 ? 8 : 4);
+    if (nw == 8 && KS <= 4) hipLaunchKernelGGL((attention_step_kernel<KS, VT, (KS <= 4 ? 8 : 4), VEC>), grid, dim3(KS <= 4 ? 512 : 256), 0, s, a);
+    else hipLaunchKernelGGL((attention_step_kernel<KS, VT, 4, VEC>), grid, dim3(256), 0, s, a);
+    return;
+  }
+  launch_append(a, s);
+  const int64_t groups = a.batch * a.heads;
+  int nq = seq_options().attention_query_tiles;
+  if (!nq) nq = groups * ((a.seqlen + 127) / 128) >= 512 ? 2 : 1;
+  if (KS > 4) nq = 1;  // the wide heads' accumulators fill the registers with one tile of queries
+  const int q_blocks = static_cast<int>((a.seqlen + 64 * nq - 1) / (64 * nq));
+  const dim3 grid(static_cast<unsigned>(groups * q_blocks)), block(256);
+  if (nq == 2) hipLaunchKernelGGL((attention_prefill_kernel<KS, VT, (KS <= 4 ? 2 : 1), VEC>), grid, block, 0, s, a, q_blocks);
+  else hipLaunchKernelGGL((attention_prefill_kernel<KS, VT, 1, VEC>), grid, block, 0, s, a, q_blocks);
+}
+
+template <bool VEC>
+void launch_mfma_by_size(const e2h_window_attention_args &a, hipStream_t s) {
+  const int64_t d = a.dim > a.vdim ? a.dim : a.vdim;
+  if (d <= 32) launch_mfma<1, 2, VEC>(a, s);
+  else if (d <= 64) launch_mfma<2, 4, VEC>(a, s);
+  else if (d <= 128) launch_mfma<4, 8, VEC>(a, s);
+  else launch_mfma<8, 16, VEC>(a, s);
+}
+
+void launch_rows(const e2h_window_attention_args &a, hipStream_t s) {
+  launch_append(a, s);
+  const dim3 grid(static_cast<unsigned>((a.batch * a.seqlen * a.heads + 3) / 4)), block(256);
+  if (a.dtype == E2H_SEQ_BF16) hipLaunchKernelGGL(attention_rows_kernel<bf16_t>, grid, block, 0, s, a);
+  else hipLaunchKernelGGL(attention_rows_kernel<float>, grid, block, 0, s, a);
+}
+
+}  // namespace
+}  // namespace e2h
+
+using namespace e2h;
+
+extern "C" int e2h_seq_window_attention(const e2h_window_attention_args *a, void *stream) {
+  if (!a || !a->proj || !a->k_cache || !a->v_cache || !a->input_pos || !a->out) return E2H_ERR_NULL_POINTER;
+  if (a->dtype != E2H_SEQ_BF16 && a->dtype != E2H_SEQ_F32) return E2H_ERR_BAD_SHAPE;
+  if (a->batch < 1 || a->seqlen < 1 || a->heads < 1 || a->kv_heads < 1 || a->heads % a->kv_heads != 0 || a->dim < 1 || a->vdim < 1 ||
+      a->dim > kMaxHeadDim || a->vdim > kMaxHeadDim || a->cache_len < 1 || a->cache_len > INT32_MAX / 2 || a->seqlen > INT32_MAX / 4)
+    return E2H_ERR_BAD_SHAPE;
+  if (a->window < 0 || a->keep_first < 0 || a->q_off < 0 || a->k_off < 0 || a->v_off < 0 || a->out_off < 0) return E2H_ERR_BAD_SHAPE;
+  if (a->q_off + a->heads * a->dim > a->ld || a->k_off + a->kv_heads * a->dim > a->ld || a->v_off + a->kv_heads * a->vdim > a->ld ||
+      (a->g_off >= 0 && a->g_off + a->heads * a->vdim > a->ld) || a->out_off + a->heads * a->vdim > a->ld_out)
+    return E2H_ERR_BAD_SHAPE;
+  if (a->batch * a->seqlen * a->heads > INT32_MAX || a->batch * a->seqlen * a->kv_heads * (a->dim + a->vdim) / 256 > INT32_MAX - 1)
+    return E2H_ERR_BAD_SHAPE;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (a->dtype == E2H_SEQ_F32 || a->heads / a->kv_heads > 16) {
+    launch_rows(*a, s);
+    return launch_status();
+  }
+  const bool vec = a->dim % 8 == 0 && a->vdim % 8 == 0 && a->ld % 8 == 0 && a->q_off % 8 == 0 && aligned16(a->proj) && aligned16(a->k_cache) &&
+                   aligned16(a->v_cache);
+  if (vec) launch_mfma_by_size<true>(*a, s);
+  else launch_mfma_by_size<false>(*a, s);
+  return launch_status();
+}

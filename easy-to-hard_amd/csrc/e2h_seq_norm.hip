@@ -1,0 +1,348 @@
+// Row kernels of the stateful decoder layers: residual add of a normalised sublayer output, the next sublayer's norm and
+// its input convolution over time in one pass over the float32 residual stream, and the elementwise steps.
+#include <string.h>
+
+#include "e2h_seq_common.h"
+
+namespace e2h {
+
+SeqOptions &seq_options() {
+  static SeqOptions o = {};
+  return o;
+}
+
+namespace {
+
+// One workgroup per run of `run` consecutive tokens of one sequence.  A thread owns NP pieces of four channels, so the
+// convolution's previous inputs stay in its registers from token to token; the taps - 1 tokens ahead of the run are
+// normalised again by the workgroup (inside the call) or come from the ring of kept inputs (before the call).
+// TAPS is the compiled depth of the convolution (0 = none); shallower ones pad their weights with zeros in front.
+template <typename T, int BLOCK, int NP, int TAPS>
+__global__ __launch_bounds__(BLOCK) void norm_conv_kernel(const e2h_norm_conv_args a, int runs, int run) {
+  constexpr int kWaves = BLOCK / 64;
+  constexpr int RING = TAPS > 1 ? TAPS - 1 : 1;
+  const int W = static_cast<int>(a.width), seqlen = static_cast<int>(a.seqlen), taps = a.taps;
+  const int b = blockIdx.x / runs, t_begin = (blockIdx.x % runs) * run;
+  const int t_end = t_begin + run < seqlen ? t_begin + run : seqlen;
+  const int64_t pos0 = TAPS ? a.input_pos[0] : 0;
+  const int64_t first = TAPS && a.first ? a.first[b] : 0;
+  const size_t row0 = static_cast<size_t>(b) * seqlen;
+  __shared__ float part[2][kWaves];
+  int phase = 0;
+
+  auto block_sum = [&](float v) {
+    v = wave_add(v);
+    if ((threadIdx.x & 63) == 0) part[phase][threadIdx.x >> 6] = v;
+    __syncthreads();
+    float s = 0.f;
+#pragma unroll
+    for (int w = 0; w < kWaves; ++w) s += part[phase][w];
+    phase ^= 1;  // the next sum writes the other half, so one barrier per sum is enough
+    return s;
+  };
+
+  f32x4_t wconv[TAPS > 0 ? TAPS : 1][NP], ring[RING][NP];
+  if (TAPS) {
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+      const int i = (p * BLOCK + threadIdx.x) * 4;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) {
+        wconv[j][p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        const int jj = j - (TAPS - taps);
+        if (i < W && jj >= 0) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) wconv[j][p][e] = a.conv[static_cast<size_t>(i + e) * taps + jj];
+        }
+      }
+#pragma unroll
+      for (int j = 0; j < RING; ++j) ring[j][p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
+  }
+
+  // h of token t (the convolution's input); emit: also store the updated residual row
+  auto norm_row = [&](int t, bool emit, f32x4_t (&h)[NP]) {
+    const size_t base = (row0 + t) * W;
+    f32x4_t d[NP];
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+      const int i = (p * BLOCK + threadIdx.x) * 4;
+      h[p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      d[p] = h[p];
+      if (i < W) {
+        h[p] = load4(a.x + base + i);
+        if (a.delta) d[p] = load4(static_cast<const T *>(a.delta) + base + i);
+      }
+    }
+    if (a.delta) {
+      float ss = 0.f;
+#pragma unroll
+      for (int p = 0; p < NP; ++p)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = __builtin_fmaf(d[p][e], d[p][e], ss);
+      const float inv = 1.0f / sqrtf(block_sum(ss) / static_cast<float>(W) + a.eps);
+#pragma unroll
+      for (int p = 0; p < NP; ++p) {
+        const int i = (p * BLOCK + threadIdx.x) * 4;
+        if (i < W) {
+          const f32x4_t w = load4(a.delta_weight + i);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) h[p][e] += d[p][e] * inv * (a.delta_offset + w[e]);
+          if (emit && a.x_out) store4(a.x_out + base + i, h[p]);
+        }
+      }
+    }
+    if (a.norm_weight) {
+      float ss = 0.f;
+#pragma unroll
+      for (int p = 0; p < NP; ++p)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss = __builtin_fmaf(h[p][e], h[p][e], ss);
+      const float inv = 1.0f / sqrtf(block_sum(ss) / static_cast<float>(W) + a.eps);
+#pragma unroll
+      for (int p = 0; p < NP; ++p) {
+        const int i = (p * BLOCK + threadIdx.x) * 4;
+        if (i < W) {
+          const f32x4_t w = load4(a.norm_weight + i);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) h[p][e] = h[p][e] * inv * (a.norm_offset + w[e]);
+        }
+      }
+    }
+    if (TAPS && pos0 + t < first) {  // padding: the convolution must not see it
+#pragma unroll
+      for (int p = 0; p < NP; ++p) h[p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
+  };
+  auto push = [&](const f32x4_t (&h)[NP]) {
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+#pragma unroll
+      for (int j = 0; j + 1 < RING; ++j) ring[j][p] = ring[j + 1][p];
+      ring[RING - 1][p] = h[p];
+    }
+  };
+
+  if (TAPS > 1) {
+    for (int s = t_begin - (taps - 1); s < t_begin; ++s) {
+      f32x4_t h[NP];
+      if (s >= 0) {
+        norm_row(s, false, h);
+      } else {
+        const int64_t pos = pos0 + s;
+        const bool live = pos >= first && pos >= 0;
+        const float *src = a.tail_in + (static_cast<size_t>(b) * taps + (live ? pos % taps : 0)) * W;
+#pragma unroll
+        for (int p = 0; p < NP; ++p) {
+          const int i = (p * BLOCK + threadIdx.x) * 4;
+          h[p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+          if (live && i < W) h[p] = load4(src + i);
+        }
+      }
+      push(h);
+    }
+  }
+  for (int t = t_begin; t < t_end; ++t) {
+    f32x4_t h[NP];
+    norm_row(t, true, h);
+    const size_t base = (row0 + t) * W;
+#pragma unroll
+    for (int p = 0; p < NP; ++p) {
+      const int i = (p * BLOCK + threadIdx.x) * 4;
+      f32x4_t y = h[p];
+      if (TAPS) {
+        f32x4_t c = h[p] * wconv[TAPS > 0 ? TAPS - 1 : 0][p];
+        if (TAPS > 1) {
+#pragma unroll
+          for (int j = 0; j < RING; ++j)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) c[e] = __builtin_fmaf(ring[j][p][e], wconv[j][p][e], c[e]);
+        }
+        y += c;
+      }
+      if (a.out && i < W) store4(static_cast<T *>(a.out) + base + i, y);
+    }
+    if (TAPS > 1) {
+      push(h);
+      if (seqlen == 1) {
+        float *dst = a.tail_out + (static_cast<size_t>(b) * taps + (pos0 > 0 ? pos0 % taps : 0)) * W;
+#pragma unroll
+        for (int p = 0; p < NP; ++p) {
+          const int i = (p * BLOCK + threadIdx.x) * 4;
+          if (i < W) store4(dst + i, h[p]);
+        }
+      }
+    }
+  }
+  if (TAPS > 1 && seqlen > 1 && t_end == seqlen) {  // the last inputs of the call, oldest first in the ring registers
+#pragma unroll
+    for (int j = 0; j < RING; ++j) {
+      const int64_t pos = pos0 + seqlen - RING + j;
+      if (j >= RING - (taps - 1) && pos >= 0) {
+        float *dst = a.tail_out + (static_cast<size_t>(b) * taps + pos % taps) * W;
+#pragma unroll
+        for (int p = 0; p < NP; ++p) {
+          const int i = (p * BLOCK + threadIdx.x) * 4;
+          if (i < W) store4(dst + i, ring[j][p]);
+        }
+      }
+    }
+  }
+}
+
+template <typename T, int BLOCK, int NP>
+void launch_norm_conv_taps(const e2h_norm_conv_args &a, int runs, int run, hipStream_t s) {
+  const dim3 grid(static_cast<unsigned>(a.batch * runs)), block(BLOCK);
+  if (!a.conv)
+    hipLaunchKernelGGL((norm_conv_kernel<T, BLOCK, NP, 0>), grid, block, 0, s, a, runs, run);
+  else if (a.taps <= 4)
+    hipLaunchKernelGGL((norm_conv_kernel<T, BLOCK, NP, 4>), grid, block, 0, s, a, runs, run);
+  else
+    hipLaunchKernelGGL((norm_conv_kernel<T, BLOCK, NP, 8>), grid, block, 0, s, a, runs, run);
+}
+
+template <typename T>
+void launch_norm_conv(const e2h_norm_conv_args &a, int runs, int run, hipStream_t s) {
+  if (a.width <= 1024) launch_norm_conv_taps<T, 256, 1>(a, runs, run, s);
+  else if (a.width <= 2048) launch_norm_conv_taps<T, 256, 2>(a, runs, run, s);
+  else if (a.width <= 4096) launch_norm_conv_taps<T, 512, 2>(a, runs, run, s);
+  else if (a.width <= 8192) launch_norm_conv_taps<T, 1024, 2>(a, runs, run, s);
+  else launch_norm_conv_taps<T, 1024, 4>(a, runs, run, s);
+}
+
+// ---- elementwise -----------------------------------------------------------------------------------------------------
+enum { kSquareRelu = 0, kSoftcap = 1 };
+
+template <int OP>
+__device__ __forceinline__ float elementwise_op(float v, float cap) {
+  if (OP == kSquareRelu) {
+    const float r = fmaxf(v, 0.f);
+    return r * r;
+  }
+  return cap * tanhf(v / cap);
+}
+
+template <typename T, int OP>
+__global__ __launch_bounds__(256) void elementwise_kernel(const T *x, T *y, int64_t n, float cap) {
+  const int64_t i = (static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x) * 4;
+  if (i + 4 <= n) {
+    f32x4_t v = load4(x + i);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = elementwise_op<OP>(v[e], cap);
+    store4(y + i, v);
+  } else {
+    for (int64_t j = i; j < n; ++j) y[j] = from_f32<T>(elementwise_op<OP>(to_f32(x[j]), cap));
+  }
+}
+
+template <int OP>
+int launch_elementwise(int dtype, const void *x, void *y, int64_t n, float cap, void *stream) {
+  if (!x || !y) return E2H_ERR_NULL_POINTER;
+  const int64_t blocks = (n + 1023) / 1024;
+  if (n < 1 || blocks > INT32_MAX || (dtype != E2H_SEQ_BF16 && dtype != E2H_SEQ_F32)) return E2H_ERR_BAD_SHAPE;
+  if (!aligned16(x) || !aligned16(y)) return E2H_ERR_MISALIGNED;
+  const dim3 grid(static_cast<unsigned>(blocks)), block(256);
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (dtype == E2H_SEQ_BF16)
+    hipLaunchKernelGGL((elementwise_kernel<bf16_t, OP>), grid, block, 0, s, static_cast<const bf16_t *>(x), static_cast<bf16_t *>(y), n, cap);
+  else
+    hipLaunchKernelGGL((elementwise_kernel<float, OP>), grid, block, 0, s, static_cast<const float *>(x), static_cast<float *>(y), n, cap);
+  return launch_status();
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void gelu_gate_rows_kernel(const T *__restrict__ gate, const T *__restrict__ table, const int64_t *__restrict__ tokens,
+                                                             T *__restrict__ y, int64_t n, int dim, int64_t ld, int64_t column, int64_t table_rows) {
+  const int64_t i = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
+  if (i >= n) return;
+  const int64_t r = i / dim, c = i % dim;
+  const int64_t tok = tokens[r];
+  const float z = to_f32(gate[i]);
+  const float e = tok >= 0 && tok < table_rows ? to_f32(table[tok * ld + column + c]) : 0.f;
+  const float g = 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+  y[i] = from_f32<T>(g * e);
+}
+
+}  // namespace
+}  // namespace e2h
+
+using namespace e2h;
+
+extern "C" int e2h_seq_abi_version(void) { return E2H_SEQ_ABI_VERSION; }
+
+extern "C" int e2h_seq_set_option(const char *name, int value) {
+  if (!name) return E2H_ERR_NULL_POINTER;
+  SeqOptions &o = seq_options();
+  if (!strcmp(name, "recurrence_form")) {
+    if (value < 0 || value > 2) return E2H_ERR_BAD_OPTION;
+    o.recurrence_form = value;
+  } else if (!strcmp(name, "recurrence_chunk")) {
+    if (value < 0 || value % 64 != 0) return E2H_ERR_BAD_OPTION;
+    o.recurrence_chunk = value;
+  } else if (!strcmp(name, "norm_run")) {
+    if (value < 0 || value > 256) return E2H_ERR_BAD_OPTION;
+    o.norm_run = value;
+  } else if (!strcmp(name, "attention_decode_waves")) {
+    if (value != 0 && value != 4 && value != 8) return E2H_ERR_BAD_OPTION;
+    o.attention_decode_waves = value;
+  } else if (!strcmp(name, "attention_query_tiles")) {
+    if (value < 0 || value > 2) return E2H_ERR_BAD_OPTION;
+    o.attention_query_tiles = value;
+  } else {
+    return E2H_ERR_BAD_OPTION;
+  }
+  return E2H_OK;
+}
+
+extern "C" int e2h_seq_norm_conv(const e2h_norm_conv_args *a, void *stream) {
+  if (!a || !a->x || (a->delta && !a->delta_weight)) return E2H_ERR_NULL_POINTER;
+  if (!a->out && !a->x_out) return E2H_ERR_NULL_POINTER;
+  if (a->conv && (!a->input_pos || (a->taps > 1 && (!a->tail_in || !a->tail_out)))) return E2H_ERR_NULL_POINTER;
+  if (a->batch < 1 || a->seqlen < 1 || a->width < 4 || a->width % 4 != 0 || a->width > 16384 || a->seqlen > INT32_MAX / 2)
+    return E2H_ERR_BAD_SHAPE;
+  if (a->dtype != E2H_SEQ_BF16 && a->dtype != E2H_SEQ_F32) return E2H_ERR_BAD_SHAPE;
+  if (a->conv && (a->taps < 1 || a->taps > 8)) return E2H_ERR_BAD_SHAPE;
+  if (a->seqlen > 1 && a->conv && ((a->taps > 1 && a->tail_in == a->tail_out) || (a->delta && a->x == a->x_out && a->taps > 1))) return E2H_ERR_BAD_SHAPE;
+  if (!aligned16(a->x) || !aligned16(a->delta) || !aligned16(a->delta_weight) || !aligned16(a->x_out) || !aligned16(a->norm_weight) ||
+      !aligned16(a->tail_in) || !aligned16(a->tail_out) || !aligned16(a->out))
+    return E2H_ERR_MISALIGNED;
+  // enough workgroups to fill the chip first, then longer runs so that fewer tokens are normalised twice
+  int run = seq_options().norm_run;
+  if (!run) {
+    run = static_cast<int>(a->batch * a->seqlen / 1024);
+    run = run < 1 ? 1 : run > 16 ? 16 : run;
+  }
+  const int64_t runs = (a->seqlen + run - 1) / run;
+  if (a->batch * runs > INT32_MAX) return E2H_ERR_BAD_SHAPE;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (a->dtype == E2H_SEQ_BF16) launch_norm_conv<bf16_t>(*a, static_cast<int>(runs), run, s);
+  else launch_norm_conv<float>(*a, static_cast<int>(runs), run, s);
+  return launch_status();
+}
+
+extern "C" int e2h_seq_square_relu(int dtype, const void *x, void *y, int64_t n, void *stream) {
+  return launch_elementwise<kSquareRelu>(dtype, x, y, n, 0.f, stream);
+}
+
+extern "C" int e2h_seq_softcap(int dtype, const void *x, void *y, int64_t n, float cap, void *stream) {
+  if (!(cap > 0.f)) return E2H_ERR_BAD_SHAPE;
+  return launch_elementwise<kSoftcap>(dtype, x, y, n, cap, stream);
+}
+
+extern "C" int e2h_seq_gelu_gate_rows(int dtype, const void *gate, const void *table, const int64_t *tokens, void *y, int64_t rows, int64_t dim,
+                                      int64_t ld, int64_t column, int64_t table_rows, void *stream) {
+  if (!gate || !table || !tokens || !y) return E2H_ERR_NULL_POINTER;
+  if (rows < 1 || dim < 1 || dim > INT32_MAX || column < 0 || column + dim > ld || table_rows < 1) return E2H_ERR_BAD_SHAPE;
+  if (dtype != E2H_SEQ_BF16 && dtype != E2H_SEQ_F32) return E2H_ERR_BAD_SHAPE;
+  const int64_t n = rows * dim, blocks = (n + 255) / 256;
+  if (blocks > INT32_MAX) return E2H_ERR_BAD_SHAPE;
+  const dim3 grid(static_cast<unsigned>(blocks)), block(256);
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (dtype == E2H_SEQ_BF16)
+    hipLaunchKernelGGL(gelu_gate_rows_kernel<bf16_t>, grid, block, 0, s, static_cast<const bf16_t *>(gate), static_cast<const bf16_t *>(table), tokens,
+                       static_cast<bf16_t *>(y), n, static_cast<int>(dim), ld, column, table_rows);
+  else
+    hipLaunchKernelGGL(gelu_gate_rows_kernel<float>, grid, block, 0, s, static_cast<const float *>(gate), static_cast<const float *>(table), tokens,
+                       static_cast<float *>(y), n, static_cast<int>(dim), ld, column, table_rows);
+  return launch_status();
+}

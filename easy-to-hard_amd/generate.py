@@ -59,11 +59,17 @@ def _next_token(logits: Tensor, temperature: Optional[float], top_k: Optional[in
 
 
 def _greedy_through_the_model(model) -> bool:
-    """True for this package's Transformer, whose forward can return the greedy token itself (a wrapped or compiled
+    """True for this package's models, whose forward can return the greedy token itself (a wrapped or compiled
     module, or a stand-in with the reference's signature, is asked for logits)."""
-    from .model import Transformer
+    return getattr(type(model), "returns_greedy_token", False)
 
-    return isinstance(model, Transformer)
+
+@torch.no_grad()
+def extend(model, tokens: Tensor, start: int, left_pad_mask_pos: Optional[Tensor] = None) -> Tensor:
+    """Run the sequences' next tokens [B, T], which stand at positions start .. start + T - 1, from what earlier calls left in
+    the caches and state -> logits [B, T, vocab].  A prompt may be handed over in portions of any size."""
+    input_pos = torch.arange(start, start + tokens.shape[1], device=tokens.device)
+    return model(tokens, input_pos, left_pad_mask_pos)
 
 
 @torch.no_grad()
@@ -148,7 +154,9 @@ def load_model(checkpoint_path, device, precision=torch.bfloat16, use_tp: bool =
     and assigned, and the model moves to `device` in `precision` (integer buffers keep their dtype).
 
     The architecture comes from the checkpoint's parent directory name, as in the reference, unless `model_name` names
-    it.  `use_tp` is accepted for signature compatibility; this build runs on one GPU and rejects it."""
+    it.  `use_tp` is accepted for signature compatibility; this build runs on one GPU and rejects it.
+
+    A folder with config.json and model.safetensors goes to `load_folder`."""
     from pathlib import Path
 
     from .model import Transformer
@@ -157,6 +165,8 @@ def load_model(checkpoint_path, device, precision=torch.bfloat16, use_tp: bool =
     if use_tp:
         raise NotImplementedError("load_model: tensor parallelism is outside this one-GPU build")
     checkpoint_path = Path(checkpoint_path)
+    if checkpoint_path.is_dir():
+        return load_folder(checkpoint_path, device, precision)
     if not checkpoint_path.is_file():
         raise FileNotFoundError(str(checkpoint_path))
     with torch.device("meta"):
@@ -183,6 +193,27 @@ def load_model(checkpoint_path, device, precision=torch.bfloat16, use_tp: bool =
     model.load_state_dict(checkpoint, assign=True)
     model = model.to(device=device, dtype=precision)
     return model.eval()
+
+
+def load_folder(folder, device, precision=torch.bfloat16):
+    """Model of a checkpoint folder (config.json + model.safetensors): the class comes from the registry by the
+    configuration's architecture name, linears and embeddings are held in `precision`, norms and gate constants in float32."""
+    from pathlib import Path
+
+    from .checkpoint import SafetensorsFile, read_config
+    from .registry import model_from_config
+
+    config = read_config(folder)
+    with torch.device("meta"):
+        model = model_from_config(config)
+    tensors = SafetensorsFile(Path(folder) / "model.safetensors")
+    state = model.state_dict_from_checkpoint(tensors.get, precision)
+    for key, want in model.state_dict().items():
+        if key not in state or tuple(state[key].shape) != tuple(want.shape):
+            got = tuple(state[key].shape) if key in state else "missing"
+            raise ValueError(f"load_folder: {key} is {got} in {folder}, the configuration gives {tuple(want.shape)}")
+    model.load_state_dict({k: v.to(device) for k, v in state.items()}, assign=True)
+    return model.eval().requires_grad_(False)
 
 
 def load_reward_model(checkpoint_path, device, precision=torch.bfloat16, use_tp: bool = False,

@@ -1,0 +1,144 @@
+"""Token mixers with per-sequence state, as modules whose projections are ordinary linears.
+
+A `Branch` is one mechanism (windowed softmax attention, HGRN2, gated delta rule).  It names the projections it reads, and
+turns their columns into its part of the mixer's output.  A `TokenMixer` runs one or several branches on the same input:
+all their input projections are one linear and all their output projections another one over the concatenated branch
+outputs, so a mixer costs two matrix products however many branches it has.  A branch's share of the sum is a factor its
+kernel applies before the output projection.
+
+The two linears are plain nn.Linear modules: a QuantHandler can replace them like any other.
+"""
+
+import torch
+import torch.nn as nn
+from torch import Tensor
+
+from . import seq_ops
+from .state import SequenceState, StatePlan
+
+_ALIGN = 8  # projections start at multiples of this many columns (16 bytes in bfloat16)
+
+
+def _vector(n):
+    return nn.Parameter(torch.zeros((n,), dtype=torch.float32), requires_grad=False)
+
+
+class Branch(nn.Module):
+    """Subclasses set `projections` [(checkpoint name, rows)], `out_width` and `vectors` {checkpoint name: attribute}."""
+
+    projections: list
+    vectors: dict
+    out_width: int
+
+    def place(self, offset: int) -> int:
+        """Lay the projections out from column `offset` on; returns the first free column."""
+        self.columns = []
+        for _, rows in self.projections:
+            offset = (offset + _ALIGN - 1) // _ALIGN * _ALIGN
+            self.columns.append(offset)
+            offset += rows
+        return offset
+
+    def run(self, proj: Tensor, bsz: int, seqlen: int, state: SequenceState, input_pos: Tensor, first, out: Tensor, out_off: int) -> None:
+        raise NotImplementedError
+
+
+class WindowAttention(Branch):
+    """Softmax attention over the last `window` positions and the first `keep_first` ones, without rotation, with biased
+    q / k / v projections and an elementwise sigmoid output gate; window 0 = no limit."""
+
+    def __init__(self, plan: StatePlan, width, heads, kv_heads, dim, vdim, scale, window, keep_first, weight=1.0):
+        super().__init__()
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
+        self.scale, self.window, self.keep_first, self.weight = scale, window, keep_first, weight
+        self.projections = [("q", heads * dim), ("k", kv_heads * dim), ("v", kv_heads * vdim), ("g", heads * vdim)]
+        self.out_width = heads * vdim
+        self.q_bias, self.k_bias, self.v_bias = _vector(heads * dim), _vector(kv_heads * dim), _vector(kv_heads * vdim)
+        self.vectors = {"q.b": "q_bias", "k.b": "k_bias", "v.b": "v_bias"}
+        self.kv_index = plan.add_kv(kv_heads, dim, vdim)
+
+    def run(self, proj, bsz, seqlen, state, input_pos, first, out, out_off):
+        seq_ops.window_attention(proj, bsz, seqlen, self.heads, self.kv_heads, self.dim, self.vdim, self.columns,
+                                 (self.q_bias, self.k_bias, self.v_bias), state.kv[self.kv_index], input_pos, first, self.window, self.keep_first,
+                                 self.scale, out, out_off, self.weight)
+
+
+class HGRN2(Branch):
+    """Linear attention whose forget gate f also decides what is written: S = diag(f) S + (1 - f) v^T, o = S^T q."""
+
+    def __init__(self, plan: StatePlan, width, heads, dim, vdim, eps, weight=1.0):
+        super().__init__()
+        self.heads, self.dim, self.vdim, self.eps, self.weight = heads, dim, vdim, eps, weight
+        self.projections = [("q", heads * dim), ("f", heads * dim), ("v", heads * vdim)]
+        self.out_width = heads * vdim
+        self.f_bias, self.lower, self.norm = _vector(heads * dim), _vector(heads * dim), _vector(vdim)
+        self.vectors = {"f.b": "f_bias", "lower": "lower", "norm": "norm"}
+        self.state_index = plan.add_recurrent(heads, dim, vdim)
+
+    def run(self, proj, bsz, seqlen, state, input_pos, first, out, out_off):
+        seq_ops.hgrn2(proj, bsz, seqlen, self.heads, self.dim, self.vdim, self.columns, self.f_bias, self.lower, self.norm, self.eps,
+                      state.recurrent[self.state_index].s, input_pos, first, out, out_off, self.weight)
+
+
+class GatedDelta(Branch):
+    """Gated delta rule on unit queries and keys, with short causal convolutions on q, k and v."""
+
+    def __init__(self, plan: StatePlan, width, heads, kv_heads, dim, vdim, taps, eps, weight=1.0):
+        super().__init__()
+        self.heads, self.kv_heads, self.dim, self.vdim, self.eps, self.weight = heads, kv_heads, dim, vdim, eps, weight
+        self.projections = [("q", kv_heads * dim), ("k", kv_heads * dim), ("v", heads * vdim), ("b", heads), ("a", heads), ("g", heads * vdim)]
+        self.out_width = heads * vdim
+        self.channels = 2 * kv_heads * dim + heads * vdim
+        self.conv = nn.Parameter(torch.zeros((self.channels, taps), dtype=torch.float32), requires_grad=False)
+        self.a_log, self.dt_bias, self.norm = _vector(heads), _vector(heads), _vector(vdim)
+        self.vectors = {("q.conv", "k.conv", "v.conv"): "conv", "A_log": "a_log", "dt_bias": "dt_bias", "norm": "norm"}
+        self.state_index = plan.add_recurrent(heads, dim, vdim)
+        self.ring_index = plan.add_ring(self.channels, taps, float32=False)
+
+    def run(self, proj, bsz, seqlen, state, input_pos, first, out, out_off):
+        seq_ops.gated_delta(proj, bsz, seqlen, self.heads, self.kv_heads, self.dim, self.vdim, self.columns, self.conv,
+                            state.rings.site(self.ring_index, seqlen), self.a_log, self.dt_bias, self.norm, self.eps,
+                            state.recurrent[self.state_index].s, input_pos, first, out, out_off, self.weight)
+
+
+class TokenMixer(nn.Module):
+    """Branches side by side on one input; `names` are their prefixes in a checkpoint ("" for a mixer that is one branch)."""
+
+    def __init__(self, width: int, branches, names):
+        super().__init__()
+        self.branches = nn.ModuleList(branches)
+        self.names = list(names)
+        offset = 0
+        for b in self.branches:
+            offset = b.place(offset)
+        self.in_proj = nn.Linear(width, (offset + _ALIGN - 1) // _ALIGN * _ALIGN, bias=False)
+        self.out_proj = nn.Linear(sum(b.out_width for b in self.branches), width, bias=False)
+
+    def forward(self, h: Tensor, bsz: int, seqlen: int, state: SequenceState, input_pos: Tensor, first) -> Tensor:
+        proj = self.in_proj(h)
+        out = torch.empty((h.shape[0], self.out_proj.in_features), dtype=proj.dtype, device=proj.device)
+        off = 0
+        for b in self.branches:
+            b.run(proj, bsz, seqlen, state, input_pos, first, out, off)
+            off += b.out_width
+        return self.out_proj(out)
+
+    def from_checkpoint(self, get, prefix: str, linear_dtype) -> dict:
+        """State-dict entries of this module from the tensors `get(name)` of a checkpoint with one linear per projection."""
+        sd = {}
+        rows = torch.zeros((self.in_proj.out_features, self.in_proj.in_features), dtype=linear_dtype)
+        outs = []
+        for i, (b, name) in enumerate(zip(self.branches, self.names)):
+            base = f"{prefix}.{name}" if name else prefix
+            for (proj, n), col in zip(b.projections, b.columns):
+                w = get(f"{base}.{proj}")
+                if tuple(w.shape) != (n, rows.shape[1]):
+                    raise ValueError(f"{base}.{proj} has shape {tuple(w.shape)}, the configuration gives {(n, rows.shape[1])}")
+                rows[col: col + n] = w.to(linear_dtype)
+            outs.append(get(f"{base}.o").to(linear_dtype))
+            for src, attr in b.vectors.items():
+                parts = [get(f"{base}.{s}").float() for s in ((src,) if isinstance(src, str) else src)]
+                sd[f"branches.{i}.{attr}"] = torch.cat(parts)
+        sd["in_proj.weight"] = rows
+        sd["out_proj.weight"] = torch.cat(outs, dim=1)
+        return sd

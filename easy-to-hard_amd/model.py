@@ -19,6 +19,7 @@ from torch import Tensor
 
 from . import ops
 from .quantize import WeightOnlyInt4Linear, WeightOnlyInt8Linear, find_multiple
+from .state import KVCache
 
 # When True (default) and the tensors are bf16 on the GPU, RMSNorm, SiLU*mul and -- for single-token steps with
 # a KV cache -- RoPE + cache write + attention run as this package's fused kernels instead of chains of stock ops.
@@ -84,23 +85,6 @@ transformer_configs = {
     "tiny-gqa-test": dict(block_size=256, vocab_size=512, n_layer=2, n_head=8, n_local_heads=2, dim=512,
                           intermediate_size=1024),
 }
-
-
-class KVCache(nn.Module):
-    """bf16 [B, H_kv, S_max, D] key and value caches written at `input_pos` (reference :112-129)."""
-
-    def __init__(self, max_batch_size, max_seq_length, n_heads, head_dim, dtype=torch.bfloat16, device=None):
-        super().__init__()
-        shape = (max_batch_size, n_heads, max_seq_length, head_dim)
-        self.register_buffer("k_cache", torch.zeros(shape, dtype=dtype, device=device))
-        self.register_buffer("v_cache", torch.zeros(shape, dtype=dtype, device=device))
-
-    def update(self, input_pos, k_val, v_val):
-        assert input_pos.shape[0] == k_val.shape[2]
-        bsz = k_val.size(0)
-        self.k_cache[:bsz].index_copy_(2, input_pos, k_val)
-        self.v_cache[:bsz].index_copy_(2, input_pos, v_val)
-        return self.k_cache[:bsz], self.v_cache[:bsz]
 
 
 class RMSNorm(nn.Module):
@@ -352,6 +336,8 @@ def _staged_block_forward(blk: "TransformerBlock", x: Tensor, delta, input_pos: 
 
 
 class Transformer(nn.Module):
+    returns_greedy_token = True  # forward(..., greedy_token=True) yields the token itself
+
     def __init__(self, config: ModelArgs) -> None:
         super().__init__()
         self.config = config

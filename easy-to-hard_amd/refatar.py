@@ -1,0 +1,209 @@
+"""The Refatar decoder: layers of parallel (windowed attention + HGRN2) and gated-delta mixers with sandwich norms, a causal
+convolution in front of every sublayer, and a per-layer embedding of the token added at the end of every layer.
+
+Per layer, with n(.) the zero-centred RMS norm and c(h) = h + conv(h):
+    x = x + n1b(mixer(c1(n1(x))))
+    x = x + n2b(ff(c2(n2(x))))                          (absent when the layer has no feed-forward)
+    x = x + rms(proj(gelu(gate x) * table[token, layer])) * w
+The residual stream is float32.  Each "x + norm(y)" is not computed where y is: it stays pending and is folded into the kernel
+that normalises x for the next sublayer, which also runs that sublayer's convolution, so a layer needs three such passes.
+"""
+
+from dataclasses import dataclass, field
+from typing import List, Optional
+
+import torch
+import torch.nn as nn
+from torch import Tensor
+
+from . import ops, seq_ops
+from .mixers import GatedDelta, HGRN2, TokenMixer, WindowAttention
+from .state import SequenceState, StatePlan
+
+
+@dataclass
+class RefatarArgs:
+    vocab_size: int
+    dim: int
+    layers: List[dict] = field(default_factory=list)  # per layer: {"type", "mixer", "mlp"} as in config.json
+    norm_eps: float = 1e-6
+    canon_taps: int = 4
+    side_dim: int = 16
+    logit_softcap: Optional[float] = None
+    block_size: int = 1 << 20  # positions do not enter any layer's weights; the caches are sized by setup_caches
+
+    @classmethod
+    def from_config(cls, config: dict) -> "RefatarArgs":
+        for i, layer in enumerate(config["layers"]):
+            if layer["type"] not in ("parallel", "delta"):
+                raise ValueError(f"layer {i}: unknown mixer type {layer['type']!r}")
+            mlp = layer.get("mlp")
+            if mlp is not None and mlp.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward kind {mlp['kind']!r}")
+        return cls(vocab_size=config["vocab"], dim=config["width"], layers=config["layers"], norm_eps=config["norm"]["eps"],
+                   canon_taps=config["canon"]["taps"], side_dim=config["token_side"]["dim"], logit_softcap=config.get("logit_softcap"))
+
+
+def build_mixer(plan: StatePlan, width: int, layer: dict, eps: float) -> TokenMixer:
+    m = layer["mixer"]
+    if layer["type"] == "delta":
+        return TokenMixer(width, [GatedDelta(plan, width, m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["conv"], eps)], [""])
+    left, right = m["left"], m["right"]
+    return TokenMixer(width, [
+        WindowAttention(plan, width, left["heads"], left["kv_heads"], left["dim"], left["vdim"], left["scale"], left["mask"]["size"],
+                        left["mask"]["keep_first"], m["left_scale"]),
+        HGRN2(plan, width, right["heads"], right["dim"], right["vdim"], eps, m["right_scale"]),
+    ], ["left", "right"])
+
+
+def _vector(n):
+    return nn.Parameter(torch.zeros((n,), dtype=torch.float32), requires_grad=False)
+
+
+class SquaredReluFF(nn.Module):
+    def __init__(self, width: int, hidden: int):
+        super().__init__()
+        self.up = nn.Linear(width, hidden, bias=False)
+        self.down = nn.Linear(hidden, width, bias=False)
+
+    def forward(self, h: Tensor) -> Tensor:
+        return self.down(seq_ops.square_relu_(self.up(h)))
+
+
+class RefatarLayer(nn.Module):
+    def __init__(self, plan: StatePlan, args: RefatarArgs, index: int):
+        super().__init__()
+        layer, w, taps = args.layers[index], args.dim, args.canon_taps
+        self.mixer = build_mixer(plan, w, layer, args.norm_eps)
+        self.norm1, self.norm1b = _vector(w), _vector(w)
+        self.canon1 = nn.Parameter(torch.zeros((w, taps), dtype=torch.float32), requires_grad=False)
+        self.ring1 = plan.add_ring(w, taps, float32=True)
+        self.feed_forward = None
+        if layer.get("mlp") is not None:
+            self.feed_forward = SquaredReluFF(w, layer["mlp"]["ff"])
+            self.norm2, self.norm2b = _vector(w), _vector(w)
+            self.canon2 = nn.Parameter(torch.zeros((w, taps), dtype=torch.float32), requires_grad=False)
+            self.ring2 = plan.add_ring(w, taps, float32=True)
+        self.side_gate = nn.Linear(w, args.side_dim, bias=False)
+        self.side_proj = nn.Linear(args.side_dim, w, bias=False)
+        self.side_norm = _vector(w)
+        self.side_column = index * args.side_dim
+
+    def from_checkpoint(self, get, prefix: str, linear_dtype) -> dict:
+        sd = {f"mixer.{k}": v for k, v in self.mixer.from_checkpoint(get, prefix + ".mix", linear_dtype).items()}
+        names = ["norm1", "norm1b", "canon1"]
+        if self.feed_forward is not None:
+            names += ["norm2", "norm2b", "canon2"]
+            sd["feed_forward.up.weight"] = get(prefix + ".mlp.up").to(linear_dtype)
+            sd["feed_forward.down.weight"] = get(prefix + ".mlp.down").to(linear_dtype)
+        for n in names:
+            sd[n] = get(f"{prefix}.{n}").float()
+        sd["side_gate.weight"] = get(prefix + ".side.gate").to(linear_dtype)
+        sd["side_proj.weight"] = get(prefix + ".side.proj").to(linear_dtype)
+        sd["side_norm"] = get(prefix + ".side.norm").float()
+        return sd
+
+
+class Refatar(nn.Module):
+    """Same interface as model.Transformer: setup_caches, then forward(idx, input_pos) over any number of new tokens."""
+
+    returns_greedy_token = True  # forward(..., greedy_token=True) yields the token itself
+
+    def __init__(self, config: RefatarArgs):
+        super().__init__()
+        self.config = config
+        self.plan = StatePlan()
+        self.tok_embeddings = nn.Embedding(config.vocab_size, config.dim)
+        self.side_embeddings = nn.Embedding(config.vocab_size, len(config.layers) * config.side_dim)
+        self.layers = nn.ModuleList(RefatarLayer(self.plan, config, i) for i in range(len(config.layers)))
+        self.norm = _vector(config.dim)
+        self.output = nn.Linear(config.dim, config.vocab_size, bias=False)
+        self.logit_softcap = config.logit_softcap
+        self.state: Optional[SequenceState] = None
+        self.max_batch_size = self.max_seq_length = -1
+
+    @classmethod
+    def from_config(cls, config: dict) -> "Refatar":
+        return cls(RefatarArgs.from_config(config))
+
+    def state_dict_from_checkpoint(self, get, linear_dtype=torch.bfloat16) -> dict:
+        """This module's state dict from a checkpoint's tensors (`get(name)`), linears in `linear_dtype`, vectors in float32."""
+        sd = {"tok_embeddings.weight": get("embed").to(linear_dtype), "side_embeddings.weight": get("side.embed").to(linear_dtype),
+              "norm": get("final.norm").float(), "output.weight": get("head").to(linear_dtype)}
+        for i, layer in enumerate(self.layers):
+            sd.update({f"layers.{i}.{k}": v for k, v in layer.from_checkpoint(get, f"l{i}", linear_dtype).items()})
+        return sd
+
+    @property
+    def dtype(self):
+        return self.tok_embeddings.weight.dtype
+
+    def _new_state(self, max_batch_size, max_seq_length):
+        w = self.tok_embeddings.weight
+        return SequenceState(self.plan, max_batch_size, max_seq_length, w.dtype, w.device)
+
+    def setup_caches(self, max_batch_size, max_seq_length, kv_cache=True):
+        """Memory for the state of `max_batch_size` sequences; kv_cache=False (scoring passes) keeps none."""
+        if not kv_cache:
+            return
+        if self.state is not None and self.max_seq_length >= max_seq_length and self.max_batch_size >= max_batch_size:
+            return
+        self.max_seq_length, self.max_batch_size = (max_seq_length + 7) // 8 * 8, max_batch_size
+        self.state = self._new_state(self.max_batch_size, self.max_seq_length)
+
+    def forward(self, idx: Tensor, input_pos: Optional[Tensor] = None, left_pad_mask_pos: Optional[Tensor] = None, fully_causal: bool = False,
+                greedy_token: bool = False) -> Tensor:
+        """idx [B, S] token ids at consecutive positions input_pos [S] -> logits [B, S, vocab], or with greedy_token int64
+        [B, 1], the arg-max of the last position.  left_pad_mask_pos [B]: positions before it are padding.  fully_causal:
+        a pass over whole sequences from position 0 that keeps no state."""
+        bsz, seqlen = idx.shape
+        idx = idx.to(torch.int64).contiguous()
+        if fully_causal:
+            assert left_pad_mask_pos is None, "Invalid mask"
+            state = self._new_state(bsz, seqlen)
+            input_pos = torch.arange(seqlen, device=idx.device)
+        else:
+            assert self.state is not None, "Caches must be initialized first"
+            assert bsz <= self.max_batch_size
+            state = self.state
+            input_pos = input_pos.to(torch.int64).contiguous()
+        first = None if left_pad_mask_pos is None else left_pad_mask_pos.to(torch.int64).contiguous()
+        h = self._hidden(idx, bsz, seqlen, state, input_pos, first)
+        logits = self.output(h[:, -1:] if greedy_token else h)
+        if self.logit_softcap is not None:
+            logits = seq_ops.softcap_(logits.contiguous(), self.logit_softcap)
+        if not greedy_token:
+            return logits
+        last = logits[:, -1]
+        if last.dtype == torch.bfloat16:
+            return ops.argmax_rows(last)
+        return torch.argmax(last, dim=-1, keepdim=True)
+
+    def _hidden(self, idx, bsz, seqlen, state, input_pos, first):
+        """Normalised output of the last layer, [B, S, dim] in the model's dtype."""
+        dtype, eps = self.dtype, self.config.norm_eps
+        tokens = idx.view(-1)
+        x = self.tok_embeddings(tokens).float()
+        delta = None  # the sublayer output that has not been added to x yet, with its norm's weight and offset
+
+        def norm(x, delta, weight=None, conv=None, ring=None, want_out=True):
+            d, dw, off = delta if delta is not None else (None, None, 0.0)
+            tails = None if ring is None else state.rings_f32.site(ring, seqlen)
+            return seq_ops.norm_conv(x, bsz, seqlen, eps, dtype, delta=d, delta_weight=dw, delta_offset=off, norm_weight=weight, norm_offset=1.0,
+                                     conv=conv, tails=tails, input_pos=input_pos, first=first, want_out=want_out)
+
+        for layer in self.layers:
+            x, h = norm(x, delta, layer.norm1, layer.canon1, layer.ring1)
+            delta = (layer.mixer(h, bsz, seqlen, state, input_pos, first), layer.norm1b, 1.0)
+            if layer.feed_forward is not None:
+                x, h = norm(x, delta, layer.norm2, layer.canon2, layer.ring2)
+                delta = (layer.feed_forward(h), layer.norm2b, 1.0)
+            x, h = norm(x, delta, want_out=dtype != torch.float32)
+            gate = layer.side_gate(x if h is None else h)
+            gate = seq_ops.gelu_gate_rows(gate, self.side_embeddings.weight, tokens, layer.side_column)
+            delta = (layer.side_proj(gate), layer.side_norm, 0.0)
+        state.commit(bsz, seqlen)
+        d, dw, off = delta
+        _, h = seq_ops.norm_conv(x, bsz, seqlen, eps, dtype, delta=d, delta_weight=dw, delta_offset=off, norm_weight=self.norm, norm_offset=1.0,
+                                 want_x=False)
+        return h.view(bsz, seqlen, -1)

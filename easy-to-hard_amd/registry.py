@@ -1,0 +1,22 @@
+"""Model classes by the name that a checkpoint folder's config.json gives under "architecture".
+
+Llama-family checkpoints carry no config.json; their shape is found by name (model.transformer_configs)."""
+
+import importlib
+
+ARCHITECTURES = {
+    # name: (module of this package, class with from_config / state_dict_from_checkpoint)
+    "Refatar": ("refatar", "Refatar"),
+}
+
+
+def model_class(config: dict):
+    name = config.get("architecture")
+    if name not in ARCHITECTURES:
+        raise ValueError(f"unknown architecture {name!r}; known: {', '.join(sorted(ARCHITECTURES))}")
+    module, cls = ARCHITECTURES[name]
+    return getattr(importlib.import_module(f"{__package__}.{module}"), cls)
+
+
+def model_from_config(config: dict):
+    return model_class(config).from_config(config)

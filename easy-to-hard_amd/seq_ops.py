@@ -1,0 +1,210 @@
+"""Tensor-level wrappers of include/e2h_seq.h: the kernels of layers that carry per-sequence state.
+
+PyTorch owns the memory and the stream; the arithmetic is in libe2h_seq.so.  Inputs live on the GPU, there is no CPU
+implementation behind these functions.  Activations are bfloat16 or float32; norms, biases, gate constants and state are
+float32.
+"""
+
+import ctypes
+
+import torch
+
+from . import _lib
+from .ops import _need_gpu, _OnDevice, _stream
+
+_DTYPES = {torch.bfloat16: _lib.SEQ_BF16, torch.float32: _lib.SEQ_F32}
+
+
+def _dtype(t, what):
+    if t.dtype not in _DTYPES:
+        raise TypeError(f"{what}: bfloat16 or float32 activations expected, got {t.dtype}")
+    return _DTYPES[t.dtype]
+
+
+def _lib_for(t):
+    lib = _lib.load_seq()
+    return lib if t.device.index == torch.cuda.current_device() else _OnDevice(lib, t.device)
+
+
+def _p(t):
+    return None if t is None else t.data_ptr()
+
+
+def _vec(t, n, what):
+    """data pointer of a float32 vector of n values (None stays None)"""
+    if t is None:
+        return None
+    if t.dtype != torch.float32 or t.numel() != n or not t.is_contiguous() or not t.is_cuda:
+        raise TypeError(f"{what}: float32 [{n}] on the GPU expected, got {t.dtype} {tuple(t.shape)} on {t.device}")
+    return t.data_ptr()
+
+
+def _positions(input_pos, first, batch, seqlen, what):
+    if input_pos.dtype != torch.int64 or not input_pos.is_cuda or input_pos.numel() != seqlen:
+        raise TypeError(f"{what}: input_pos must be int64 [{seqlen}] on the GPU")
+    if first is not None and (first.dtype != torch.int64 or not first.is_cuda or first.numel() != batch or not first.is_contiguous()):
+        raise TypeError(f"{what}: left padding must be int64 [{batch}] on the GPU")
+    return _p(input_pos), _p(first)
+
+
+def _rows(t, batch, seqlen, what, width=None):
+    if t.dim() != 2 or t.shape[0] != batch * seqlen or not t.is_contiguous() or (width is not None and t.shape[1] != width):
+        raise RuntimeError(f"{what}: contiguous [{batch * seqlen}, {width if width is not None else '*'}] expected, got {tuple(t.shape)}")
+
+
+def _check_tail(tails, batch, taps, channels, dtype, what):
+    for t in tails:
+        if t.dtype != dtype or t.dim() != 3 or t.shape[0] < batch or tuple(t.shape[1:]) != (taps, channels) or not t.is_contiguous() or not t.is_cuda:
+            raise RuntimeError(f"{what}: convolution ring must be {dtype} [>= {batch}, {taps}, {channels}], got {t.dtype} {tuple(t.shape)}")
+
+
+def norm_conv(x, batch, seqlen, eps, dtype, delta=None, delta_weight=None, delta_offset=0.0, norm_weight=None, norm_offset=0.0, conv=None,
+              tails=None, input_pos=None, first=None, want_x=True, want_out=True):
+    """x + norm(delta), its norm and the norm's convolution over time (each optional) in one pass; x float32 [rows, width].
+
+    Returns (x_out float32 or x itself when there is no delta, out in `dtype` or None)."""
+    _need_gpu(x)
+    width = x.shape[-1]
+    if x.dtype != torch.float32:
+        raise TypeError("norm_conv: the residual stream is float32")
+    _rows(x, batch, seqlen, "norm_conv", width)
+    a = _lib.NormConvArgs(dtype=_DTYPES[dtype], batch=batch, seqlen=seqlen, width=width, eps=eps, delta_offset=delta_offset, norm_offset=norm_offset,
+                          x=_p(x))
+    x_out = x
+    if delta is not None:
+        _need_gpu(delta)
+        _rows(delta, batch, seqlen, "norm_conv delta", width)
+        if delta.dtype != dtype:
+            raise TypeError(f"norm_conv: delta is {delta.dtype}, expected {dtype}")
+        a.delta, a.delta_weight = _p(delta), _vec(delta_weight, width, "norm_conv delta_weight")
+        if want_x:
+            x_out = torch.empty_like(x)
+            a.x_out = _p(x_out)
+    a.norm_weight = _vec(norm_weight, width, "norm_conv norm_weight")
+    if conv is not None:
+        taps = conv.shape[-1]
+        a.taps, a.conv = taps, _vec(conv, width * taps, "norm_conv conv")
+        a.input_pos, a.first = _positions(input_pos, first, batch, seqlen, "norm_conv")
+        if taps > 1:
+            _check_tail(tails, batch, taps, width, torch.float32, "norm_conv")
+            a.tail_in, a.tail_out = _p(tails[0]), _p(tails[1])
+    out = torch.empty((batch * seqlen, width), dtype=dtype, device=x.device) if want_out else None
+    a.out = _p(out)
+    _lib.check_seq(_lib_for(x).e2h_seq_norm_conv(ctypes.byref(a), _stream(x)), "e2h_seq_norm_conv")
+    return x_out, out
+
+
+def square_relu_(x):
+    """max(x, 0)^2 in place."""
+    _need_gpu(x)
+    assert x.is_contiguous()
+    _lib.check_seq(_lib_for(x).e2h_seq_square_relu(_dtype(x, "square_relu_"), _p(x), _p(x), x.numel(), _stream(x)), "e2h_seq_square_relu")
+    return x
+
+
+def softcap_(x, cap):
+    """cap * tanh(x / cap) in place."""
+    _need_gpu(x)
+    assert x.is_contiguous()
+    _lib.check_seq(_lib_for(x).e2h_seq_softcap(_dtype(x, "softcap_"), _p(x), _p(x), x.numel(), cap, _stream(x)), "e2h_seq_softcap")
+    return x
+
+
+def gelu_gate_rows(gate, table, tokens, column):
+    """gelu_tanh(gate) * table[tokens, column : column + dim]; gate [rows, dim], tokens int64 [rows]."""
+    _need_gpu(gate, table, tokens)
+    rows, dim = gate.shape
+    if table.dtype != gate.dtype or table.dim() != 2 or not table.is_contiguous() or not gate.is_contiguous():
+        raise TypeError("gelu_gate_rows: gate and table must be contiguous and of one dtype")
+    if tokens.dtype != torch.int64 or tokens.numel() != rows or not tokens.is_contiguous():
+        raise TypeError("gelu_gate_rows: one int64 token per row expected")
+    y = torch.empty_like(gate)
+    _lib.check_seq(_lib_for(gate).e2h_seq_gelu_gate_rows(_dtype(gate, "gelu_gate_rows"), _p(gate), _p(table), _p(tokens), _p(y), rows, dim,
+                                                         table.shape[1], column, table.shape[0], _stream(gate)), "e2h_seq_gelu_gate_rows")
+    return y
+
+
+def window_attention(proj, batch, seqlen, heads, kv_heads, dim, vdim, offsets, biases, cache, input_pos, first, window, keep_first, scale,
+                     out, out_off, out_scale=1.0):
+    """Softmax attention over a window and the first `keep_first` positions (window 0: all positions), with projection biases
+    and output gate; see e2h_seq_window_attention.  offsets = columns of (q, k, v, gate or -1) in proj, biases = (q, k, v)
+    float32 or None, cache a state.KVCache.  Appends the new keys and values and writes out[:, out_off : ...]."""
+    _need_gpu(proj, out)
+    _rows(proj, batch, seqlen, "window_attention proj")
+    _rows(out, batch, seqlen, "window_attention out")
+    kc, vc = cache.k_cache, cache.v_cache
+    if kc.dtype != proj.dtype or vc.dtype != proj.dtype or out.dtype != proj.dtype:
+        raise TypeError("window_attention: projections, caches and output must have one dtype")
+    if kc.shape[0] < batch or tuple(kc.shape[1::2]) != (kv_heads, dim) or tuple(vc.shape) != (*kc.shape[:3], vdim):
+        raise RuntimeError(f"window_attention: cache shapes {tuple(kc.shape)}, {tuple(vc.shape)} do not fit")
+    a = _lib.WindowAttentionArgs(dtype=_dtype(proj, "window_attention"), batch=batch, seqlen=seqlen, heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim,
+                                 cache_len=kc.shape[2], proj=_p(proj), ld=proj.shape[1], q_off=offsets[0], k_off=offsets[1], v_off=offsets[2],
+                                 g_off=offsets[3], k_cache=_p(kc), v_cache=_p(vc), window=window, keep_first=keep_first, scale=scale,
+                                 out_scale=out_scale, out=_p(out), ld_out=out.shape[1], out_off=out_off)
+    a.q_bias = _vec(biases[0], heads * dim, "window_attention q bias")
+    a.k_bias = _vec(biases[1], kv_heads * dim, "window_attention k bias")
+    a.v_bias = _vec(biases[2], kv_heads * vdim, "window_attention v bias")
+    a.input_pos, a.first = _positions(input_pos, first, batch, seqlen, "window_attention")
+    _lib.check_seq(_lib_for(proj).e2h_seq_window_attention(ctypes.byref(a), _stream(proj)), "e2h_seq_window_attention")
+
+
+def _scratch(args, query, like):
+    n = query(ctypes.byref(args))
+    if n < 0:
+        _lib.check_seq(int(n), query.__name__ if hasattr(query, "__name__") else "scratch query")
+    if n == 0:
+        return None
+    buf = torch.empty((n,), dtype=torch.uint8, device=like.device)
+    args.scratch, args.scratch_bytes = _p(buf), n
+    return buf
+
+
+def _check_state(state, batch, heads, dim, vdim, what):
+    if state.dtype != torch.float32 or state.shape[0] < batch or tuple(state.shape[1:]) != (heads, dim, vdim) or not state.is_contiguous() or not state.is_cuda:
+        raise RuntimeError(f"{what}: state must be float32 [>= {batch}, {heads}, {dim}, {vdim}], got {state.dtype} {tuple(state.shape)}")
+
+
+def hgrn2(proj, batch, seqlen, heads, dim, vdim, offsets, f_bias, lower, norm_weight, eps, state, input_pos, first, out, out_off, out_scale=1.0):
+    """HGRN2 recurrence with RMS-normed heads; see e2h_seq_hgrn2.  offsets = columns of (q, f, v) in proj; state float32
+    [B, heads, dim, vdim], updated in place; writes out[:, out_off : out_off + heads * vdim]."""
+    _need_gpu(proj, out, state)
+    _rows(proj, batch, seqlen, "hgrn2 proj")
+    _rows(out, batch, seqlen, "hgrn2 out")
+    _check_state(state, batch, heads, dim, vdim, "hgrn2")
+    if out.dtype != proj.dtype:
+        raise TypeError("hgrn2: projections and output must have one dtype")
+    a = _lib.Hgrn2Args(dtype=_dtype(proj, "hgrn2"), eps=eps, batch=batch, seqlen=seqlen, heads=heads, dim=dim, vdim=vdim, proj=_p(proj), ld=proj.shape[1],
+                       q_off=offsets[0], f_off=offsets[1], v_off=offsets[2], f_bias=_vec(f_bias, heads * dim, "hgrn2 f_bias"),
+                       lower=_vec(lower, heads * dim, "hgrn2 lower"), norm_weight=_vec(norm_weight, vdim, "hgrn2 norm"), state=_p(state),
+                       out_scale=out_scale, out=_p(out), ld_out=out.shape[1], out_off=out_off)
+    a.input_pos, a.first = _positions(input_pos, first, batch, seqlen, "hgrn2")
+    lib = _lib_for(proj)
+    scratch = _scratch(a, lib.e2h_seq_hgrn2_scratch_bytes, proj)
+    _lib.check_seq(lib.e2h_seq_hgrn2(ctypes.byref(a), _stream(proj)), "e2h_seq_hgrn2")
+    del scratch
+
+
+def gated_delta(proj, batch, seqlen, heads, kv_heads, dim, vdim, offsets, conv, tails, a_log, dt_bias, norm_weight, eps, state, input_pos, first,
+                out, out_off, out_scale=1.0):
+    """Gated delta rule with short convolutions and a gated RMS norm; see e2h_seq_delta.  offsets = columns of
+    (q, k, v, b, a, gate) in proj; conv float32 [channels, taps] in the order q, k, v; tails = (ring to read, ring to write)."""
+    _need_gpu(proj, out, state)
+    _rows(proj, batch, seqlen, "gated_delta proj")
+    _rows(out, batch, seqlen, "gated_delta out")
+    _check_state(state, batch, heads, dim, vdim, "gated_delta")
+    if out.dtype != proj.dtype:
+        raise TypeError("gated_delta: projections and output must have one dtype")
+    channels, taps = 2 * kv_heads * dim + heads * vdim, conv.shape[-1]
+    a = _lib.DeltaArgs(dtype=_dtype(proj, "gated_delta"), taps=taps, batch=batch, seqlen=seqlen, heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim,
+                       proj=_p(proj), ld=proj.shape[1], q_off=offsets[0], k_off=offsets[1], v_off=offsets[2], b_off=offsets[3], a_off=offsets[4],
+                       g_off=offsets[5], conv=_vec(conv, channels * taps, "gated_delta conv"), a_log=_vec(a_log, heads, "gated_delta a_log"),
+                       dt_bias=_vec(dt_bias, heads, "gated_delta dt_bias"), norm_weight=_vec(norm_weight, vdim, "gated_delta norm"), state=_p(state),
+                       eps=eps, out_scale=out_scale, out=_p(out), ld_out=out.shape[1], out_off=out_off)
+    if taps > 1:
+        _check_tail(tails, batch, taps, channels, proj.dtype, "gated_delta")
+        a.tail_in, a.tail_out = _p(tails[0]), _p(tails[1])
+    a.input_pos, a.first = _positions(input_pos, first, batch, seqlen, "gated_delta")
+    lib = _lib_for(proj)
+    scratch = _scratch(a, lib.e2h_seq_delta_scratch_bytes, proj)
+    _lib.check_seq(lib.e2h_seq_delta(ctypes.byref(a), _stream(proj)), "e2h_seq_delta")
+    del scratch

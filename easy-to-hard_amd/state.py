@@ -1,0 +1,111 @@
+"""Per-sequence state of a decoder: key/value caches, recurrent state and the kept inputs of causal convolutions.
+
+A model's layers register what they need with a `StatePlan` while they are built and get an index back; a
+`SequenceState` then holds the memory of one batch of sequences for the whole model.  Row b of every buffer belongs to
+sequence b.  Nothing is cleared between sequences: the kernels take recurrent state and convolution inputs as empty when
+a call starts at position 0, and attention only reads cache rows that the sequence has written, so starting a sequence at
+position 0 in a row is what gives that row's previous contents back.
+"""
+
+import torch
+import torch.nn as nn
+
+
+class KVCache(nn.Module):
+    """[B, H_kv, S_max, D] key and value caches written at `input_pos` (reference models/model.py:112-129); the value
+    heads may have a size of their own."""
+
+    def __init__(self, max_batch_size, max_seq_length, n_heads, head_dim, dtype=torch.bfloat16, device=None, v_head_dim=None):
+        super().__init__()
+        shape = (max_batch_size, n_heads, max_seq_length)
+        self.register_buffer("k_cache", torch.zeros((*shape, head_dim), dtype=dtype, device=device))
+        self.register_buffer("v_cache", torch.zeros((*shape, v_head_dim or head_dim), dtype=dtype, device=device))
+
+    def update(self, input_pos, k_val, v_val):
+        assert input_pos.shape[0] == k_val.shape[2]
+        bsz = k_val.size(0)
+        self.k_cache[:bsz].index_copy_(2, input_pos, k_val)
+        self.v_cache[:bsz].index_copy_(2, input_pos, v_val)
+        return self.k_cache[:bsz], self.v_cache[:bsz]
+
+
+class RecurrentState(nn.Module):
+    """float32 [B, H, D, Dv] matrix state of a linear-attention layer, updated in place by its kernel."""
+
+    def __init__(self, max_batch_size, n_heads, dim, v_dim, device=None):
+        super().__init__()
+        self.register_buffer("s", torch.zeros((max_batch_size, n_heads, dim, v_dim), dtype=torch.float32, device=device))
+
+
+class ConvRings(nn.Module):
+    """The last inputs of a model's causal convolutions, each a ring [B, taps, channels] with slot = position mod taps.
+
+    A single-token step writes its slot in place (no other slot is free of readers, that one is).  A call with more tokens
+    may have several workgroups reading the old inputs while another one is ready with the new ones, so its kernels write
+    into a second copy that `commit` moves over at the end of the call."""
+
+    def __init__(self, max_batch_size, sites, dtype, device=None):
+        super().__init__()
+        self.max_batch_size = max_batch_size
+        self.shapes, self.offsets, total = [], [], 0
+        for channels, taps in sites:
+            self.shapes.append((max_batch_size, taps, channels))
+            self.offsets.append(total)
+            total += (max_batch_size * taps * channels + 31) // 32 * 32
+        self.register_buffer("live", torch.zeros((total,), dtype=dtype, device=device))
+        self.register_buffer("pending", torch.zeros((total,), dtype=dtype, device=device))
+
+    def _view(self, flat, i):
+        b, t, c = self.shapes[i]
+        return flat[self.offsets[i]: self.offsets[i] + b * t * c].view(b, t, c)
+
+    def site(self, i, seqlen):
+        """(ring to read, ring to write) of convolution i for a call with `seqlen` tokens per sequence."""
+        live = self._view(self.live, i)
+        return live, (live if seqlen == 1 else self._view(self.pending, i))
+
+    def commit(self, bsz, seqlen):
+        if seqlen == 1 or self.live.numel() == 0:
+            return
+        if bsz == self.max_batch_size:
+            self.live.copy_(self.pending)
+            return
+        for i in range(len(self.shapes)):  # rows of sequences outside this call keep their inputs
+            self._view(self.live, i)[:bsz].copy_(self._view(self.pending, i)[:bsz])
+
+
+class StatePlan:
+    """What the layers of one model keep per sequence; filled in while the model is built."""
+
+    def __init__(self):
+        self.kv, self.recurrent, self.rings_f32, self.rings = [], [], [], []
+
+    def _add(self, items, item):
+        items.append(item)
+        return len(items) - 1
+
+    def add_kv(self, n_heads, head_dim, v_head_dim):
+        return self._add(self.kv, (n_heads, head_dim, v_head_dim))
+
+    def add_recurrent(self, n_heads, dim, v_dim):
+        return self._add(self.recurrent, (n_heads, dim, v_dim))
+
+    def add_ring(self, channels, taps, float32):
+        """A convolution over float32 values or over activations in the model's dtype."""
+        return self._add(self.rings_f32 if float32 else self.rings, (channels, taps))
+
+
+class SequenceState(nn.Module):
+    """The memory behind a StatePlan for up to `max_batch_size` sequences of up to `max_seq_length` positions."""
+
+    def __init__(self, plan: StatePlan, max_batch_size, max_seq_length, dtype, device):
+        super().__init__()
+        self.max_batch_size, self.max_seq_length = max_batch_size, max_seq_length
+        self.kv = nn.ModuleList(KVCache(max_batch_size, max_seq_length, h, d, dtype, device, dv) for h, d, dv in plan.kv)
+        self.recurrent = nn.ModuleList(RecurrentState(max_batch_size, h, d, dv, device) for h, d, dv in plan.recurrent)
+        self.rings_f32 = ConvRings(max_batch_size, plan.rings_f32, torch.float32, device)
+        self.rings = ConvRings(max_batch_size, plan.rings, dtype, device)
+
+    def commit(self, bsz, seqlen):
+        self.rings_f32.commit(bsz, seqlen)
+        self.rings.commit(bsz, seqlen)

@@ -1,0 +1,146 @@
+/*
+ * e2h_seq.h -- C ABI of libe2h_seq.so: the kernels of decoder layers that carry per-sequence state beside a KV cache
+ * (windowed attention with kept first tokens, HGRN2, gated delta rule, causal convolutions over time), for AMD MI355X
+ * (gfx950).
+ *
+ * Conventions
+ *   - every pointer is a DEVICE pointer into memory the caller owns; nothing here allocates, frees or synchronises.
+ *     Kernels are enqueued on `stream` (a hipStream_t passed as void*) and may be recorded into a HIP graph.
+ *   - activations are bfloat16 or float32 (`dtype`: E2H_SEQ_BF16 / E2H_SEQ_F32); norms, biases, gates, convolution
+ *     weights of the norm kernels, the residual stream and recurrent state are float32 in both cases.
+ *   - a call covers `seqlen` consecutive tokens of each of `batch` sequences; row b * seqlen + t is token t of sequence b.
+ *     `input_pos` points at the position of token 0 (int64, device memory: graph replays move it), `first` (NULL = all
+ *     zero) at one int64 per sequence: positions before it are padding and do not exist for the sequence.
+ *   - state is continued from the previous call when the position is not 0 and taken as empty when it is.
+ *   - the convolutions keep their last inputs in a ring of `taps` slots, slot = position mod taps.  With seqlen == 1 the
+ *     kernel puts the new input into tail_out, which may be tail_in itself; with seqlen > 1 tail_out must be different
+ *     memory, receives the last taps - 1 inputs, and the caller copies it over tail_in afterwards.
+ *   - every entry point returns E2H_OK or a negative E2H_ERR_* code of e2h_quant.h; sizes that a kernel does not take give
+ *     E2H_ERR_BAD_SHAPE.
+ */
+#ifndef E2H_SEQ_H
+#define E2H_SEQ_H
+
+#include <stdint.h>
+
+#include "e2h_quant.h"
+
+#ifdef __cplusplus
+extern "C" {
+#endif
+
+#define E2H_SEQ_ABI_VERSION 1
+#define E2H_SEQ_BF16 0
+#define E2H_SEQ_F32 1
+
+int e2h_seq_abi_version(void);
+/* Experiment switches (0 = built-in choice): "recurrence_form" 1 = token by token, 2 = chunked; "recurrence_chunk" = tokens a
+ * workgroup of the chunked HGRN2 form covers; "norm_run" = tokens a workgroup of the norm kernel covers;
+ * "attention_decode_waves" = 4 or 8; "attention_query_tiles" = 1 or 2. */
+int e2h_seq_set_option(const char *name, int value);
+
+/* x_out = x + norm(delta); h = norm(x_out); out = h + conv(h), each step optional:
+ *   norm(z) = z / sqrt(mean(z^2) + eps) * (offset + weight)
+ *   conv(h)[t] = sum_j w[:, j] h[t - taps + 1 + j], zero before the sequence starts.
+ * delta NULL: x_out = x, not stored.  norm_weight NULL: h = x_out.  conv NULL: out = h.  One of x_out and out may be NULL. */
+typedef struct {
+  int32_t dtype; /* of delta and out */
+  int32_t taps;
+  int64_t batch, seqlen, width;
+  float eps, delta_offset, norm_offset;
+  int32_t pad_;
+  const float *x;            /* [rows, width] */
+  const void *delta;         /* [rows, width] or NULL */
+  const float *delta_weight; /* [width] */
+  float *x_out;              /* [rows, width], different memory from x when seqlen > 1 */
+  const float *norm_weight;  /* [width] or NULL */
+  const float *conv;         /* [width, taps] or NULL */
+  const float *tail_in;      /* [batch, taps, width] */
+  float *tail_out;
+  void *out;                 /* [rows, width] */
+  const int64_t *input_pos;
+  const int64_t *first;
+} e2h_norm_conv_args;
+int e2h_seq_norm_conv(const e2h_norm_conv_args *a, void *stream);
+
+/* Elementwise steps.  square_relu: y = max(x, 0)^2.  softcap: y = cap tanh(x / cap).  x and y may be the same memory.
+ * gelu_gate_rows: y[r, i] = gelu_tanh(gate[r, i]) * table[tokens[r], column + i], i < dim; table rows are ld values long. */
+int e2h_seq_square_relu(int dtype, const void *x, void *y, int64_t n, void *stream);
+int e2h_seq_softcap(int dtype, const void *x, void *y, int64_t n, float cap, void *stream);
+int e2h_seq_gelu_gate_rows(int dtype, const void *gate, const void *table, const int64_t *tokens, void *y, int64_t rows, int64_t dim,
+                           int64_t ld, int64_t column, int64_t table_rows, void *stream);
+
+/* Softmax attention of each sequence's new tokens over its cache: position i sees j <= i with i - j < window (window 0: no
+ * limit) or j < keep_first, counted from the sequence's first position.  The new tokens' keys and values are appended to
+ * the caches first.  Query head h reads key/value head h / (heads / kv_heads).  Biases (NULL = none) are added to the projections;
+ * the result is out_scale * attention * sigmoid(gate) (no gate when g_off < 0), written at out + row * ld_out + out_off. */
+typedef struct {
+  int32_t dtype;
+  int32_t pad_;
+  int64_t batch, seqlen, heads, kv_heads, dim, vdim, cache_len;
+  const void *proj; /* [rows, ld]: q, k, v, gate at columns q_off, k_off, v_off, g_off */
+  int64_t ld, q_off, k_off, v_off, g_off;
+  const float *q_bias, *k_bias, *v_bias;
+  void *k_cache, *v_cache; /* [batch, kv_heads, cache_len, dim | vdim] */
+  const int64_t *input_pos;
+  const int64_t *first;
+  int64_t window, keep_first;
+  float scale, out_scale;
+  void *out;
+  int64_t ld_out, out_off;
+} e2h_window_attention_args;
+int e2h_seq_window_attention(const e2h_window_attention_args *a, void *stream);
+
+/* HGRN2.  Per head: q = silu(q_proj), f = lower + (1 - lower) sigmoid(f_proj + f_bias), S = diag(f) S + (1 - f) v^T,
+ * o = S^T q; result out_scale * o / rms(o) * norm_weight at out + row * ld_out + out_off. */
+typedef struct {
+  int32_t dtype;
+  float eps;
+  int64_t batch, seqlen, heads, dim, vdim;
+  const void *proj;
+  int64_t ld, q_off, f_off, v_off;
+  const float *f_bias, *lower; /* [heads * dim] */
+  const float *norm_weight;    /* [vdim] */
+  float *state;                /* [batch, heads, dim, vdim] */
+  const int64_t *input_pos;
+  const int64_t *first;
+  void *scratch;
+  int64_t scratch_bytes; /* e2h_seq_hgrn2_scratch_bytes() */
+  float out_scale;
+  int32_t pad_;
+  void *out;
+  int64_t ld_out, out_off;
+} e2h_hgrn2_args;
+int64_t e2h_seq_hgrn2_scratch_bytes(const e2h_hgrn2_args *a);
+int e2h_seq_hgrn2(const e2h_hgrn2_args *a, void *stream);
+
+/* Gated delta rule.  q, k (kv_heads x dim) and v (heads x vdim) pass a causal convolution over time and silu; q and k become
+ * unit vectors, q is scaled by dim^-1/2; beta = sigmoid(b), g = exp(-exp(A_log) softplus(a + dt_bias)).
+ * Per head: S = g S, u = beta (v - S^T k), S = S + k u^T, o = S^T q; result o / rms(o) * norm_weight * silu(gate). */
+typedef struct {
+  int32_t dtype;
+  int32_t taps;
+  int64_t batch, seqlen, heads, kv_heads, dim, vdim;
+  const void *proj;
+  int64_t ld, q_off, k_off, v_off, b_off, a_off, g_off;
+  const float *conv; /* [2 kv_heads dim + heads vdim, taps], channels in the order q, k, v */
+  const void *tail_in; /* [batch, taps, channels], activations' dtype */
+  void *tail_out;
+  const float *a_log, *dt_bias, *norm_weight;
+  float *state; /* [batch, heads, dim, vdim] */
+  const int64_t *input_pos;
+  const int64_t *first;
+  void *scratch;
+  int64_t scratch_bytes; /* e2h_seq_delta_scratch_bytes() */
+  float eps, out_scale;
+  void *out;
+  int64_t ld_out, out_off;
+} e2h_delta_args;
+int64_t e2h_seq_delta_scratch_bytes(const e2h_delta_args *a);
+int e2h_seq_delta(const e2h_delta_args *a, void *stream);
+
+#ifdef __cplusplus
+}
+#endif
+
+#endif
