@@ -14,7 +14,6 @@
 namespace e2h {
 namespace {
 
-constexpr float kLog2e = 1.4426950408889634f;
 constexpr float kMasked = -1e30f;
 
 struct KeyList {  // virtual index n -> key position

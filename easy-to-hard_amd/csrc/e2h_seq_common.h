@@ -51,6 +51,16 @@ __device__ __forceinline__ float wave_add(float v) {
   return v;
 }
 
+constexpr float kLog2e = 1.4426950408889634f;
+
+// acc += A B over 16 rows of B in four steps of v_mfma_f32_16x16x4_f32.  Lane (b, c) = 16 b + c gives A[c][4 b .. 4 b + 3] and
+// B[4 b .. 4 b + 3][c]: step r multiplies rows {4 b + r}, so B may be the accumulators of another product as they are.
+__device__ __forceinline__ f32x4_t mfma4(f32x4_t a, f32x4_t b, f32x4_t acc) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[r], b[r], acc, 0, 0, 0);
+  return acc;
+}
+
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }

@@ -3,6 +3,16 @@
 //
 // delta_tokens_kernel: one workgroup per (sequence, head) with the head's state in registers.  For a single token it runs the
 // convolutions, the unit norms and the gates itself; for more tokens delta_prepare_kernel has put them into scratch memory.
+//
+// Chunked form (many tokens), float32 matrix cores throughout.  Within a chunk of 64 tokens that starts from state S0, with
+// G_t the decay from the chunk's start through token t,
+//   u_t + sum_{s<t} beta_t (G_t / G_s) (k_t . k_s) u_s = beta_t (v_t - G_t S0^T k_t)
+//   o_t = G_t S0^T q_t + sum_{s<=t} (G_t / G_s) (q_t . k_s) u_s,   S = G_end S0 + sum_s (G_end / G_s) k_s u_s^T
+// 1. delta_chunk_kernel, parallel over chunks: T = (I + M)^-1 diag(beta) for the strictly lower triangular M above (the four
+//    16 x 16 diagonal blocks by substitution, the others from products of blocks), and the masked, decayed products q k^T;
+// 2. delta_scan_kernel, one workgroup per (sequence, head, 16 value columns), chunk after chunk: read-outs, u = T (v - G S0^T k),
+//    outputs and the next state;
+// 3. delta_gate_kernel: RMS norm over the head and the silu gate.
 #include "e2h_seq_common.h"
 
 namespace e2h {
@@ -248,6 +258,316 @@ __global__ __launch_bounds__(BLOCK) void delta_tokens_kernel(const e2h_delta_arg
   }
 }
 
+// ---- chunked form ----------------------------------------------------------------------------------------------------------
+constexpr int kChunk = 64;
+
+struct ChunkScratch {
+  float *t;  // [batch * heads, chunks, 64, 64]
+  float *p;  // [batch * heads, chunks, 64, 64]
+  int chunks;
+};
+
+// four consecutive values of row `row` at column d; zero beyond the row's n values or when the row does not exist
+__device__ __forceinline__ f32x4_t row4(const float *base, bool exists, int d, int n) {
+  f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+  if (exists) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (d + e < n) v[e] = base[d + e];
+  }
+  return v;
+}
+template <bool VEC>
+__device__ __forceinline__ f32x4_t row4(const float *base, bool exists, int d, int n) {
+  if (!VEC) return row4(base, exists, d, n);
+  return exists && d < n ? load4(base + d) : f32x4_t{0.f, 0.f, 0.f, 0.f};  // n % 4 == 0
+}
+
+// step 1: 4 waves, one (sequence, head, chunk) each; wave w owns the token rows 16 w .. 16 w + 15
+template <bool VEC>
+__global__ __launch_bounds__(256) void delta_chunk_kernel(const e2h_delta_args a, Prepared p, ChunkScratch cs) {
+  constexpr int kRow = kChunk + 4;
+  __shared__ __attribute__((aligned(16))) float sm[kChunk * kRow];  // M, then its blocks are replaced by the inverse's
+  __shared__ __attribute__((aligned(16))) float si[kChunk * kRow];  // inverse
+  __shared__ float sg[kChunk], sb[kChunk];
+  const int D = static_cast<int>(a.dim), H = static_cast<int>(a.heads), kvh = static_cast<int>(a.kv_heads), seqlen = static_cast<int>(a.seqlen);
+  const int chunk = blockIdx.x % cs.chunks, bh = blockIdx.x / cs.chunks;
+  const int b = bh / H, h = bh % H, hk = h / (H / kvh);
+  const int wave = threadIdx.x >> 6, c = threadIdx.x & 15, b4 = (threadIdx.x & 63) >> 4;
+  const size_t row0 = static_cast<size_t>(b) * seqlen + static_cast<size_t>(chunk) * kChunk;
+  const int live = seqlen - chunk * kChunk < kChunk ? seqlen - chunk * kChunk : kChunk;  // tokens past the end: beta 0, decay 1, q = k = 0
+  if (threadIdx.x < 64) {
+    const int t = threadIdx.x;
+    float g = t < live ? p.log_g[(row0 + t) * H + h] : 0.f;
+#pragma unroll
+    for (int off = 1; off < 64; off <<= 1) {
+      const float up = __shfl_up(g, off);
+      if (t >= off) g += up;
+    }
+    sg[t] = g * kLog2e;
+    sb[t] = t < live ? p.beta[(row0 + t) * H + h] : 0.f;
+  }
+  for (int i = threadIdx.x; i < kChunk * kRow; i += 256) si[i] = 0.f;
+  // k k^T and q k^T for the column blocks up to this wave's
+  f32x4_t kk[4], qk[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) kk[j] = qk[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const size_t stride = static_cast<size_t>(kvh) * D;
+  const float *kb = p.k + (row0 * kvh + hk) * D, *qb = p.q + (row0 * kvh + hk) * D;
+  const int tr = 16 * wave + c;
+  for (int d = 4 * b4; d < (D + 15) / 16 * 16; d += 16) {
+    const f32x4_t ka = row4<VEC>(kb + tr * stride, tr < live, d, D), qa = row4<VEC>(qb + tr * stride, tr < live, d, D);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (j > wave) break;
+      const f32x4_t kc = j == wave ? ka : row4<VEC>(kb + (16 * j + c) * stride, 16 * j + c < live, d, D);
+      kk[j] = mfma4(ka, kc, kk[j]);
+      qk[j] = mfma4(qa, kc, qk[j]);
+    }
+  }
+  __syncthreads();
+  float *pt = cs.p + (static_cast<size_t>(bh) * cs.chunks + chunk) * kChunk * kChunk;
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    if (j > wave) break;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = 16 * wave + 4 * b4 + r, s = 16 * j + c;
+      const float dec = s <= t ? __builtin_amdgcn_exp2f(sg[t] - sg[s]) : 0.f;
+      sm[t * kRow + s] = s < t ? sb[t] * dec * kk[j][r] : 0.f;
+      pt[t * kChunk + s] = dec * qk[j][r];
+    }
+  }
+  __syncthreads();
+  // inverse of the unit lower triangular diagonal blocks: wave w, lane c = column c of block w, substitution down the rows
+  if (b4 == 0) {
+    float x[16];
+    const float *m = sm + (16 * wave) * kRow + 16 * wave;
+#pragma unroll
+    for (int t = 0; t < 16; ++t) {
+      float v = t == c ? 1.f : 0.f;
+#pragma unroll
+      for (int s = 0; s < 16; ++s)
+        if (s < t) v = __builtin_fmaf(-m[t * kRow + s], x[s], v);
+      x[t] = v;
+      si[(16 * wave + t) * kRow + 16 * wave + c] = v;
+    }
+  }
+  __syncthreads();
+  // blocks off the diagonal, by distance: I_ij = -I_ii sum_{j <= l < i} M_il I_lj
+#pragma unroll
+  for (int dist = 1; dist < 4; ++dist) {
+    const int i = wave, j = wave - dist;
+    f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+    if (j >= 0) {
+      for (int l = j; l < i; ++l) {
+        f32x4_t bb;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) bb[r] = si[(16 * l + 4 * b4 + r) * kRow + 16 * j + c];
+        acc = mfma4(load4(sm + (16 * i + c) * kRow + 16 * l + 4 * b4), bb, acc);
+      }
+      const f32x4_t res = mfma4(load4(si + (16 * i + c) * kRow + 16 * i + 4 * b4), acc, f32x4_t{0.f, 0.f, 0.f, 0.f});
+#pragma unroll
+      for (int r = 0; r < 4; ++r) si[(16 * i + 4 * b4 + r) * kRow + 16 * j + c] = -res[r];
+    }
+    __syncthreads();
+  }
+  float *tt = cs.t + (static_cast<size_t>(bh) * cs.chunks + chunk) * kChunk * kChunk;
+  for (int i = threadIdx.x; i < kChunk * kChunk; i += 256) {
+    const int s = i & 63;
+    tt[i] = si[(i >> 6) * kRow + s] * sb[s];
+  }
+}
+
+// step 2: DT = head dimension in tiles of 16.  Four waves; wave w owns the token rows 16 w .. 16 w + 15 of every chunk and the
+// state's row tiles w, w + 4, ...  The state is kept twice: in accumulators by its owner, and in LDS, transposed, as the B
+// operand of everybody's read-outs.
+template <int DT, bool VEC>
+__global__ __launch_bounds__(256) void delta_scan_kernel(const e2h_delta_args a, Prepared p, ChunkScratch cs, int v_blocks) {
+  constexpr int DP = DT * 16, OWN = (DT + 3) / 4, kRow = DP + 4, kTok = 20;
+  __shared__ __attribute__((aligned(16))) float st[16 * kRow];                       // state, [value column][row]
+  __shared__ __attribute__((aligned(16))) float sx[kChunk * kTok], su[kChunk * kTok];  // [token][value column]
+  __shared__ float sg[2][kChunk];
+  const int D = static_cast<int>(a.dim), DV = static_cast<int>(a.vdim), H = static_cast<int>(a.heads), kvh = static_cast<int>(a.kv_heads);
+  const int seqlen = static_cast<int>(a.seqlen), bh_count = static_cast<int>(a.batch) * H;
+  // the value blocks of one head read the same keys and queries: keep them on one die (workgroups go round robin over 8)
+  int bh, vb;
+  const int whole = bh_count / 8 * 8 * v_blocks;
+  if (static_cast<int>(blockIdx.x) < whole) {
+    const int die = blockIdx.x & 7, i = blockIdx.x >> 3;
+    bh = (i / v_blocks) * 8 + die;
+    vb = i % v_blocks;
+  } else {
+    bh = bh_count / 8 * 8 + (blockIdx.x - whole) / v_blocks;
+    vb = (blockIdx.x - whole) % v_blocks;
+  }
+  const int b = bh / H, h = bh % H, hk = h / (H / kvh);
+  const int wave = threadIdx.x >> 6, c = threadIdx.x & 15, b4 = (threadIdx.x & 63) >> 4;
+  const int col = vb * 16 + c;
+  const bool col_ok = col < DV;
+  float *state = a.state + static_cast<size_t>(bh) * D * DV;
+  const bool carried = a.input_pos[0] > 0;
+  f32x4_t s[OWN];
+#pragma unroll
+  for (int i = 0; i < OWN; ++i) {
+    const int dt = wave + 4 * i;
+    s[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = dt * 16 + 4 * b4 + r;
+      if (carried && d < D && col_ok) s[i][r] = state[static_cast<size_t>(d) * DV + col];
+    }
+    if (dt < DT) store4(st + c * kRow + dt * 16 + 4 * b4, s[i]);
+  }
+  const size_t stride = static_cast<size_t>(kvh) * D;
+  const int tr = 16 * wave + c;
+  for (int chunk = 0; chunk < cs.chunks; ++chunk) {
+    const size_t row0 = static_cast<size_t>(b) * seqlen + static_cast<size_t>(chunk) * kChunk;
+    const int live = seqlen - chunk * kChunk < kChunk ? seqlen - chunk * kChunk : kChunk;
+    const float *kb = p.k + (row0 * kvh + hk) * D, *qb = p.q + (row0 * kvh + hk) * D;
+    const float *tt = cs.t + (static_cast<size_t>(bh) * cs.chunks + chunk) * kChunk * kChunk, *pt = cs.p + (static_cast<size_t>(bh) * cs.chunks + chunk) * kChunk * kChunk;
+    // operands of this wave's rows: independent of the state, so the loads are in flight while the previous chunk ends
+    f32x4_t ka[DT], qa[DT], ta[4], pa[4], kt[OWN][4], v;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      ka[dt] = row4<VEC>(kb + tr * stride, tr < live, dt * 16 + 4 * b4, D);
+      qa[dt] = row4<VEC>(qb + tr * stride, tr < live, dt * 16 + 4 * b4, D);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      ta[j] = pa[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if (j <= wave) {
+        ta[j] = load4(tt + tr * kChunk + 16 * j + 4 * b4);
+        pa[j] = load4(pt + tr * kChunk + 16 * j + 4 * b4);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = 16 * wave + 4 * b4 + r;
+      v[r] = t < live && col_ok ? p.v[((row0 + t) * H + h) * DV + col] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < OWN; ++i) {
+      const int d = (wave + 4 * i) * 16 + c;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = 16 * j + 4 * b4 + r;
+          kt[i][j][r] = t < live && d < D ? kb[t * stride + d] : 0.f;
+        }
+    }
+    float *g = sg[chunk & 1];
+    if (wave == 0) {
+      const int t = threadIdx.x;
+      float x = t < live ? p.log_g[(row0 + t) * H + h] : 0.f;
+#pragma unroll
+      for (int off = 1; off < 64; off <<= 1) {
+        const float up = __shfl_up(x, off);
+        if (t >= off) x += up;
+      }
+      g[t] = x * kLog2e;
+    }
+    __syncthreads();  // the state in LDS and the decays are complete
+    f32x4_t ks = {0.f, 0.f, 0.f, 0.f}, qs = ks;
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      const f32x4_t sb = load4(st + c * kRow + dt * 16 + 4 * b4);
+      ks = mfma4(ka[dt], sb, ks);
+      qs = mfma4(qa[dt], sb, qs);
+    }
+    f32x4_t gt;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      gt[r] = __builtin_amdgcn_exp2f(g[16 * wave + 4 * b4 + r]);
+      sx[(16 * wave + 4 * b4 + r) * kTok + c] = v[r] - gt[r] * ks[r];
+    }
+    __syncthreads();
+    f32x4_t u = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      if (j > wave) break;
+      f32x4_t x;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) x[r] = sx[(16 * j + 4 * b4 + r) * kTok + c];
+      u = mfma4(ta[j], x, u);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) su[(16 * wave + 4 * b4 + r) * kTok + c] = u[r];
+    __syncthreads();
+    f32x4_t o, ub[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) o[r] = gt[r] * qs[r];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) ub[j][r] = su[(16 * j + 4 * b4 + r) * kTok + c];
+      if (j <= wave) o = mfma4(pa[j], ub[j], o);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {  // over the values this workgroup has read
+      const int t = 16 * wave + 4 * b4 + r;
+      if (t < live && col_ok) p.v[((row0 + t) * H + h) * DV + col] = o[r];
+    }
+    const float g_end = g[kChunk - 1], dec = __builtin_amdgcn_exp2f(g_end);
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) ub[j][r] *= __builtin_amdgcn_exp2f(g_end - g[16 * j + 4 * b4 + r]);
+#pragma unroll
+    for (int i = 0; i < OWN; ++i) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) s[i][r] *= dec;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) s[i] = mfma4(kt[i][j], ub[j], s[i]);
+      if (wave + 4 * i < DT) store4(st + c * kRow + (wave + 4 * i) * 16 + 4 * b4, s[i]);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < OWN; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = (wave + 4 * i) * 16 + 4 * b4 + r;
+      if (d < D && col_ok) state[static_cast<size_t>(d) * DV + col] = s[i][r];
+    }
+}
+
+// step 3: one wave per (token, head); the read-outs stand where the values were
+template <typename T>
+__global__ __launch_bounds__(256) void delta_gate_kernel(const e2h_delta_args a, Prepared p) {
+  const int64_t item = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);
+  if (item >= a.batch * a.seqlen * a.heads) return;  // whole waves
+  const int cg = threadIdx.x & 63;
+  const bool mine = cg * 4 < a.vdim;
+  f32x4_t o = {0.f, 0.f, 0.f, 0.f};
+  if (mine) o = load4(p.v + item * a.vdim + cg * 4);
+  gated_norm_store<T>(a, static_cast<size_t>(item / a.heads), static_cast<int>(item % a.heads), cg, mine, o);
+}
+
+bool use_chunks(const e2h_delta_args &a) {
+  if (a.seqlen == 1 || seq_options().recurrence_form == 1) return false;
+  return seq_options().recurrence_form == 2 || a.seqlen >= 24;
+}
+
+template <int DT>
+void launch_scan(const e2h_delta_args &a, const Prepared &p, const ChunkScratch &cs, hipStream_t s) {
+  const int v_blocks = static_cast<int>((a.vdim + 15) / 16);
+  const dim3 grid(static_cast<unsigned>(a.batch * a.heads * v_blocks)), block(256);
+  if (a.dim % 4 == 0) hipLaunchKernelGGL((delta_scan_kernel<DT, true>), grid, block, 0, s, a, p, cs, v_blocks);
+  else hipLaunchKernelGGL((delta_scan_kernel<DT, false>), grid, block, 0, s, a, p, cs, v_blocks);
+}
+
+template <typename T>
+void launch_chunks(const e2h_delta_args &a, const Prepared &p, const ChunkScratch &cs, hipStream_t s) {
+  const dim3 grid(static_cast<unsigned>(a.batch * a.heads * cs.chunks)), block(256);
+  if (a.dim % 4 == 0) hipLaunchKernelGGL(delta_chunk_kernel<true>, grid, block, 0, s, a, p, cs);
+  else hipLaunchKernelGGL(delta_chunk_kernel<false>, grid, block, 0, s, a, p, cs);
+  if (a.dim <= 64) launch_scan<4>(a, p, cs, s);
+  else if (a.dim <= 128) launch_scan<8>(a, p, cs, s);
+  else launch_scan<16>(a, p, cs, s);
+  hipLaunchKernelGGL(delta_gate_kernel<T>, dim3(static_cast<unsigned>((a.batch * a.seqlen * a.heads + 3) / 4)), block, 0, s, a, p);
+}
+
 template <typename T, bool ONE>
 void launch_tokens(const e2h_delta_args &a, const Prepared &p, hipStream_t s) {
   int cp = 1;
@@ -262,7 +582,7 @@ void launch_tokens(const e2h_delta_args &a, const Prepared &p, hipStream_t s) {
 int64_t round256(int64_t n) { return (n + 255) / 256 * 256; }
 
 // scratch layout; returns its size in bytes
-int64_t carve(const e2h_delta_args &a, Prepared *p) {
+int64_t carve(const e2h_delta_args &a, Prepared *p, ChunkScratch *cs) {
   if (a.seqlen == 1) return 0;
   const int64_t rows = a.batch * a.seqlen;
   const int64_t qk = round256(rows * a.kv_heads * a.dim * 4), v = round256(rows * a.heads * a.vdim * 4), g = round256(rows * a.heads * 4);
@@ -274,7 +594,15 @@ int64_t carve(const e2h_delta_args &a, Prepared *p) {
     p->beta = reinterpret_cast<float *>(base + 2 * qk + v);
     p->log_g = reinterpret_cast<float *>(base + 2 * qk + v + g);
   }
-  return 2 * qk + v + 2 * g;
+  const int64_t prepared = 2 * qk + v + 2 * g;
+  if (!use_chunks(a)) return prepared;
+  const int64_t chunks = (a.seqlen + kChunk - 1) / kChunk, squares = a.batch * a.heads * chunks * kChunk * kChunk * 4;
+  if (cs) {
+    cs->t = reinterpret_cast<float *>(static_cast<uint8_t *>(a.scratch) + prepared);
+    cs->p = reinterpret_cast<float *>(static_cast<uint8_t *>(a.scratch) + prepared + squares);
+    cs->chunks = static_cast<int>(chunks);
+  }
+  return prepared + 2 * squares;
 }
 
 template <typename T>
@@ -284,10 +612,12 @@ int launch_delta(const e2h_delta_args &a, hipStream_t s) {
     launch_tokens<T, true>(a, p, s);
     return launch_status();
   }
-  carve(a, &p);
+  ChunkScratch cs = {};
+  carve(a, &p, &cs);
   const int64_t items = a.batch * a.seqlen * (2 * a.kv_heads + a.heads + 1);
   hipLaunchKernelGGL(delta_prepare_kernel<T>, dim3(static_cast<unsigned>((items + 3) / 4)), dim3(256), 0, s, a, p);
-  launch_tokens<T, false>(a, p, s);
+  if (use_chunks(a)) launch_chunks<T>(a, p, cs, s);
+  else launch_tokens<T, false>(a, p, s);
   return launch_status();
 }
 
@@ -300,7 +630,8 @@ bool shape_ok(const e2h_delta_args &a) {
   if (a.q_off + a.kv_heads * a.dim > a.ld || a.k_off + a.kv_heads * a.dim > a.ld || a.v_off + a.heads * a.vdim > a.ld || a.b_off + a.heads > a.ld ||
       a.a_off + a.heads > a.ld || a.g_off + a.heads * a.vdim > a.ld || a.out_off + a.heads * a.vdim > a.ld_out)
     return false;
-  return a.batch * a.heads <= INT32_MAX && a.batch * a.seqlen * (2 * a.kv_heads + a.heads + 1) / 4 < INT32_MAX &&
+  return a.batch * a.heads * ((a.seqlen + kChunk - 1) / kChunk) <= INT32_MAX && a.batch * a.heads * ((a.vdim + 15) / 16) <= INT32_MAX &&
+         a.batch * a.seqlen * (2 * a.kv_heads + a.heads + 1) / 4 < INT32_MAX &&
          2 * a.kv_heads * a.dim + a.heads * a.vdim <= INT32_MAX;
 }
 
@@ -312,7 +643,7 @@ using namespace e2h;
 extern "C" int64_t e2h_seq_delta_scratch_bytes(const e2h_delta_args *a) {
   if (!a) return E2H_ERR_NULL_POINTER;
   if (!shape_ok(*a)) return E2H_ERR_BAD_SHAPE;
-  return carve(*a, nullptr);
+  return carve(*a, nullptr, nullptr);
 }
 
 extern "C" int e2h_seq_delta(const e2h_delta_args *a, void *stream) {
@@ -321,7 +652,7 @@ extern "C" int e2h_seq_delta(const e2h_delta_args *a, void *stream) {
   if (a->taps > 1 && (!a->tail_in || !a->tail_out)) return E2H_ERR_NULL_POINTER;
   if (a->taps > 1 && a->seqlen > 1 && a->tail_in == a->tail_out) return E2H_ERR_BAD_SHAPE;
   if (!aligned16(a->state) || !aligned16(a->scratch)) return E2H_ERR_MISALIGNED;
-  const int64_t need = carve(*a, nullptr);
+  const int64_t need = carve(*a, nullptr, nullptr);
   if (need > 0 && !a->scratch) return E2H_ERR_NULL_POINTER;
   if (need > a->scratch_bytes) return E2H_ERR_SCRATCH_TOO_SMALL;
   if (a->dtype == E2H_SEQ_BF16) return launch_delta<bf16_t>(*a, static_cast<hipStream_t>(stream));
