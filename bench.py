@@ -77,6 +77,11 @@ def parse_args():
                     help="launch floor of this machine for the step's dequant-GEMV launches: a kernel of the library that only reads "
                          "(e2h_stream_read_probe) is launched once per quantized-linear launch of a decode step on as many bytes as that "
                          "launch has to read, from a HIP graph over a rotating region; prints the time per launch size and their sum")
+    ap.add_argument("--refatar", default="", metavar="SIZE", choices=["", "1b", "7b"],
+                    help="instead of the default workload: prefill and decode throughput of the Refatar decoder at layer sizes of a model of "
+                         "this class (random weights, bf16), beside the Llama-family model of equal size; prints one JSON line")
+    ap.add_argument("--refatar-model", default="both", choices=["both", "refatar", "llama"], help="with --refatar: measure only one of the two")
+    ap.add_argument("--refatar-phase", default="both", choices=["both", "prefill", "decode"], help="with --refatar: measure only one phase")
     ap.add_argument("--gemv-only", action="store_true",
                     help="only the back-to-back dequant-GEMV pass plus a 256 MiB calibration copy (for counter runs)")
     return ap.parse_args()
@@ -498,6 +503,14 @@ def main():
     from easy_to_hard_amd.generate import GraphedDecodeStep, prefill
     from easy_to_hard_amd.model import ModelArgs, random_quantized_transformer
 
+    if args.refatar:
+        from easy_to_hard_amd import layer_bench
+
+        _lib.load_seq()
+        assert torch.cuda.is_available(), "bench.py needs the GPU"
+        torch.cuda.set_device(0)
+        print(json.dumps(layer_bench.run(args.refatar, args.refatar_model, args.refatar_phase, torch.device("cuda", 0), min(args.steps, 64))))
+        return
     _lib.load()  # no fallback: fail here if the HIP library is not built
     for item in args.option:
         name, _, value = item.partition("=")

@@ -22,7 +22,7 @@ struct KeyList {  // virtual index n -> key position
 };
 
 // keys of the queries at positions pa .. pb of one sequence
-__device__ __forceinline__ KeyList key_list(int pa, int pb, int first, int64_t window, int64_t keep_first) {
+__device__ __forceinline__ KeyList key_list(int pa, int pb, int first, int window, int keep_first) {
   KeyList k;
   k.first = first;
   if (pb < first) {
@@ -30,17 +30,17 @@ __device__ __forceinline__ KeyList key_list(int pa, int pb, int first, int64_t w
     k.start = first;
     return k;
   }
-  const int64_t live = static_cast<int64_t>(pb) - first + 1;
-  k.kept = static_cast<int>(keep_first < live ? keep_first : live);
-  int64_t lo = window > 0 ? static_cast<int64_t>(pa) - window + 1 : 0;
-  if (lo < first + k.kept) lo = first + k.kept;
-  k.start = static_cast<int>(lo);
-  k.count = k.kept + (lo <= pb ? static_cast<int>(pb - lo) + 1 : 0);
+  const int live = pb - first + 1;
+  k.kept = keep_first < live ? keep_first : live;
+  k.start = pa - window + 1;  // window > 0: no overflow
+  if (k.start < first + k.kept) k.start = first + k.kept;
+  k.count = k.kept + (k.start <= pb ? pb - k.start + 1 : 0);
   return k;
 }
 
-__device__ __forceinline__ bool sees(int i, int j, int first, int64_t window, int64_t keep_first) {
-  return j <= i && j >= first && (window <= 0 || static_cast<int64_t>(i) - j < window || static_cast<int64_t>(j) - first < keep_first);
+// window and keep_first fit 31 bits here, window 0 has become the largest value
+__device__ __forceinline__ bool sees(int i, int j, int first, int window, int keep_first) {
+  return j <= i && j >= first && (i - j < window || j - first < keep_first);
 }
 
 // eight consecutive bfloat16 values starting at p, of which `valid` exist; VEC: 16-byte accesses are aligned and valid is 8 or <= 0
@@ -92,6 +92,29 @@ __global__ __launch_bounds__(256) void kv_append_kernel(const e2h_window_attenti
   dst[((b * a.kv_heads + c / d) * a.cache_len + pos) * d + c % d] = from_f32<T>(v);
 }
 
+// the same for bfloat16, eight values per thread (head sizes and columns multiples of eight)
+__global__ __launch_bounds__(256) void kv_append8_kernel(const e2h_window_attention_args a) {
+  const int kw = static_cast<int>(a.kv_heads * a.dim) / 8, per_row = kw + static_cast<int>(a.kv_heads * a.vdim) / 8;
+  const int64_t idx = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
+  if (idx >= a.batch * a.seqlen * per_row) return;
+  const int row = static_cast<int>(idx / per_row), seqlen = static_cast<int>(a.seqlen);
+  const bool is_k = idx % per_row < kw;
+  const int c = static_cast<int>(idx % per_row - (is_k ? 0 : kw)) * 8;
+  const int64_t b = row / seqlen, pos = a.input_pos[0] + row % seqlen;
+  if (pos < 0 || pos >= a.cache_len) return;
+  const int d = static_cast<int>(is_k ? a.dim : a.vdim);
+  const bf16_t *src = static_cast<const bf16_t *>(a.proj) + row * a.ld + (is_k ? a.k_off : a.v_off) + c;
+  f32x4_t lo = load4(src), hi = load4(src + 4);
+  const float *bias = is_k ? a.k_bias : a.v_bias;
+  if (bias) {
+    lo += load4(bias + c);
+    hi += load4(bias + c + 4);
+  }
+  bf16_t *dst = static_cast<bf16_t *>(is_k ? a.k_cache : a.v_cache) + ((b * a.kv_heads + c / d) * a.cache_len + pos) * d + c % d;
+  store4(dst, lo);
+  store4(dst + 4, hi);
+}
+
 // ---- float32: one wave per (row, head) ------------------------------------------------------------------------------------
 constexpr int kMaxHeadDim = 256;
 
@@ -112,7 +135,7 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(const e2h_window_at
   const T *src = static_cast<const T *>(a.proj) + row * a.ld;
   for (int d = lane; d < D; d += 64) sh_q[wave][d] = to_f32(src[a.q_off + static_cast<int64_t>(h) * D + d]) + (a.q_bias ? a.q_bias[h * D + d] : 0.f);
   const int last = pos < a.cache_len ? pos : static_cast<int>(a.cache_len) - 1;
-  const KeyList kl = key_list(pos, last, first, a.window, a.keep_first);
+  const KeyList kl = key_list(pos, last, first, static_cast<int>(a.window), static_cast<int>(a.keep_first));
   const int count = active ? kl.count : 0;
   const T *kc = static_cast<const T *>(a.k_cache) + (b * a.kv_heads + g) * a.cache_len * D;
   const T *vc = static_cast<const T *>(a.v_cache) + (b * a.kv_heads + g) * a.cache_len * DV;
@@ -126,7 +149,7 @@ __global__ __launch_bounds__(256) void attention_rows_kernel(const e2h_window_at
       const T *kr = kc + static_cast<size_t>(j) * D;
       float dot = 0.f;
       for (int d = 0; d < D; ++d) dot = __builtin_fmaf(sh_q[wave][d], to_f32(kr[d]), dot);
-      if (sees(pos, j, first, a.window, a.keep_first)) s = dot * a.scale;
+      if (sees(pos, j, first, static_cast<int>(a.window), static_cast<int>(a.keep_first))) s = dot * a.scale;
     }
     float mx = s;
 #pragma unroll
@@ -170,16 +193,15 @@ __device__ __forceinline__ void split_weights(const float (&p)[8], bf16x8_t &hi,
   for (int i = 0; i < 4; ++i) {
     const uint32_t a = __builtin_bit_cast(uint32_t, p[2 * i]) & 0xFFFF0000u, b = __builtin_bit_cast(uint32_t, p[2 * i + 1]) & 0xFFFF0000u;
     h[i] = (a >> 16) | b;
-    l[i] = static_cast<uint32_t>(f32_to_bf16_rne(p[2 * i] - __builtin_bit_cast(float, a))) |
-           (static_cast<uint32_t>(f32_to_bf16_rne(p[2 * i + 1] - __builtin_bit_cast(float, b))) << 16);
+    l[i] = pack_bf16(p[2 * i] - __builtin_bit_cast(float, a), p[2 * i + 1] - __builtin_bit_cast(float, b));
   }
   hi = __builtin_bit_cast(bf16x8_t, h);
   lo = __builtin_bit_cast(bf16x8_t, l);
 }
 
-// ---- bfloat16, many tokens: 4 waves x NQ x 16 queries of one head, key tiles of 64 shared through LDS ----------------------
+// ---- bfloat16, many tokens: 4 waves x 16 queries of one head, key tiles of 64 shared through LDS ----------------------
 // KS: head dimension in steps of 32 (zero padded), VT: value dimension in tiles of 16.
-template <int KS, int VT, int NQ, bool VEC>
+template <int KS, int VT, bool VEC>
 __global__ __launch_bounds__(256) void attention_prefill_kernel(const e2h_window_attention_args a, int q_blocks) {
   constexpr int kKeys = 64;
   constexpr int kKRow = KS * 64 + 16;   // bytes per key row (padding spreads the rows over the banks)
@@ -200,39 +222,29 @@ __global__ __launch_bounds__(256) void attention_prefill_kernel(const e2h_window
   const int h = g * rep + r;
   const int pos0 = static_cast<int>(a.input_pos[0]);
   const int first = a.first ? static_cast<int>(a.first[bi]) : 0;
-  const int t0 = qb * (64 * NQ);
-  const int t_last = t0 + 64 * NQ - 1 < seqlen - 1 ? t0 + 64 * NQ - 1 : seqlen - 1;
+  const int t0 = qb * 64;
+  const int t_last = t0 + 63 < seqlen - 1 ? t0 + 63 : seqlen - 1;
   const int cache_last = static_cast<int>(a.cache_len) - 1;
   const int pb = pos0 + t_last < cache_last ? pos0 + t_last : cache_last;
-  const KeyList kl = key_list(pos0 + t0, pb, first, a.window, a.keep_first);
+  const KeyList kl = key_list(pos0 + t0, pb, first, static_cast<int>(a.window), static_cast<int>(a.keep_first));
   const bf16_t *proj = static_cast<const bf16_t *>(a.proj);
   const bf16_t *kc = static_cast<const bf16_t *>(a.k_cache) + (static_cast<size_t>(bi) * a.kv_heads + g) * a.cache_len * D;
   const bf16_t *vc = static_cast<const bf16_t *>(a.v_cache) + (static_cast<size_t>(bi) * a.kv_heads + g) * a.cache_len * DV;
   const size_t row0 = static_cast<size_t>(bi) * seqlen;
 
-  int tq[NQ];
-  bf16x8_t qf[NQ][KS];
+  const int tq = t0 + wave * 16 + c, tc = tq < seqlen ? tq : seqlen - 1;
+  bf16x8_t qf[KS];
 #pragma unroll
-  for (int n = 0; n < NQ; ++n) {
-    tq[n] = t0 + (wave * NQ + n) * 16 + c;
-    const int tc = tq[n] < seqlen ? tq[n] : seqlen - 1;
-#pragma unroll
-    for (int s = 0; s < KS; ++s) {
-      const int d = 32 * s + 8 * b4;
-      u32x4_t raw = load8<VEC>(proj + (row0 + tc) * a.ld + a.q_off + static_cast<int64_t>(h) * D + d, D - d);
-      if (a.q_bias) raw = add_bias8(raw, a.q_bias + static_cast<int64_t>(h) * D + d, D - d);
-      qf[n][s] = __builtin_bit_cast(bf16x8_t, raw);
-    }
+  for (int s = 0; s < KS; ++s) {
+    const int d = 32 * s + 8 * b4;
+    u32x4_t raw = load8<VEC>(proj + (row0 + tc) * a.ld + a.q_off + static_cast<int64_t>(h) * D + d, D - d);
+    if (a.q_bias) raw = add_bias8(raw, a.q_bias + static_cast<int64_t>(h) * D + d, D - d);
+    qf[s] = __builtin_bit_cast(bf16x8_t, raw);
   }
-  f32x4_t oacc[NQ][VT];
-  float m_run[NQ], l_run[NQ];
+  f32x4_t oacc[VT];
+  float m_run = kMasked, l_run = 0.f;
 #pragma unroll
-  for (int n = 0; n < NQ; ++n) {
-    m_run[n] = kMasked;
-    l_run[n] = 0.f;
-#pragma unroll
-    for (int v = 0; v < VT; ++v) oacc[n][v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  }
+  for (int v = 0; v < VT; ++v) oacc[v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   const float sc = a.scale * kLog2e;
 
   constexpr int kKPieces = kKeys * KS * 4, kVPieces = kKeys * VT * 2;  // 16-byte pieces per tile
@@ -274,102 +286,99 @@ __global__ __launch_bounds__(256) void attention_prefill_kernel(const e2h_window
     __syncthreads();
     if (n0 + kKeys < kl.count) fetch(n0 + kKeys);
 
-    f32x4_t st[NQ][4];
+    f32x4_t st[4];
 #pragma unroll
     for (int kt = 0; kt < 4; ++kt) {
-#pragma unroll
-      for (int n = 0; n < NQ; ++n) st[n][kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      st[kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int s = 0; s < KS; ++s) {
         const bf16x8_t kf = *reinterpret_cast<const bf16x8_t *>(sh_k + (16 * kt + c) * kKRow + s * 64 + b4 * 16);
-#pragma unroll
-        for (int n = 0; n < NQ; ++n) st[n][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[n][s], st[n][kt], 0, 0, 0);
+        st[kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], st[kt], 0, 0, 0);
       }
     }
-    // positions of this lane's keys
-    int j[4][4];
+    // a tile inside every query's window needs no masks: whole, behind the kept keys, not beyond the first query, not out of
+    // the last one's window
+    const int q_lo = pos0 + t0 + wave * 16, q_hi = q_lo + 15;
+    const bool open = n0 >= kl.kept && n0 + kKeys <= kl.count && kl.at(n0 + kKeys - 1) <= q_lo && q_hi - kl.at(n0) < static_cast<int>(a.window);
+    if (!__builtin_amdgcn_readfirstlane(open)) {
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int n = n0 + 16 * kt + 4 * b4 + e;
+          const int j = n < kl.count ? kl.at(n) : INT32_MAX;
+          if (!sees(pos0 + tq, j, first, static_cast<int>(a.window), static_cast<int>(a.keep_first))) st[kt][e] = kMasked;
+        }
+    }
+    float mx = st[0][0];
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) mx = fmaxf(mx, st[kt][e]);
+    mx = fmaxf(mx, __shfl_xor(mx, 16));
+    mx = fmaxf(mx, __shfl_xor(mx, 32));
+    const float m_new = fmaxf(m_run, mx);
+    // while a query has seen no key its maximum is the mask value: exponents are then taken against 0, where masked scores give 0
+    const float m_ref = m_new > 0.5f * kMasked ? m_new * sc : 0.f;
+    const float corr = __builtin_amdgcn_exp2f(__builtin_fmaf(m_run, sc, -m_ref));
+    m_run = m_new;
+    float ls = 0.f;
 #pragma unroll
     for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        const int n = n0 + 16 * kt + 4 * b4 + e;
-        j[kt][e] = n < kl.count ? kl.at(n) : INT32_MAX;
+        st[kt][e] = __builtin_amdgcn_exp2f(__builtin_fmaf(st[kt][e], sc, -m_ref));
+        ls += st[kt][e];
       }
+    l_run = l_run * corr + ls;
 #pragma unroll
-    for (int n = 0; n < NQ; ++n) {
-      const int pq = pos0 + tq[n];
-      float mx = kMasked;
+    for (int v = 0; v < VT; ++v)
 #pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const float v = sees(pq, j[kt][e], first, a.window, a.keep_first) ? st[n][kt][e] * sc : kMasked;
-          st[n][kt][e] = v;
-          mx = fmaxf(mx, v);
-        }
-      mx = fmaxf(mx, __shfl_xor(mx, 16));
-      mx = fmaxf(mx, __shfl_xor(mx, 32));
-      const float m_new = fmaxf(m_run[n], mx);
-      const float corr = __builtin_amdgcn_exp2f(m_run[n] - m_new);
-      m_run[n] = m_new;
-      float ls = 0.f;
-#pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const float p = st[n][kt][e] > 0.5f * kMasked ? __builtin_amdgcn_exp2f(st[n][kt][e] - m_new) : 0.f;
-          st[n][kt][e] = p;
-          ls += p;
-        }
-      l_run[n] = l_run[n] * corr + ls;
-#pragma unroll
-      for (int v = 0; v < VT; ++v)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) oacc[n][v][e] *= corr;
-    }
+      for (int e = 0; e < 4; ++e) oacc[v][e] *= corr;
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
-      bf16x8_t hi[NQ], lo[NQ];
+      bf16x8_t hi, lo;
+      float p[8];
 #pragma unroll
-      for (int n = 0; n < NQ; ++n) {
-        float p[8];
-#pragma unroll
-        for (int e = 0; e < 8; ++e) p[e] = st[n][2 * half + (e >> 2)][e & 3];
-        split_weights(p, hi[n], lo[n]);
-      }
+      for (int e = 0; e < 8; ++e) p[e] = st[2 * half + (e >> 2)][e & 3];
+      split_weights(p, hi, lo);
 #pragma unroll
       for (int v = 0; v < VT; ++v) {
         const uint8_t *vp = sh_v + (16 * v + c) * kVRow + half * 64 + b4 * 8;
         const u32x2_t v0 = *reinterpret_cast<const u32x2_t *>(vp), v1 = *reinterpret_cast<const u32x2_t *>(vp + 32);
         const bf16x8_t vf = __builtin_bit_cast(bf16x8_t, u32x4_t{v0[0], v0[1], v1[0], v1[1]});
-#pragma unroll
-        for (int n = 0; n < NQ; ++n) {
-          oacc[n][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[n], oacc[n][v], 0, 0, 0);
-          oacc[n][v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[n], oacc[n][v], 0, 0, 0);
-        }
+        oacc[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi, oacc[v], 0, 0, 0);
+        oacc[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo, oacc[v], 0, 0, 0);
       }
     }
   }
   // lane (b, c): value columns 16 v + 4 b .. + 3 of query c
+  float l = l_run;
+  l += __shfl_xor(l, 16);
+  l += __shfl_xor(l, 32);
+  const float inv = l > 0.f ? a.out_scale / l : 0.f;
+  if (tq >= seqlen) return;
+  const size_t row = row0 + tq;
 #pragma unroll
-  for (int n = 0; n < NQ; ++n) {
-    float l = l_run[n];
-    l += __shfl_xor(l, 16);
-    l += __shfl_xor(l, 32);
-    const float inv = l > 0.f ? a.out_scale / l : 0.f;
-    if (tq[n] >= seqlen) continue;
-    const size_t row = row0 + tq[n];
+  for (int v = 0; v < VT; ++v) {
+    const int d = 16 * v + 4 * b4;
+    f32x4_t o = oacc[v] * inv;
+    const bf16_t *gate = proj + row * a.ld + a.g_off + static_cast<int64_t>(h) * DV + d;
+    bf16_t *dst = static_cast<bf16_t *>(a.out) + row * a.ld_out + a.out_off + static_cast<int64_t>(h) * DV + d;
+    if (VEC) {
+      if (d < DV) {
+        if (a.g_off >= 0) {
+          const f32x4_t g = load4(gate);
 #pragma unroll
-    for (int v = 0; v < VT; ++v)
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-        const int d = 16 * v + 4 * b4 + e;
-        if (d < DV) {
-          float o = oacc[n][v][e] * inv;
-          if (a.g_off >= 0) o *= sigmoid_f32(to_f32(proj[row * a.ld + a.g_off + static_cast<int64_t>(h) * DV + d]));
-          static_cast<bf16_t *>(a.out)[row * a.ld_out + a.out_off + static_cast<int64_t>(h) * DV + d] = f32_to_bf16_rne(o);
+          for (int e = 0; e < 4; ++e) o[e] *= fast_sigmoid(g[e]);
         }
+        store4(dst, o);
       }
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (d + e < DV) dst[e] = from_f32<bf16_t>(a.g_off >= 0 ? o[e] * fast_sigmoid(to_f32(gate[e])) : o[e]);
+    }
   }
 }
 
@@ -401,14 +410,14 @@ __global__ __launch_bounds__(64 * NW) void attention_step_kernel(const e2h_windo
       float v = to_f32(proj[(is_k ? a.k_off : a.v_off) + col]);
       const float *bias = is_k ? a.k_bias : a.v_bias;
       if (bias) v += bias[col];
-      (is_k ? kc + static_cast<size_t>(pos) * D : vc + static_cast<size_t>(pos) * DV)[d] = f32_to_bf16_rne(v);
+      (is_k ? kc + static_cast<size_t>(pos) * D : vc + static_cast<size_t>(pos) * DV)[d] = from_f32<bf16_t>(v);
     }
   }
   __threadfence_block();
   __syncthreads();  // the new row is visible to the workgroup
 
   const int last = pos < a.cache_len ? pos : static_cast<int>(a.cache_len) - 1;
-  const KeyList kl = key_list(pos, last, first, a.window, a.keep_first);
+  const KeyList kl = key_list(pos, last, first, static_cast<int>(a.window), static_cast<int>(a.keep_first));
   bf16x8_t qf[KS];
 #pragma unroll
   for (int s = 0; s < KS; ++s) {
@@ -529,11 +538,16 @@ __global__ __launch_bounds__(64 * NW) void attention_step_kernel(const e2h_windo
     const int col = (g * rep + r) * DV + d;
     o = l > 0.f ? o / l * a.out_scale : 0.f;
     if (a.g_off >= 0) o *= sigmoid_f32(to_f32(proj[a.g_off + col]));
-    static_cast<bf16_t *>(a.out)[static_cast<size_t>(bi) * a.ld_out + a.out_off + col] = f32_to_bf16_rne(o);
+    static_cast<bf16_t *>(a.out)[static_cast<size_t>(bi) * a.ld_out + a.out_off + col] = from_f32<bf16_t>(o);
   }
 }
 
-void launch_append(const e2h_window_attention_args &a, hipStream_t s) {
+void launch_append(const e2h_window_attention_args &a, bool vec, hipStream_t s) {
+  if (vec) {
+    const int64_t n8 = a.batch * a.seqlen * a.kv_heads * (a.dim + a.vdim) / 8;
+    hipLaunchKernelGGL(kv_append8_kernel, dim3(static_cast<unsigned>((n8 + 255) / 256)), dim3(256), 0, s, a);
+    return;
+  }
   const int64_t n = a.batch * a.seqlen * a.kv_heads * (a.dim + a.vdim);
   const dim3 grid(static_cast<unsigned>((n + 255) / 256)), block(256);
   if (a.dtype == E2H_SEQ_BF16) hipLaunchKernelGGL(kv_append_kernel<bf16_t>, grid, block, 0, s, a);
@@ -551,15 +565,9 @@ void launch_mfma(const e2h_window_attention_args &a, hipStream_t s) {
     else hipLaunchKernelGGL((attention_step_kernel<KS, VT, 4, VEC>), grid, dim3(256), 0, s, a);
     return;
   }
-  launch_append(a, s);
-  const int64_t groups = a.batch * a.heads;
-  int nq = seq_options().attention_query_tiles;
-  if (!nq) nq = groups * ((a.seqlen + 127) / 128) >= 512 ? 2 : 1;
-  if (KS > 4) nq = 1;  // the wide heads' accumulators fill the registers with one tile of queries
-  const int q_blocks = static_cast<int>((a.seqlen + 64 * nq - 1) / (64 * nq));
-  const dim3 grid(static_cast<unsigned>(groups * q_blocks)), block(256);
-  if (nq == 2) hipLaunchKernelGGL((attention_prefill_kernel<KS, VT, (KS <= 4 ? 2 : 1), VEC>), grid, block, 0, s, a, q_blocks);
-  else hipLaunchKernelGGL((attention_prefill_kernel<KS, VT, 1, VEC>), grid, block, 0, s, a, q_blocks);
+  launch_append(a, VEC && aligned16(a.k_bias) && aligned16(a.v_bias) && a.k_off % 8 == 0 && a.v_off % 8 == 0, s);
+  const int q_blocks = static_cast<int>((a.seqlen + 63) / 64);
+  hipLaunchKernelGGL((attention_prefill_kernel<KS, VT, VEC>), dim3(static_cast<unsigned>(a.batch * a.heads * q_blocks)), dim3(256), 0, s, a, q_blocks);
 }
 
 template <bool VEC>
@@ -572,7 +580,7 @@ void launch_mfma_by_size(const e2h_window_attention_args &a, hipStream_t s) {
 }
 
 void launch_rows(const e2h_window_attention_args &a, hipStream_t s) {
-  launch_append(a, s);
+  launch_append(a, false, s);
   const dim3 grid(static_cast<unsigned>((a.batch * a.seqlen * a.heads + 3) / 4)), block(256);
   if (a.dtype == E2H_SEQ_BF16) hipLaunchKernelGGL(attention_rows_kernel<bf16_t>, grid, block, 0, s, a);
   else hipLaunchKernelGGL(attention_rows_kernel<float>, grid, block, 0, s, a);
@@ -596,12 +604,17 @@ extern "C" int e2h_seq_window_attention(const e2h_window_attention_args *a, void
   if (a->batch * a->seqlen * a->heads > INT32_MAX || a->batch * a->seqlen * a->kv_heads * (a->dim + a->vdim) / 256 > INT32_MAX - 1)
     return E2H_ERR_BAD_SHAPE;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (a->dtype == E2H_SEQ_F32 || a->heads / a->kv_heads > 16) {
+  e2h_window_attention_args v = *a;
+  const int64_t most = INT32_MAX / 2;  // no limit, as far as any cache reaches
+  v.window = v.window == 0 || v.window > most ? most : v.window;
+  v.keep_first = v.keep_first > most ? most : v.keep_first;
+  a = &v;
+  if (a->dtype == E2H_SEQ_F32 || a->heads / a->kv_heads > 16 || !(a->scale > 0.f)) {
     launch_rows(*a, s);
     return launch_status();
   }
-  const bool vec = a->dim % 8 == 0 && a->vdim % 8 == 0 && a->ld % 8 == 0 && a->q_off % 8 == 0 && aligned16(a->proj) && aligned16(a->k_cache) &&
-                   aligned16(a->v_cache);
+  const bool vec = a->dim % 8 == 0 && a->vdim % 8 == 0 && a->ld % 8 == 0 && a->q_off % 8 == 0 && (a->g_off < 0 || a->g_off % 4 == 0) &&
+                   a->ld_out % 4 == 0 && a->out_off % 4 == 0 && aligned16(a->proj) && aligned16(a->k_cache) && aligned16(a->v_cache) && aligned16(a->out);
   if (vec) launch_mfma_by_size<true>(*a, s);
   else launch_mfma_by_size<false>(*a, s);
   return launch_status();

@@ -11,7 +11,6 @@ struct SeqOptions {
   int recurrence_chunk;        // 0 = heuristic, else tokens per workgroup of the chunked HGRN2 form (multiple of 16)
   int norm_run;                // 0 = heuristic, else tokens per workgroup of the norm kernel
   int attention_decode_waves;  // 0 = by window, else 4 or 8
-  int attention_query_tiles;   // 0 = by token count, else 1 or 2 tiles of 16 queries per wave
 };
 SeqOptions &seq_options();
 
@@ -20,11 +19,17 @@ typedef uint16_t bf16_t;
 
 __device__ __forceinline__ float to_f32(bf16_t v) { return bf16_to_f32(v); }
 __device__ __forceinline__ float to_f32(float v) { return v; }
+// two values rounded to the nearest bfloat16 (one conversion instruction), the first in the low half
+__device__ __forceinline__ uint32_t pack_bf16(float lo, float hi) {
+  typedef float f32x2 __attribute__((ext_vector_type(2)));
+  typedef __bf16 bf16x2 __attribute__((ext_vector_type(2)));
+  return __builtin_bit_cast(uint32_t, __builtin_convertvector(f32x2{lo, hi}, bf16x2));
+}
 template <typename T>
 __device__ __forceinline__ T from_f32(float v);
 template <>
 __device__ __forceinline__ bf16_t from_f32<bf16_t>(float v) {
-  return f32_to_bf16_rne(v);
+  return static_cast<bf16_t>(pack_bf16(v, v));
 }
 template <>
 __device__ __forceinline__ float from_f32<float>(float v) {
@@ -39,10 +44,7 @@ __device__ __forceinline__ f32x4_t load4(const bf16_t *p) {
 }
 __device__ __forceinline__ void store4(float *p, f32x4_t v) { *reinterpret_cast<f32x4_t *>(p) = v; }
 __device__ __forceinline__ void store4(bf16_t *p, f32x4_t v) {
-  u32x2_t r;
-  r[0] = static_cast<uint32_t>(f32_to_bf16_rne(v[0])) | (static_cast<uint32_t>(f32_to_bf16_rne(v[1])) << 16);
-  r[1] = static_cast<uint32_t>(f32_to_bf16_rne(v[2])) | (static_cast<uint32_t>(f32_to_bf16_rne(v[3])) << 16);
-  *reinterpret_cast<u32x2_t *>(p) = r;
+  *reinterpret_cast<u32x2_t *>(p) = u32x2_t{pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3])};
 }
 
 __device__ __forceinline__ float wave_add(float v) {
@@ -61,8 +63,59 @@ __device__ __forceinline__ f32x4_t mfma4(f32x4_t a, f32x4_t b, f32x4_t acc) {
   return acc;
 }
 
+// A decay factor 1 - k as the pair (c1, c2) with decayed(s) = c1 s + c2 s: near one it is s - k s, so that the factor's own rounding
+// does not add up over the tokens of a long memory; elsewhere f s.
+struct Decay {
+  float c1, c2;
+};
+__device__ __forceinline__ Decay decay_of(float f, float k) { return k < 0.5f ? Decay{-k, 1.0f} : Decay{f, 0.0f}; }
+__device__ __forceinline__ float decayed(Decay d, float s) { return __builtin_fmaf(d.c1, s, d.c2 * s); }
+
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
+
+
+// The same on the hardware's exponential and reciprocal (a few units in the last place), for kernels that evaluate them per
+// token and channel of a prompt
+__device__ __forceinline__ float fast_sigmoid(float z) { return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-z * kLog2e)); }
+__device__ __forceinline__ float fast_silu(float z) { return z * fast_sigmoid(z); }
+// log2(1 - k), 0 <= k <= 1, f = 1 - k given as well: below one half by the series of the inverse hyperbolic tangent,
+// log(1 - k) = -2 atanh(k / (2 - k)), so that small k keep their relative accuracy
+__device__ __forceinline__ float log2_one_minus(float k, float f) {
+  const float s = k * __builtin_amdgcn_rcpf(2.0f - k), s2 = s * s;
+  float p = 1.0f / 15.0f;
+  p = __builtin_fmaf(p, s2, 1.0f / 13.0f);
+  p = __builtin_fmaf(p, s2, 1.0f / 11.0f);
+  p = __builtin_fmaf(p, s2, 1.0f / 9.0f);
+  p = __builtin_fmaf(p, s2, 1.0f / 7.0f);
+  p = __builtin_fmaf(p, s2, 1.0f / 5.0f);
+  p = __builtin_fmaf(p, s2, 1.0f / 3.0f);
+  p = __builtin_fmaf(p * s2, s, s);
+  return k < 0.5f ? p * (-2.0f * kLog2e) : __builtin_amdgcn_logf(fmaxf(f, 1e-37f));
+}
+
+// unpacked or raw four activations, for loads that are issued well before they are used
+template <typename T>
+struct Quad;
+template <>
+struct Quad<float> {
+  f32x4_t raw;
+  __device__ __forceinline__ f32x4_t f32() const { return raw; }
+};
+template <>
+struct Quad<bf16_t> {
+  u32x2_t raw;
+  __device__ __forceinline__ f32x4_t f32() const {
+    return f32x4_t{__builtin_bit_cast(float, raw[0] << 16), __builtin_bit_cast(float, raw[0] & 0xFFFF0000u), __builtin_bit_cast(float, raw[1] << 16),
+                   __builtin_bit_cast(float, raw[1] & 0xFFFF0000u)};
+  }
+};
+template <typename T>
+__device__ __forceinline__ Quad<T> load_quad(const T *p) {
+  Quad<T> q;
+  q.raw = *reinterpret_cast<const decltype(q.raw) *>(p);
+  return q;
+}
 
 }  // namespace e2h

@@ -108,6 +108,99 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(const e2h_delta_args
   }
 }
 
+// The same for convolutions of up to four taps with everything in multiples of four channels: `cp` lanes (a power of two) hold
+// one head's channels, four each, and walk kPrepareRun tokens with the previous inputs in registers.
+constexpr int kPrepareRun = 8;
+
+template <typename T>
+__global__ __launch_bounds__(256) void delta_prepare4_kernel(const e2h_delta_args a, Prepared o, int cp, int runs) {
+  const int kvh = static_cast<int>(a.kv_heads), H = static_cast<int>(a.heads), D = static_cast<int>(a.dim), DV = static_cast<int>(a.vdim);
+  const int heads = 2 * kvh + H, per_wave = 64 / cp, groups = (heads + per_wave - 1) / per_wave, seqlen = static_cast<int>(a.seqlen), taps = a.taps;
+  const int lane = threadIdx.x & 63;
+  const int64_t item = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);  // (sequence, run, group of heads)
+  if (item >= a.batch * runs * groups) return;  // whole waves
+  const int u = static_cast<int>(item % groups) * per_wave + lane / cp;
+  const int64_t br = item / groups;
+  const int b = static_cast<int>(br / runs), t_begin = static_cast<int>(br % runs) * kPrepareRun;
+  const int t_end = t_begin + kPrepareRun < seqlen ? t_begin + kPrepareRun : seqlen;
+  const bool is_q = u < kvh, is_k = !is_q && u < 2 * kvh;
+  const int head = is_q ? u : is_k ? u - kvh : u - 2 * kvh, n = is_q || is_k ? D : DV, d = (lane & (cp - 1)) * 4;
+  const bool mine = u < heads && d < n;
+  const int ch = mine ? (is_q ? head * D : is_k ? (kvh + head) * D : 2 * kvh * D + head * DV) + d : 0;
+  const int64_t col = mine ? (is_q ? a.q_off : is_k ? a.k_off : a.v_off) + static_cast<int64_t>(head) * n + d : a.q_off;
+  const int64_t pos0 = a.input_pos[0], first = a.first ? a.first[b] : 0;
+  const int channels = 2 * kvh * D + H * DV;
+  const size_t row0 = static_cast<size_t>(b) * seqlen;
+  const T *src = static_cast<const T *>(a.proj) + row0 * a.ld + col;
+  const T *tail = static_cast<const T *>(a.tail_in) + static_cast<size_t>(b) * taps * channels + ch;
+  const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
+  f32x4_t w[4];  // shallower convolutions: zero weights in front
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    w[j] = zero;
+    const int jj = j - (4 - taps);
+    if (jj >= 0) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) w[j][e] = a.conv[static_cast<size_t>(ch + e) * taps + jj];
+    }
+  }
+  Quad<T> x[kPrepareRun + 3];
+  bool there[kPrepareRun + 3];
+#pragma unroll
+  for (int i = 0; i < kPrepareRun + 3; ++i) {
+    const int t = t_begin - 3 + i;
+    const int64_t pos = pos0 + t;
+    there[i] = pos >= first && pos >= 0 && t >= -(taps - 1);
+    if (t >= 0) x[i] = load_quad(src + static_cast<int64_t>(t < seqlen ? t : seqlen - 1) * a.ld);
+    else x[i] = load_quad(there[i] ? tail + (pos % taps) * channels : src);
+  }
+#pragma unroll
+  for (int i = 0; i < kPrepareRun; ++i) {
+    const int t = t_begin + i;
+    if (t >= t_end) break;
+    f32x4_t y = zero;
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (there[i + j]) {
+        const f32x4_t v = x[i + j].f32();
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y[e] = __builtin_fmaf(w[j][e], v[e], y[e]);
+      }
+    float ss = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      y[e] = mine ? fast_silu(y[e]) : 0.f;
+      ss = __builtin_fmaf(y[e], y[e], ss);
+    }
+    for (int off = 1; off < cp; off <<= 1) ss += __shfl_xor(ss, off);
+    if (is_q || is_k) y *= is_q ? 1.0f / (sqrtf(ss + kUnitEps) * sqrtf(static_cast<float>(D))) : 1.0f / sqrtf(ss + kUnitEps);
+    const size_t row = row0 + t;
+    if (mine) store4(is_q ? o.q + (row * kvh + head) * D + d : is_k ? o.k + (row * kvh + head) * D + d : o.v + (row * H + head) * DV + d, y);
+  }
+  if (taps > 1 && t_end == seqlen && mine) {  // the last taps - 1 inputs, some of them carried over when the call is that short
+    T *dst = static_cast<T *>(a.tail_out) + static_cast<size_t>(b) * taps * channels + ch;
+#pragma unroll
+    for (int i = 0; i < kPrepareRun + 3; ++i) {
+      const int t = t_begin - 3 + i;
+      if (t < t_end && t >= t_end - (taps - 1) && pos0 + t >= 0)
+        *reinterpret_cast<decltype(x[i].raw) *>(dst + ((pos0 + t) % taps) * channels) = x[i].raw;
+    }
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void delta_gates_kernel(const e2h_delta_args a, Prepared o) {
+  const int H = static_cast<int>(a.heads);
+  const int64_t i = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
+  if (i >= a.batch * a.seqlen * H) return;
+  const int64_t row = i / H;
+  const int h = static_cast<int>(i % H);
+  const bool live = a.input_pos[0] + row % a.seqlen >= (a.first ? a.first[row / a.seqlen] : 0);
+  const T *src = static_cast<const T *>(a.proj) + row * a.ld;
+  o.beta[i] = live ? sigmoid_f32(to_f32(src[a.b_off + h])) : 0.f;
+  o.log_g[i] = live ? delta_log_decay(to_f32(src[a.a_off + h]), a.a_log[h], a.dt_bias[h]) : 0.f;
+}
+
 // RMS norm over the head, norm weight and silu gate of one head's read-out; four columns per lane of wave 0
 template <typename T>
 __device__ __forceinline__ void gated_norm_store(const e2h_delta_args &a, size_t row, int h, int cg, bool mine, f32x4_t o) {
@@ -144,7 +237,7 @@ __global__ __launch_bounds__(BLOCK) void delta_tokens_kernel(const e2h_delta_arg
   const T *proj = static_cast<const T *>(a.proj);
   for (int t = 0; t < seqlen; ++t) {
     const size_t row = static_cast<size_t>(b) * seqlen + t;
-    float g, beta;
+    float log_g, beta;
     if (ONE) {
       const int channels = 2 * kvh * D + H * DV;
       float qs = 0.f, ks = 0.f;
@@ -188,7 +281,7 @@ __global__ __launch_bounds__(BLOCK) void delta_tokens_kernel(const e2h_delta_arg
         sh_k[i] *= ks;
       }
       const bool live = pos0 >= first;
-      g = live ? expf(delta_log_decay(to_f32(proj[row * a.ld + a.a_off + h]), a.a_log[h], a.dt_bias[h])) : 1.f;
+      log_g = live ? delta_log_decay(to_f32(proj[row * a.ld + a.a_off + h]), a.a_log[h], a.dt_bias[h]) : 0.f;
       beta = live ? sigmoid_f32(to_f32(proj[row * a.ld + a.b_off + h])) : 0.f;
     } else {
       for (int i = threadIdx.x; i < D; i += BLOCK) {
@@ -196,10 +289,11 @@ __global__ __launch_bounds__(BLOCK) void delta_tokens_kernel(const e2h_delta_arg
         sh_k[i] = p.k[(row * kvh + hk) * D + i];
       }
       for (int i = threadIdx.x; i < DV; i += BLOCK) sh_v[i] = p.v[(row * H + h) * DV + i];
-      g = expf(p.log_g[row * H + h]);
+      log_g = p.log_g[row * H + h];
       beta = p.beta[row * H + h];
     }
     __syncthreads();
+    const Decay g = decay_of(expf(log_g), -expm1f(log_g));
     // both read-outs of the decayed state in one pass: (S + k u^T)^T q = S^T q + (k . q) u
     f32x4_t ak = {0.f, 0.f, 0.f, 0.f}, aq = ak;
 #pragma unroll
@@ -209,7 +303,7 @@ __global__ __launch_bounds__(BLOCK) void delta_tokens_kernel(const e2h_delta_arg
         const float k = sh_k[r], q = sh_q[r];
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          s[i][e] *= g;
+          s[i][e] = decayed(g, s[i][e]);
           ak[e] = __builtin_fmaf(k, s[i][e], ak[e]);
           aq[e] = __builtin_fmaf(q, s[i][e], aq[e]);
         }
@@ -267,24 +361,12 @@ struct ChunkScratch {
   int chunks;
 };
 
-// four consecutive values of row `row` at column d; zero beyond the row's n values or when the row does not exist
+// four consecutive values of a row at column d; zero beyond the row's n values (n % 4 == 0) or when the row does not exist
 __device__ __forceinline__ f32x4_t row4(const float *base, bool exists, int d, int n) {
-  f32x4_t v = {0.f, 0.f, 0.f, 0.f};
-  if (exists) {
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-      if (d + e < n) v[e] = base[d + e];
-  }
-  return v;
-}
-template <bool VEC>
-__device__ __forceinline__ f32x4_t row4(const float *base, bool exists, int d, int n) {
-  if (!VEC) return row4(base, exists, d, n);
-  return exists && d < n ? load4(base + d) : f32x4_t{0.f, 0.f, 0.f, 0.f};  // n % 4 == 0
+  return exists && d < n ? load4(base + d) : f32x4_t{0.f, 0.f, 0.f, 0.f};
 }
 
 // step 1: 4 waves, one (sequence, head, chunk) each; wave w owns the token rows 16 w .. 16 w + 15
-template <bool VEC>
 __global__ __launch_bounds__(256) void delta_chunk_kernel(const e2h_delta_args a, Prepared p, ChunkScratch cs) {
   constexpr int kRow = kChunk + 4;
   __shared__ __attribute__((aligned(16))) float sm[kChunk * kRow];  // M, then its blocks are replaced by the inverse's
@@ -316,11 +398,11 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(const e2h_delta_args a
   const float *kb = p.k + (row0 * kvh + hk) * D, *qb = p.q + (row0 * kvh + hk) * D;
   const int tr = 16 * wave + c;
   for (int d = 4 * b4; d < (D + 15) / 16 * 16; d += 16) {
-    const f32x4_t ka = row4<VEC>(kb + tr * stride, tr < live, d, D), qa = row4<VEC>(qb + tr * stride, tr < live, d, D);
+    const f32x4_t ka = row4(kb + tr * stride, tr < live, d, D), qa = row4(qb + tr * stride, tr < live, d, D);
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       if (j > wave) break;
-      const f32x4_t kc = j == wave ? ka : row4<VEC>(kb + (16 * j + c) * stride, 16 * j + c < live, d, D);
+      const f32x4_t kc = j == wave ? ka : row4(kb + (16 * j + c) * stride, 16 * j + c < live, d, D);
       kk[j] = mfma4(ka, kc, kk[j]);
       qk[j] = mfma4(qa, kc, qk[j]);
     }
@@ -379,13 +461,25 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(const e2h_delta_args a
   }
 }
 
+// What one wave of the scan reads of a chunk: its 16 token rows of k, q, T and the decayed q k^T, its values and, in wave 0, the
+// decays.  None of it depends on the state, so it is fetched a chunk ahead.
+template <int DT>
+struct ChunkRows {
+  f32x4_t k[DT], q[DT], t[4], p[4], v;
+  float log_g;
+};
+
 // step 2: DT = head dimension in tiles of 16.  Four waves; wave w owns the token rows 16 w .. 16 w + 15 of every chunk and the
 // state's row tiles w, w + 4, ...  The state is kept twice: in accumulators by its owner, and in LDS, transposed, as the B
-// operand of everybody's read-outs.
-template <int DT, bool VEC>
-__global__ __launch_bounds__(256) void delta_scan_kernel(const e2h_delta_args a, Prepared p, ChunkScratch cs, int v_blocks) {
-  constexpr int DP = DT * 16, OWN = (DT + 3) / 4, kRow = DP + 4, kTok = 20;
+// operand of everybody's read-outs.  The keys go through LDS once to be read transposed in the state update.
+// WHOLE: the head dimension fills its tiles, so no load needs a mask (rows past the end are read from the last token: their beta is
+// 0, which keeps them out of u, and their outputs are not stored).
+template <int DT, bool WHOLE>
+__global__ __launch_bounds__(256, 1) void delta_scan_kernel(const e2h_delta_args a, Prepared p, ChunkScratch cs, int v_blocks) {
+  constexpr int DP = DT * 16, OWN = DT / 4, kRow = DP + 4, kTok = 20;
+  constexpr bool kAhead = DT <= 8;  // wider heads leave no registers for the next chunk
   __shared__ __attribute__((aligned(16))) float st[16 * kRow];                       // state, [value column][row]
+  __shared__ __attribute__((aligned(16))) float sk[kChunk * kRow];                   // keys, [token][channel]
   __shared__ __attribute__((aligned(16))) float sx[kChunk * kTok], su[kChunk * kTok];  // [token][value column]
   __shared__ float sg[2][kChunk];
   const int D = static_cast<int>(a.dim), DV = static_cast<int>(a.vdim), H = static_cast<int>(a.heads), kvh = static_cast<int>(a.kv_heads);
@@ -402,7 +496,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const e2h_delta_args a,
     vb = (blockIdx.x - whole) % v_blocks;
   }
   const int b = bh / H, h = bh % H, hk = h / (H / kvh);
-  const int wave = threadIdx.x >> 6, c = threadIdx.x & 15, b4 = (threadIdx.x & 63) >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), c = threadIdx.x & 15, b4 = (threadIdx.x & 63) >> 4;
   const int col = vb * 16 + c;
   const bool col_ok = col < DV;
   float *state = a.state + static_cast<size_t>(bh) * D * DV;
@@ -417,72 +511,70 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const e2h_delta_args a,
       const int d = dt * 16 + 4 * b4 + r;
       if (carried && d < D && col_ok) s[i][r] = state[static_cast<size_t>(d) * DV + col];
     }
-    if (dt < DT) store4(st + c * kRow + dt * 16 + 4 * b4, s[i]);
+    store4(st + c * kRow + dt * 16 + 4 * b4, s[i]);
   }
   const size_t stride = static_cast<size_t>(kvh) * D;
   const int tr = 16 * wave + c;
-  for (int chunk = 0; chunk < cs.chunks; ++chunk) {
-    const size_t row0 = static_cast<size_t>(b) * seqlen + static_cast<size_t>(chunk) * kChunk;
+  const size_t seq0 = static_cast<size_t>(b) * seqlen;
+  const float *squares_t = cs.t + static_cast<size_t>(bh) * cs.chunks * kChunk * kChunk, *squares_p = cs.p + static_cast<size_t>(bh) * cs.chunks * kChunk * kChunk;
+
+  auto fetch = [&](int chunk, ChunkRows<DT> &x) {
+    const size_t row0 = seq0 + static_cast<size_t>(chunk) * kChunk;
     const int live = seqlen - chunk * kChunk < kChunk ? seqlen - chunk * kChunk : kChunk;
     const float *kb = p.k + (row0 * kvh + hk) * D, *qb = p.q + (row0 * kvh + hk) * D;
-    const float *tt = cs.t + (static_cast<size_t>(bh) * cs.chunks + chunk) * kChunk * kChunk, *pt = cs.p + (static_cast<size_t>(bh) * cs.chunks + chunk) * kChunk * kChunk;
-    // operands of this wave's rows: independent of the state, so the loads are in flight while the previous chunk ends
-    f32x4_t ka[DT], qa[DT], ta[4], pa[4], kt[OWN][4], v;
+    const float *tt = squares_t + static_cast<size_t>(chunk) * kChunk * kChunk, *pt = squares_p + static_cast<size_t>(chunk) * kChunk * kChunk;
+    const size_t mine = (tr < live ? tr : live - 1) * stride;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
-      ka[dt] = row4<VEC>(kb + tr * stride, tr < live, dt * 16 + 4 * b4, D);
-      qa[dt] = row4<VEC>(qb + tr * stride, tr < live, dt * 16 + 4 * b4, D);
+      const int d = dt * 16 + 4 * b4;
+      x.k[dt] = WHOLE ? load4(kb + mine + d) : row4(kb + mine, true, d, D);
+      x.q[dt] = WHOLE ? load4(qb + mine + d) : row4(qb + mine, true, d, D);
     }
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      ta[j] = pa[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int j = 0; j < 4; ++j)
       if (j <= wave) {
-        ta[j] = load4(tt + tr * kChunk + 16 * j + 4 * b4);
-        pa[j] = load4(pt + tr * kChunk + 16 * j + 4 * b4);
+        x.t[j] = load4(tt + tr * kChunk + 16 * j + 4 * b4);
+        x.p[j] = load4(pt + tr * kChunk + 16 * j + 4 * b4);
       }
-    }
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int t = 16 * wave + 4 * b4 + r;
-      v[r] = t < live && col_ok ? p.v[((row0 + t) * H + h) * DV + col] : 0.f;
+      x.v[r] = p.v[((row0 + (t < live ? t : live - 1)) * H + h) * DV + (col_ok ? col : 0)];
     }
-#pragma unroll
-    for (int i = 0; i < OWN; ++i) {
-      const int d = (wave + 4 * i) * 16 + c;
-#pragma unroll
-      for (int j = 0; j < 4; ++j)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int t = 16 * j + 4 * b4 + r;
-          kt[i][j][r] = t < live && d < D ? kb[t * stride + d] : 0.f;
-        }
-    }
+    if (wave == 0) x.log_g = p.log_g[(row0 + (static_cast<int>(threadIdx.x) < live ? threadIdx.x : live - 1)) * H + h];
+  };
+
+  ChunkRows<DT> cur, next;
+  fetch(0, cur);
+  for (int chunk = 0; chunk < cs.chunks; ++chunk) {
     float *g = sg[chunk & 1];
     if (wave == 0) {
-      const int t = threadIdx.x;
-      float x = t < live ? p.log_g[(row0 + t) * H + h] : 0.f;
+      float x = static_cast<int>(threadIdx.x) < seqlen - chunk * kChunk ? cur.log_g : 0.f;
 #pragma unroll
       for (int off = 1; off < 64; off <<= 1) {
         const float up = __shfl_up(x, off);
-        if (t >= off) x += up;
+        if (static_cast<int>(threadIdx.x) >= off) x += up;
       }
-      g[t] = x * kLog2e;
+      g[threadIdx.x] = x * kLog2e;
     }
-    __syncthreads();  // the state in LDS and the decays are complete
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) store4(sk + tr * kRow + dt * 16 + 4 * b4, cur.k[dt]);
+    if (kAhead && chunk + 1 < cs.chunks) fetch(chunk + 1, next);
+    lds_barrier();  // state, keys and decays of this chunk are in LDS; the loads above stay in flight
     f32x4_t ks = {0.f, 0.f, 0.f, 0.f}, qs = ks;
 #pragma unroll
     for (int dt = 0; dt < DT; ++dt) {
       const f32x4_t sb = load4(st + c * kRow + dt * 16 + 4 * b4);
-      ks = mfma4(ka[dt], sb, ks);
-      qs = mfma4(qa[dt], sb, qs);
+      ks = mfma4(cur.k[dt], sb, ks);
+      qs = mfma4(cur.q[dt], sb, qs);
     }
     f32x4_t gt;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       gt[r] = __builtin_amdgcn_exp2f(g[16 * wave + 4 * b4 + r]);
-      sx[(16 * wave + 4 * b4 + r) * kTok + c] = v[r] - gt[r] * ks[r];
+      sx[(16 * wave + 4 * b4 + r) * kTok + c] = cur.v[r] - gt[r] * ks[r];
     }
-    __syncthreads();
+    lds_barrier();
     f32x4_t u = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
@@ -490,11 +582,11 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const e2h_delta_args a,
       f32x4_t x;
 #pragma unroll
       for (int r = 0; r < 4; ++r) x[r] = sx[(16 * j + 4 * b4 + r) * kTok + c];
-      u = mfma4(ta[j], x, u);
+      u = mfma4(cur.t[j], x, u);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r) su[(16 * wave + 4 * b4 + r) * kTok + c] = u[r];
-    __syncthreads();
+    lds_barrier();
     f32x4_t o, ub[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) o[r] = gt[r] * qs[r];
@@ -502,12 +594,13 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const e2h_delta_args a,
     for (int j = 0; j < 4; ++j) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) ub[j][r] = su[(16 * j + 4 * b4 + r) * kTok + c];
-      if (j <= wave) o = mfma4(pa[j], ub[j], o);
+      if (j <= wave) o = mfma4(cur.p[j], ub[j], o);
     }
+    const int live = seqlen - chunk * kChunk < kChunk ? seqlen - chunk * kChunk : kChunk;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {  // over the values this workgroup has read
       const int t = 16 * wave + 4 * b4 + r;
-      if (t < live && col_ok) p.v[((row0 + t) * H + h) * DV + col] = o[r];
+      if (t < live && col_ok) p.v[((seq0 + static_cast<size_t>(chunk) * kChunk + t) * H + h) * DV + col] = o[r];
     }
     const float g_end = g[kChunk - 1], dec = __builtin_amdgcn_exp2f(g_end);
 #pragma unroll
@@ -519,9 +612,17 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const e2h_delta_args a,
 #pragma unroll
       for (int r = 0; r < 4; ++r) s[i][r] *= dec;
 #pragma unroll
-      for (int j = 0; j < 4; ++j) s[i] = mfma4(kt[i][j], ub[j], s[i]);
-      if (wave + 4 * i < DT) store4(st + c * kRow + (wave + 4 * i) * 16 + 4 * b4, s[i]);
+      for (int j = 0; j < 4; ++j) {
+        f32x4_t kt;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) kt[r] = sk[(16 * j + 4 * b4 + r) * kRow + (wave + 4 * i) * 16 + c];
+        s[i] = mfma4(kt, ub[j], s[i]);
+      }
+      store4(st + c * kRow + (wave + 4 * i) * 16 + 4 * b4, s[i]);
     }
+    lds_barrier();  // the keys have been read; the next chunk's take their place
+    if (kAhead) cur = next;
+    else if (chunk + 1 < cs.chunks) fetch(chunk + 1, cur);
   }
 #pragma unroll
   for (int i = 0; i < OWN; ++i)
@@ -532,20 +633,40 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const e2h_delta_args a,
     }
 }
 
-// step 3: one wave per (token, head); the read-outs stand where the values were
+// step 3: `cp` lanes per (token, head), four columns each; the read-outs stand where the values were
 template <typename T>
-__global__ __launch_bounds__(256) void delta_gate_kernel(const e2h_delta_args a, Prepared p) {
-  const int64_t item = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);
-  if (item >= a.batch * a.seqlen * a.heads) return;  // whole waves
-  const int cg = threadIdx.x & 63;
-  const bool mine = cg * 4 < a.vdim;
-  f32x4_t o = {0.f, 0.f, 0.f, 0.f};
-  if (mine) o = load4(p.v + item * a.vdim + cg * 4);
-  gated_norm_store<T>(a, static_cast<size_t>(item / a.heads), static_cast<int>(item % a.heads), cg, mine, o);
+__global__ __launch_bounds__(256) void delta_gate_kernel(const e2h_delta_args a, Prepared p, int cp) {
+  const int64_t item = (static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x) / cp;
+  const int d = static_cast<int>(threadIdx.x & (cp - 1)) * 4, DV = static_cast<int>(a.vdim), H = static_cast<int>(a.heads);
+  const bool mine = d < DV && item < a.batch * a.seqlen * H;
+  const int64_t row = mine ? item / H : 0;
+  const int h = mine ? static_cast<int>(item % H) : 0, dc = mine ? d : 0;
+  const f32x4_t o = load4(p.v + (row * H + h) * DV + dc), w = load4(a.norm_weight + dc);
+  const f32x4_t gate = load4(static_cast<const T *>(a.proj) + row * a.ld + a.g_off + static_cast<int64_t>(h) * DV + dc);
+  float ss = mine ? o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3] : 0.f;
+  for (int off = 1; off < cp; off <<= 1) ss += __shfl_xor(ss, off);
+  const float inv = a.out_scale / sqrtf(ss / static_cast<float>(DV) + a.eps);
+  if (!mine) return;
+  f32x4_t y;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) y[e] = o[e] * inv * w[e] * fast_silu(gate[e]);
+  store4(static_cast<T *>(a.out) + row * a.ld_out + a.out_off + static_cast<int64_t>(h) * DV + d, y);
+}
+
+int lanes_for(int64_t values) {  // power of two, four values per lane
+  int cp = 1;
+  while (cp * 4 < values) cp *= 2;
+  return cp;
+}
+
+// four channels per access everywhere
+bool quads_ok(const e2h_delta_args &a) {
+  return a.dim % 4 == 0 && a.ld % 4 == 0 && a.q_off % 4 == 0 && a.k_off % 4 == 0 && a.v_off % 4 == 0 && a.g_off % 4 == 0 && a.ld_out % 4 == 0 &&
+         a.out_off % 4 == 0 && aligned16(a.proj) && aligned16(a.tail_in) && aligned16(a.tail_out) && aligned16(a.out) && aligned16(a.norm_weight);
 }
 
 bool use_chunks(const e2h_delta_args &a) {
-  if (a.seqlen == 1 || seq_options().recurrence_form == 1) return false;
+  if (a.seqlen == 1 || seq_options().recurrence_form == 1 || !quads_ok(a)) return false;
   return seq_options().recurrence_form == 2 || a.seqlen >= 24;
 }
 
@@ -553,19 +674,19 @@ template <int DT>
 void launch_scan(const e2h_delta_args &a, const Prepared &p, const ChunkScratch &cs, hipStream_t s) {
   const int v_blocks = static_cast<int>((a.vdim + 15) / 16);
   const dim3 grid(static_cast<unsigned>(a.batch * a.heads * v_blocks)), block(256);
-  if (a.dim % 4 == 0) hipLaunchKernelGGL((delta_scan_kernel<DT, true>), grid, block, 0, s, a, p, cs, v_blocks);
+  if (a.dim == DT * 16) hipLaunchKernelGGL((delta_scan_kernel<DT, true>), grid, block, 0, s, a, p, cs, v_blocks);
   else hipLaunchKernelGGL((delta_scan_kernel<DT, false>), grid, block, 0, s, a, p, cs, v_blocks);
 }
 
 template <typename T>
 void launch_chunks(const e2h_delta_args &a, const Prepared &p, const ChunkScratch &cs, hipStream_t s) {
   const dim3 grid(static_cast<unsigned>(a.batch * a.heads * cs.chunks)), block(256);
-  if (a.dim % 4 == 0) hipLaunchKernelGGL(delta_chunk_kernel<true>, grid, block, 0, s, a, p, cs);
-  else hipLaunchKernelGGL(delta_chunk_kernel<false>, grid, block, 0, s, a, p, cs);
+  hipLaunchKernelGGL(delta_chunk_kernel, grid, block, 0, s, a, p, cs);
   if (a.dim <= 64) launch_scan<4>(a, p, cs, s);
   else if (a.dim <= 128) launch_scan<8>(a, p, cs, s);
   else launch_scan<16>(a, p, cs, s);
-  hipLaunchKernelGGL(delta_gate_kernel<T>, dim3(static_cast<unsigned>((a.batch * a.seqlen * a.heads + 3) / 4)), block, 0, s, a, p);
+  const int cp = lanes_for(a.vdim);
+  hipLaunchKernelGGL(delta_gate_kernel<T>, dim3(static_cast<unsigned>((a.batch * a.seqlen * a.heads * cp + 255) / 256)), block, 0, s, a, p, cp);
 }
 
 template <typename T, bool ONE>
@@ -614,8 +735,15 @@ int launch_delta(const e2h_delta_args &a, hipStream_t s) {
   }
   ChunkScratch cs = {};
   carve(a, &p, &cs);
-  const int64_t items = a.batch * a.seqlen * (2 * a.kv_heads + a.heads + 1);
-  hipLaunchKernelGGL(delta_prepare_kernel<T>, dim3(static_cast<unsigned>((items + 3) / 4)), dim3(256), 0, s, a, p);
+  if (a.taps <= 4 && quads_ok(a)) {
+    const int cp = lanes_for(a.dim > a.vdim ? a.dim : a.vdim), runs = static_cast<int>((a.seqlen + kPrepareRun - 1) / kPrepareRun);
+    const int64_t waves = a.batch * runs * ((2 * a.kv_heads + a.heads + 64 / cp - 1) / (64 / cp));
+    hipLaunchKernelGGL(delta_prepare4_kernel<T>, dim3(static_cast<unsigned>((waves + 3) / 4)), dim3(256), 0, s, a, p, cp, runs);
+    hipLaunchKernelGGL(delta_gates_kernel<T>, dim3(static_cast<unsigned>((a.batch * a.seqlen * a.heads + 255) / 256)), dim3(256), 0, s, a, p);
+  } else {
+    const int64_t items = a.batch * a.seqlen * (2 * a.kv_heads + a.heads + 1);
+    hipLaunchKernelGGL(delta_prepare_kernel<T>, dim3(static_cast<unsigned>((items + 3) / 4)), dim3(256), 0, s, a, p);
+  }
   if (use_chunks(a)) launch_chunks<T>(a, p, cs, s);
   else launch_tokens<T, false>(a, p, s);
   return launch_status();

@@ -31,7 +31,8 @@ __device__ __forceinline__ Gate hgrn_gate(float z, float low) {
 
 template <typename T, int BLOCK, int RPT>
 __global__ __launch_bounds__(BLOCK) void hgrn2_tokens_kernel(const e2h_hgrn2_args a, int cp) {
-  __shared__ float sh_q[kMaxDim], sh_f[kMaxDim], sh_k[kMaxDim];
+  __shared__ float sh_q[kMaxDim], sh_k[kMaxDim];
+  __shared__ Decay sh_f[kMaxDim];
   __shared__ __attribute__((aligned(16))) float sh_v[kMaxDim];
   __shared__ __attribute__((aligned(16))) f32x4_t part[BLOCK];
   const int D = static_cast<int>(a.dim), DV = static_cast<int>(a.vdim), seqlen = static_cast<int>(a.seqlen);
@@ -56,7 +57,7 @@ __global__ __launch_bounds__(BLOCK) void hgrn2_tokens_kernel(const e2h_hgrn2_arg
       const int ch = h * D + i;
       const Gate g = hgrn_gate(to_f32(src[a.f_off + ch]) + a.f_bias[ch], a.lower[ch]);
       sh_q[i] = silu_f32(to_f32(src[a.q_off + ch]));
-      sh_f[i] = live ? g.f : 1.f;
+      sh_f[i] = live ? decay_of(g.f, g.k) : Decay{0.f, 1.f};
       sh_k[i] = live ? g.k : 0.f;
     }
     for (int i = threadIdx.x; i < DV; i += BLOCK) sh_v[i] = to_f32(src[a.v_off + static_cast<int64_t>(h) * DV + i]);
@@ -68,10 +69,11 @@ __global__ __launch_bounds__(BLOCK) void hgrn2_tokens_kernel(const e2h_hgrn2_arg
     for (int i = 0; i < RPT; ++i) {
       const int r = rg + RG * i;
       if (r < D) {
-        const float f = sh_f[r], k = sh_k[r], q = sh_q[r];
+        const Decay f = sh_f[r];
+        const float k = sh_k[r], q = sh_q[r];
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          s[i][e] = __builtin_fmaf(k, v[e], f * s[i][e]);
+          s[i][e] = __builtin_fmaf(k, v[e], decayed(f, s[i][e]));
           acc[e] = __builtin_fmaf(q, s[i][e], acc[e]);
         }
       }
@@ -100,57 +102,98 @@ __global__ __launch_bounds__(BLOCK) void hgrn2_tokens_kernel(const e2h_hgrn2_arg
 
 // ---- chunked form ----------------------------------------------------------------------------------------------------------
 constexpr int kBlockTokens = 16;
-__device__ __forceinline__ float load_act(const void *p, int bf16, int64_t i) {
-  return bf16 ? to_f32(static_cast<const bf16_t *>(p)[i]) : static_cast<const float *>(p)[i];
-}
-
 struct ChunkPlan {
   float *delta;  // [chunks, batch * heads, dim, vdim]: a chunk's contribution, then the state at its start
   float *decay;  // [chunks, batch * heads, dim]
   int chunks, tokens;  // tokens per chunk
 };
 
-// Block's gates, keys and values into LDS (rows of DP + 4 / VP + 4 floats), tokens past the end and padding tokens as ones that
-// leave the state alone, then base-2 log decays summed over the block.  NT threads.
-template <int DP, int VP, int NT, bool QUERIES>
-__device__ __forceinline__ void stage_block(const e2h_hgrn2_args &a, size_t row0, int h, int t0, int64_t pos0, int64_t first, float *sq, float *sk,
-                                            float *sc, float *sv) {
-  const int D = static_cast<int>(a.dim), DV = static_cast<int>(a.vdim), seqlen = static_cast<int>(a.seqlen);
-  const int bf16 = a.dtype == E2H_SEQ_BF16;
-  for (int i = threadIdx.x; i < kBlockTokens * DP; i += NT) {
-    const int t = i / DP, d = i % DP;
-    float q = 0.f, k = 0.f, lg = 0.f;
-    if (d < D && t0 + t < seqlen) {
-      const int64_t base = static_cast<int64_t>(row0 + t0 + t) * a.ld;
-      const int ch = h * D + d;
-      if (QUERIES) q = silu_f32(load_act(a.proj, bf16, base + a.q_off + ch));
-      if (pos0 + t0 + t >= first) {
-        const Gate g = hgrn_gate(load_act(a.proj, bf16, base + a.f_off + ch) + a.f_bias[ch], a.lower[ch]);
-        k = g.k;
-        // log1p where 1 - k would round the decay, the plain logarithm (of a number that never is 0) elsewhere
-        lg = (k < 0.5f ? log1pf(-k) : logf(fmaxf(g.f, 1e-38f))) * kLog2e;
-      }
-    }
-    if (QUERIES) sq[t * (DP + 4) + d] = q;
-    sk[t * (DP + 4) + d] = k;
-    sc[t * (DP + 4) + d] = lg;
+// A block's projections on their way into LDS (rows of DP + 4 / VP + 4 floats).  `fetch` issues the loads, one block ahead of
+// `commit`, which turns them into queries, keys and base-2 log decays summed over the block.  Tokens past the end and
+// padding tokens become ones that leave the state alone.  NT threads; a thread's channels are the same in every block.
+template <typename T, int DP, int VP, int NT, bool QUERIES>
+struct BlockLoader {
+  static constexpr int kQuads = kBlockTokens * DP / 4 / NT, kVQuads = kBlockTokens * VP / 4 / NT;
+  static_assert(kQuads * NT * 4 == kBlockTokens * DP && kVQuads * NT * 4 == kBlockTokens * VP && NT % (DP / 4) == 0 && NT % (VP / 4) == 0);
+  Quad<T> q[kQuads], f[kQuads], v[kVQuads];
+  f32x4_t bias, low;
+  const T *src;  // the sequence's first row
+  int64_t ld;
+  int d, vd, seqlen, dim, vdim;
+
+  __device__ __forceinline__ BlockLoader(const e2h_hgrn2_args &a, size_t row0, int h) {
+    d = static_cast<int>(threadIdx.x % (DP / 4)) * 4;
+    vd = static_cast<int>(threadIdx.x % (VP / 4)) * 4;
+    dim = static_cast<int>(a.dim);
+    vdim = static_cast<int>(a.vdim);
+    seqlen = static_cast<int>(a.seqlen);
+    ld = a.ld;
+    src = static_cast<const T *>(a.proj) + row0 * a.ld;
+    const int ch = h * dim + (d < dim ? d : 0);
+    bias = load4(a.f_bias + ch);
+    low = load4(a.lower + ch);
+    q_col = a.q_off + ch;
+    f_col = a.f_off + ch;
+    v_col = a.v_off + static_cast<int64_t>(h) * vdim + (vd < vdim ? vd : 0);
   }
-  for (int i = threadIdx.x; i < kBlockTokens * VP; i += NT) {
-    const int t = i / VP, d = i % VP;
-    sv[t * (VP + 4) + d] =
-        d < DV && t0 + t < seqlen ? load_act(a.proj, bf16, static_cast<int64_t>(row0 + t0 + t) * a.ld + a.v_off + static_cast<int64_t>(h) * DV + d) : 0.f;
-  }
-  __syncthreads();
-  for (int d = threadIdx.x; d < DP; d += NT) {
-    float c = 0.f;
+  int64_t q_col, f_col, v_col;
+
+  __device__ __forceinline__ void fetch(int t0) {
 #pragma unroll
-    for (int t = 0; t < kBlockTokens; ++t) {
-      c += sc[t * (DP + 4) + d];
-      sc[t * (DP + 4) + d] = c;
+    for (int i = 0; i < kQuads; ++i) {
+      const int t = t0 + static_cast<int>(threadIdx.x / (DP / 4)) + i * (NT / (DP / 4));
+      const T *row = src + static_cast<int64_t>(t < seqlen ? t : seqlen - 1) * ld;
+      if (QUERIES) q[i] = load_quad(row + q_col);
+      f[i] = load_quad(row + f_col);
+    }
+#pragma unroll
+    for (int i = 0; i < kVQuads; ++i) {
+      const int t = t0 + static_cast<int>(threadIdx.x / (VP / 4)) + i * (NT / (VP / 4));
+      v[i] = load_quad(src + static_cast<int64_t>(t < seqlen ? t : seqlen - 1) * ld + v_col);
     }
   }
-  __syncthreads();
-}
+
+  __device__ __forceinline__ void commit(int t0, int64_t pos0, int64_t first, float *sq, float *sk, float *sc, float *sv) {
+    const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < kQuads; ++i) {
+      const int t = static_cast<int>(threadIdx.x / (DP / 4)) + i * (NT / (DP / 4));
+      const bool there = d < dim && t0 + t < seqlen, live = there && pos0 + t0 + t >= first;
+      f32x4_t qv = zero, kv = zero, lg = zero;
+      const f32x4_t fz = f[i].f32() + bias;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float up = 1.0f - low[e], sn = fast_sigmoid(-fz[e]);
+        kv[e] = up * sn;
+        lg[e] = log2_one_minus(kv[e], __builtin_fmaf(up, fast_sigmoid(fz[e]), low[e]));
+      }
+      if (QUERIES) {
+        qv = q[i].f32();
+#pragma unroll
+        for (int e = 0; e < 4; ++e) qv[e] = fast_silu(qv[e]);
+        store4(sq + t * (DP + 4) + d, there ? qv : zero);
+      }
+      store4(sk + t * (DP + 4) + d, live ? kv : zero);
+      store4(sc + t * (DP + 4) + d, live ? lg : zero);
+    }
+#pragma unroll
+    for (int i = 0; i < kVQuads; ++i) {
+      const int t = static_cast<int>(threadIdx.x / (VP / 4)) + i * (NT / (VP / 4));
+      store4(sv + t * (VP + 4) + vd, vd < vdim && t0 + t < seqlen ? v[i].f32() : zero);
+    }
+    __syncthreads();
+    if (threadIdx.x < DP) {
+      float c[kBlockTokens];
+#pragma unroll
+      for (int t = 0; t < kBlockTokens; ++t) c[t] = sc[t * (DP + 4) + threadIdx.x];
+#pragma unroll
+      for (int t = 1; t < kBlockTokens; ++t) c[t] += c[t - 1];
+#pragma unroll
+      for (int t = 0; t < kBlockTokens; ++t) sc[t * (DP + 4) + threadIdx.x] = c[t];
+    }
+    __syncthreads();
+  }
+};
 
 // S = decay of the block * S + k~^T V, k~ the keys decayed to the block's end (in sk)
 template <int DT, int VTW, int DP, int VP>
@@ -180,7 +223,7 @@ __device__ __forceinline__ void update_state(const float *sk, const float *sc, c
 }
 
 // step 1
-template <int DT, int VTW, int NW>
+template <typename T, int DT, int VTW, int NW>
 __global__ __launch_bounds__(64 * NW) void hgrn2_chunk_state_kernel(const e2h_hgrn2_args a, ChunkPlan plan) {
   constexpr int DP = DT * 16, VP = VTW * NW * 16, NT = 64 * NW;
   __shared__ __attribute__((aligned(16))) float sk[kBlockTokens * (DP + 4)], sc[kBlockTokens * (DP + 4)], sv[kBlockTokens * (VP + 4)];
@@ -197,8 +240,11 @@ __global__ __launch_bounds__(64 * NW) void hgrn2_chunk_state_kernel(const e2h_hg
 #pragma unroll
     for (int v = 0; v < VTW; ++v) s[dt][v] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float total[(DP + NT - 1) / NT] = {};
+  BlockLoader<T, DP, VP, NT, false> loader(a, row0, h);
+  loader.fetch(chunk * plan.tokens);
   for (int t0 = chunk * plan.tokens; t0 < (chunk + 1) * plan.tokens; t0 += kBlockTokens) {  // all chunks but the last are whole
-    stage_block<DP, VP, NT, false>(a, row0, h, t0, pos0, first, nullptr, sk, sc, sv);
+    loader.commit(t0, pos0, first, nullptr, sk, sc, sv);
+    loader.fetch(t0 + kBlockTokens);
     for (int i = threadIdx.x; i < kBlockTokens * DP; i += NT) {
       const int t = i / DP, d = i % DP;
       sk[t * (DP + 4) + d] *= __builtin_amdgcn_exp2f(sc[(kBlockTokens - 1) * (DP + 4) + d] - sc[t * (DP + 4) + d]);
@@ -252,7 +298,7 @@ __global__ __launch_bounds__(256) void hgrn2_scan_kernel(const e2h_hgrn2_args a,
 }
 
 // step 3
-template <int DT, int VTW, int NW>
+template <typename T, int DT, int VTW, int NW>
 __global__ __launch_bounds__(64 * NW) void hgrn2_chunk_output_kernel(const e2h_hgrn2_args a, ChunkPlan plan) {
   constexpr int DP = DT * 16, VP = VTW * NW * 16, NT = 64 * NW;
   constexpr int kLevels = 5;
@@ -283,9 +329,12 @@ __global__ __launch_bounds__(64 * NW) void hgrn2_chunk_output_kernel(const e2h_h
 #pragma unroll
   for (int v = 0; v < VTW; ++v) w[v] = (vt0 + v) * 16 + c < DV ? a.norm_weight[(vt0 + v) * 16 + c] * a.out_scale : 0.f;
 
+  BlockLoader<T, DP, VP, NT, true> loader(a, row0, h);
+  loader.fetch(chunk * plan.tokens);
   const int t_end = (chunk + 1) * plan.tokens < seqlen ? (chunk + 1) * plan.tokens : seqlen;
   for (int t0 = chunk * plan.tokens; t0 < t_end; t0 += kBlockTokens) {
-    stage_block<DP, VP, NT, true>(a, row0, h, t0, pos0, first, sq, sk, sc, sv);
+    loader.commit(t0, pos0, first, sq, sk, sc, sv);
+    loader.fetch(t0 + kBlockTokens);
     // products among the block's tokens: this wave's share of the channels, one accumulator per level
     f32x4_t lev[kLevels];
 #pragma unroll
@@ -373,8 +422,7 @@ __global__ __launch_bounds__(64 * NW) void hgrn2_chunk_output_kernel(const e2h_h
           const int col = (vt0 + v) * 16 + c;
           if (col < DV) {
             const float y = o[v][r] * inv * w[v];
-            if (a.dtype == E2H_SEQ_BF16) static_cast<bf16_t *>(a.out)[base + col] = f32_to_bf16_rne(y);
-            else static_cast<float *>(a.out)[base + col] = y;
+            static_cast<T *>(a.out)[base + col] = from_f32<T>(y);
           }
         }
       }
@@ -408,6 +456,7 @@ ChunkPlan plan_chunks(const e2h_hgrn2_args &a) {
 
 bool use_chunks(const e2h_hgrn2_args &a) {
   if (seq_options().recurrence_form == 1) return false;
+  if (a.dim % 4 != 0 || a.ld % 4 != 0 || a.q_off % 4 != 0 || a.f_off % 4 != 0 || a.v_off % 4 != 0) return false;  // four channels per load
   return seq_options().recurrence_form == 2 ? a.seqlen > 1 : a.seqlen >= 24;
 }
 
@@ -419,32 +468,33 @@ int64_t chunk_scratch_bytes(const e2h_hgrn2_args &a) {
   return p.chunks > 1 ? delta_bytes(a, p) + p.chunks * a.batch * a.heads * a.dim * 4 : 0;
 }
 
-template <int DT, int VTW, int NW>
+template <typename T, int DT, int VTW, int NW>
 void launch_chunks_sized(const e2h_hgrn2_args &a, const ChunkPlan &p, hipStream_t s) {
   const int64_t bh = a.batch * a.heads;
   if (p.chunks > 1) {
-    hipLaunchKernelGGL((hgrn2_chunk_state_kernel<DT, VTW, NW>), dim3(static_cast<unsigned>(bh * (p.chunks - 1))), dim3(64 * NW), 0, s, a, p);
+    hipLaunchKernelGGL((hgrn2_chunk_state_kernel<T, DT, VTW, NW>), dim3(static_cast<unsigned>(bh * (p.chunks - 1))), dim3(64 * NW), 0, s, a, p);
     hipLaunchKernelGGL(hgrn2_scan_kernel, dim3(static_cast<unsigned>((bh * a.dim * a.vdim / 4 + 255) / 256)), dim3(256), 0, s, a, p);
   }
-  hipLaunchKernelGGL((hgrn2_chunk_output_kernel<DT, VTW, NW>), dim3(static_cast<unsigned>(bh * p.chunks)), dim3(64 * NW), 0, s, a, p);
+  hipLaunchKernelGGL((hgrn2_chunk_output_kernel<T, DT, VTW, NW>), dim3(static_cast<unsigned>(bh * p.chunks)), dim3(64 * NW), 0, s, a, p);
 }
 
-template <int DT>
+template <typename T, int DT>
 void launch_chunks_dim(const e2h_hgrn2_args &a, const ChunkPlan &p, hipStream_t s) {
-  if (a.vdim <= 64) launch_chunks_sized<DT, 1, 4>(a, p, s);
-  else if (a.vdim <= 128) launch_chunks_sized<DT, 2, 4>(a, p, s);
-  else launch_chunks_sized<DT, 2, 8>(a, p, s);
+  if (a.vdim <= 64) launch_chunks_sized<T, DT, 1, 4>(a, p, s);
+  else if (a.vdim <= 128) launch_chunks_sized<T, DT, 2, 4>(a, p, s);
+  else launch_chunks_sized<T, DT, (DT <= 4 ? 4 : 2), (DT <= 4 ? 4 : 8)>(a, p, s);
 }
 
+template <typename T>
 void launch_chunks(const e2h_hgrn2_args &a, hipStream_t s) {
   ChunkPlan p = plan_chunks(a);
   if (p.chunks > 1) {
     p.delta = static_cast<float *>(a.scratch);
     p.decay = reinterpret_cast<float *>(static_cast<uint8_t *>(a.scratch) + delta_bytes(a, p));
   }
-  if (a.dim <= 64) launch_chunks_dim<4>(a, p, s);
-  else if (a.dim <= 128) launch_chunks_dim<8>(a, p, s);
-  else launch_chunks_dim<16>(a, p, s);
+  if (a.dim <= 64) launch_chunks_dim<T, 4>(a, p, s);
+  else if (a.dim <= 128) launch_chunks_dim<T, 8>(a, p, s);
+  else launch_chunks_dim<T, 16>(a, p, s);
 }
 
 template <typename T>
@@ -485,7 +535,9 @@ extern "C" int e2h_seq_hgrn2(const e2h_hgrn2_args *a, void *stream) {
     if (a->batch * a->heads * p.chunks > INT32_MAX || a->batch * a->heads * a->dim * a->vdim / 1024 > INT32_MAX - 1) return E2H_ERR_BAD_SHAPE;
     if (need > 0 && !a->scratch) return E2H_ERR_NULL_POINTER;
     if (need > a->scratch_bytes) return E2H_ERR_SCRATCH_TOO_SMALL;
-    launch_chunks(*a, static_cast<hipStream_t>(stream));
+    if (!aligned16(a->proj) || !aligned16(a->f_bias) || !aligned16(a->lower)) return E2H_ERR_MISALIGNED;
+    if (a->dtype == E2H_SEQ_BF16) launch_chunks<bf16_t>(*a, static_cast<hipStream_t>(stream));
+    else launch_chunks<float>(*a, static_cast<hipStream_t>(stream));
     return launch_status();
   }
   if (a->dtype == E2H_SEQ_BF16) launch_tokens<bf16_t>(*a, static_cast<hipStream_t>(stream));

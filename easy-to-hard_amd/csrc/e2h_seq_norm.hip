@@ -13,105 +13,134 @@ SeqOptions &seq_options() {
 
 namespace {
 
-// One workgroup per run of `run` consecutive tokens of one sequence.  A thread owns NP pieces of four channels, so the
-// convolution's previous inputs stay in its registers from token to token; the taps - 1 tokens ahead of the run are
-// normalised again by the workgroup (inside the call) or come from the ring of kept inputs (before the call).
-// TAPS is the compiled depth of the convolution (0 = none); shallower ones pad their weights with zeros in front.
-template <typename T, int BLOCK, int NP, int TAPS>
+// One workgroup per run of `run` consecutive tokens of one sequence, NB tokens at a time so that the loads of NB rows are in
+// flight together and one barrier serves NB row sums.  A thread owns NP pieces of four channels, so the convolution's previous
+// inputs stay in its registers from token to token; the taps - 1 tokens ahead of the run are normalised again by the
+// workgroup (inside the call) or come from the ring of kept inputs (before the call).  TAPS is the compiled depth of the
+// convolution (0 = none); shallower ones pad their weights with zeros in front.
+template <typename T, int BLOCK, int NP, int TAPS, int NB>
 __global__ __launch_bounds__(BLOCK) void norm_conv_kernel(const e2h_norm_conv_args a, int runs, int run) {
   constexpr int kWaves = BLOCK / 64;
   constexpr int RING = TAPS > 1 ? TAPS - 1 : 1;
+  const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
   const int W = static_cast<int>(a.width), seqlen = static_cast<int>(a.seqlen), taps = a.taps;
   const int b = blockIdx.x / runs, t_begin = (blockIdx.x % runs) * run;
   const int t_end = t_begin + run < seqlen ? t_begin + run : seqlen;
-  const int64_t pos0 = TAPS ? a.input_pos[0] : 0;
-  const int64_t first = TAPS && a.first ? a.first[b] : 0;
+  const int pos0 = TAPS ? static_cast<int>(a.input_pos[0]) : 0;
+  const int first = TAPS && a.first ? static_cast<int>(a.first[b]) : 0;
   const size_t row0 = static_cast<size_t>(b) * seqlen;
-  __shared__ float part[2][kWaves];
+  __shared__ float part[2][kWaves][NB];
   int phase = 0;
 
-  auto block_sum = [&](float v) {
-    v = wave_add(v);
-    if ((threadIdx.x & 63) == 0) part[phase][threadIdx.x >> 6] = v;
-    __syncthreads();
-    float s = 0.f;
+  auto block_sum = [&](float (&v)[NB]) {
 #pragma unroll
-    for (int w = 0; w < kWaves; ++w) s += part[phase][w];
-    phase ^= 1;  // the next sum writes the other half, so one barrier per sum is enough
-    return s;
+    for (int k = 0; k < NB; ++k) v[k] = wave_add(v[k]);
+    if ((threadIdx.x & 63) == 0) {
+#pragma unroll
+      for (int k = 0; k < NB; ++k) part[phase][threadIdx.x >> 6][k] = v[k];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < NB; ++k) {
+      v[k] = 0.f;
+#pragma unroll
+      for (int w = 0; w < kWaves; ++w) v[k] += part[phase][w][k];
+      v[k] = 1.0f / sqrtf(v[k] / static_cast<float>(W) + a.eps);
+    }
+    phase ^= 1;  // the next sums go to the other half, so one barrier per sum is enough
   };
 
-  f32x4_t wconv[TAPS > 0 ? TAPS : 1][NP], ring[RING][NP];
-  if (TAPS) {
+  // everything that does not depend on the rows; zero weights and rows beyond the width contribute nothing
+  f32x4_t wconv[TAPS > 0 ? TAPS : 1][NP], wd[NP], wn[NP], ring[RING][NP];
 #pragma unroll
-    for (int p = 0; p < NP; ++p) {
-      const int i = (p * BLOCK + threadIdx.x) * 4;
+  for (int p = 0; p < NP; ++p) {
+    const int i = (p * BLOCK + threadIdx.x) * 4;
+    wd[p] = wn[p] = zero;
+    if (a.delta && i < W) wd[p] = load4(a.delta_weight + i) + a.delta_offset;
+    if (a.norm_weight && i < W) wn[p] = load4(a.norm_weight + i) + a.norm_offset;
+    if (TAPS) {
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) {
-        wconv[j][p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
         const int jj = j - (TAPS - taps);
-        if (i < W && jj >= 0) {
-#pragma unroll
-          for (int e = 0; e < 4; ++e) wconv[j][p][e] = a.conv[static_cast<size_t>(i + e) * taps + jj];
-        }
+        wconv[j][p] = zero;
+        if (i < W && jj >= 0) wconv[j][p] = load4(a.conv + static_cast<size_t>(jj) * W + i);
       }
-#pragma unroll
-      for (int j = 0; j < RING; ++j) ring[j][p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
   }
 
-  // h of token t (the convolution's input); emit: also store the updated residual row
-  auto norm_row = [&](int t, bool emit, f32x4_t (&h)[NP]) {
-    const size_t base = (row0 + t) * W;
-    f32x4_t d[NP];
+  // kept inputs of the positions before the call, for a run at its start
+  auto kept = [&](int t, f32x4_t (&h)[NP]) {
+    const int pos = pos0 + t;
+    const bool live = pos >= first && pos >= 0 && t >= -(taps - 1);
+    const float *src = a.tail_in + (static_cast<size_t>(b) * taps + (live ? static_cast<uint32_t>(pos) % static_cast<uint32_t>(taps) : 0u)) * W;
 #pragma unroll
     for (int p = 0; p < NP; ++p) {
       const int i = (p * BLOCK + threadIdx.x) * 4;
-      h[p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-      d[p] = h[p];
-      if (i < W) {
-        h[p] = load4(a.x + base + i);
-        if (a.delta) d[p] = load4(static_cast<const T *>(a.delta) + base + i);
+      h[p] = zero;
+      if (live && i < W) h[p] = load4(src + i);
+    }
+  };
+
+  // h (the convolution's inputs) of the tokens t .. t + NB - 1; emit: also store the updated residual rows
+  auto norm_rows = [&](int t, bool emit, f32x4_t (&h)[NB][NP]) {
+    f32x4_t d[NB][NP];
+#pragma unroll
+    for (int k = 0; k < NB; ++k) {
+      const int tc = t + k < 0 ? 0 : t + k < seqlen ? t + k : seqlen - 1;
+      const size_t base = (row0 + tc) * W;
+#pragma unroll
+      for (int p = 0; p < NP; ++p) {
+        const int i = (p * BLOCK + threadIdx.x) * 4;
+        h[k][p] = d[k][p] = zero;
+        if (i < W) {
+          h[k][p] = load4(a.x + base + i);
+          if (a.delta) d[k][p] = load4(static_cast<const T *>(a.delta) + base + i);
+        }
       }
     }
     if (a.delta) {
-      float ss = 0.f;
+      float ss[NB];
 #pragma unroll
-      for (int p = 0; p < NP; ++p)
+      for (int k = 0; k < NB; ++k) {
+        ss[k] = 0.f;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) ss = __builtin_fmaf(d[p][e], d[p][e], ss);
-      const float inv = 1.0f / sqrtf(block_sum(ss) / static_cast<float>(W) + a.eps);
+        for (int p = 0; p < NP; ++p)
 #pragma unroll
-      for (int p = 0; p < NP; ++p) {
-        const int i = (p * BLOCK + threadIdx.x) * 4;
-        if (i < W) {
-          const f32x4_t w = load4(a.delta_weight + i);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) h[p][e] += d[p][e] * inv * (a.delta_offset + w[e]);
-          if (emit && a.x_out) store4(a.x_out + base + i, h[p]);
-        }
+          for (int e = 0; e < 4; ++e) ss[k] = __builtin_fmaf(d[k][p][e], d[k][p][e], ss[k]);
       }
+      block_sum(ss);
+#pragma unroll
+      for (int k = 0; k < NB; ++k)
+#pragma unroll
+        for (int p = 0; p < NP; ++p) {
+          const int i = (p * BLOCK + threadIdx.x) * 4;
+          h[k][p] += d[k][p] * ss[k] * wd[p];
+          if (emit && a.x_out && i < W && t + k < t_end) store4(a.x_out + (row0 + t + k) * W + i, h[k][p]);
+        }
     }
     if (a.norm_weight) {
-      float ss = 0.f;
+      float ss[NB];
 #pragma unroll
-      for (int p = 0; p < NP; ++p)
+      for (int k = 0; k < NB; ++k) {
+        ss[k] = 0.f;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) ss = __builtin_fmaf(h[p][e], h[p][e], ss);
-      const float inv = 1.0f / sqrtf(block_sum(ss) / static_cast<float>(W) + a.eps);
+        for (int p = 0; p < NP; ++p)
 #pragma unroll
-      for (int p = 0; p < NP; ++p) {
-        const int i = (p * BLOCK + threadIdx.x) * 4;
-        if (i < W) {
-          const f32x4_t w = load4(a.norm_weight + i);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) h[p][e] = h[p][e] * inv * (a.norm_offset + w[e]);
-        }
+          for (int e = 0; e < 4; ++e) ss[k] = __builtin_fmaf(h[k][p][e], h[k][p][e], ss[k]);
       }
-    }
-    if (TAPS && pos0 + t < first) {  // padding: the convolution must not see it
+      block_sum(ss);
 #pragma unroll
-      for (int p = 0; p < NP; ++p) h[p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      for (int k = 0; k < NB; ++k)
+#pragma unroll
+        for (int p = 0; p < NP; ++p) h[k][p] = h[k][p] * ss[k] * wn[p];
+    }
+    if (TAPS) {
+#pragma unroll
+      for (int k = 0; k < NB; ++k)
+        if (pos0 + t + k < first) {  // padding: the convolution must not see it
+#pragma unroll
+          for (int p = 0; p < NP; ++p) h[k][p] = zero;
+        }
     }
   };
   auto push = [&](const f32x4_t (&h)[NP]) {
@@ -124,62 +153,55 @@ __global__ __launch_bounds__(BLOCK) void norm_conv_kernel(const e2h_norm_conv_ar
   };
 
   if (TAPS > 1) {
-    for (int s = t_begin - (taps - 1); s < t_begin; ++s) {
-      f32x4_t h[NP];
-      if (s >= 0) {
-        norm_row(s, false, h);
-      } else {
-        const int64_t pos = pos0 + s;
-        const bool live = pos >= first && pos >= 0;
-        const float *src = a.tail_in + (static_cast<size_t>(b) * taps + (live ? pos % taps : 0)) * W;
+    if (t_begin == 0) {
 #pragma unroll
-        for (int p = 0; p < NP; ++p) {
-          const int i = (p * BLOCK + threadIdx.x) * 4;
-          h[p] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-          if (live && i < W) h[p] = load4(src + i);
-        }
-      }
-      push(h);
-    }
-  }
-  for (int t = t_begin; t < t_end; ++t) {
-    f32x4_t h[NP];
-    norm_row(t, true, h);
-    const size_t base = (row0 + t) * W;
+      for (int j = 0; j < RING; ++j) kept(j - RING, ring[j]);
+    } else {
 #pragma unroll
-    for (int p = 0; p < NP; ++p) {
-      const int i = (p * BLOCK + threadIdx.x) * 4;
-      f32x4_t y = h[p];
-      if (TAPS) {
-        f32x4_t c = h[p] * wconv[TAPS > 0 ? TAPS - 1 : 0][p];
-        if (TAPS > 1) {
+      for (int s = -((RING + NB - 1) / NB * NB); s < 0; s += NB) {
+        f32x4_t h[NB][NP];
+        norm_rows(t_begin + s, false, h);
 #pragma unroll
-          for (int j = 0; j < RING; ++j)
-#pragma unroll
-            for (int e = 0; e < 4; ++e) c[e] = __builtin_fmaf(ring[j][p][e], wconv[j][p][e], c[e]);
-        }
-        y += c;
-      }
-      if (a.out && i < W) store4(static_cast<T *>(a.out) + base + i, y);
-    }
-    if (TAPS > 1) {
-      push(h);
-      if (seqlen == 1) {
-        float *dst = a.tail_out + (static_cast<size_t>(b) * taps + (pos0 > 0 ? pos0 % taps : 0)) * W;
-#pragma unroll
-        for (int p = 0; p < NP; ++p) {
-          const int i = (p * BLOCK + threadIdx.x) * 4;
-          if (i < W) store4(dst + i, h[p]);
+        for (int k = 0; k < NB; ++k) {
+          if (t_begin + s + k < 0) kept(t_begin + s + k, h[k]);
+          push(h[k]);
         }
       }
     }
   }
-  if (TAPS > 1 && seqlen > 1 && t_end == seqlen) {  // the last inputs of the call, oldest first in the ring registers
+  for (int t = t_begin; t < t_end; t += NB) {
+    f32x4_t h[NB][NP];
+    norm_rows(t, true, h);
+#pragma unroll
+    for (int k = 0; k < NB; ++k) {
+      if (t + k < t_end) {
+        const size_t base = (row0 + t + k) * W;
+#pragma unroll
+        for (int p = 0; p < NP; ++p) {
+          const int i = (p * BLOCK + threadIdx.x) * 4;
+          f32x4_t y = h[k][p];
+          if (TAPS) {
+            f32x4_t c = y * wconv[TAPS > 0 ? TAPS - 1 : 0][p];
+            if (TAPS > 1) {
+#pragma unroll
+              for (int j = 0; j < RING; ++j)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) c[e] = __builtin_fmaf(ring[j][p][e], wconv[j][p][e], c[e]);
+            }
+            y += c;
+          }
+          if (a.out && i < W) store4(static_cast<T *>(a.out) + base + i, y);
+        }
+        if (TAPS > 1) push(h[k]);
+      }
+    }
+  }
+  if (TAPS > 1 && t_end == seqlen) {  // the last inputs of the call, oldest first in the ring registers; one token replaces one slot
 #pragma unroll
     for (int j = 0; j < RING; ++j) {
-      const int64_t pos = pos0 + seqlen - RING + j;
-      if (j >= RING - (taps - 1) && pos >= 0) {
-        float *dst = a.tail_out + (static_cast<size_t>(b) * taps + pos % taps) * W;
+      const int pos = pos0 + seqlen - RING + j;
+      if (j >= RING - (seqlen == 1 ? 1 : taps - 1) && pos >= 0 && taps > 1) {
+        float *dst = a.tail_out + (static_cast<size_t>(b) * taps + static_cast<uint32_t>(pos) % static_cast<uint32_t>(taps)) * W;
 #pragma unroll
         for (int p = 0; p < NP; ++p) {
           const int i = (p * BLOCK + threadIdx.x) * 4;
@@ -190,23 +212,28 @@ __global__ __launch_bounds__(BLOCK) void norm_conv_kernel(const e2h_norm_conv_ar
   }
 }
 
+template <typename T, int BLOCK, int NP, int TAPS>
+void launch_norm_conv_rows(const e2h_norm_conv_args &a, int runs, int run, hipStream_t s) {
+  const dim3 grid(static_cast<unsigned>(a.batch * runs)), block(BLOCK);
+  constexpr int NB = NP > 1 || TAPS > 4 ? 1 : TAPS ? 2 : 4;  // rows that fit the registers
+  if (run == 1) hipLaunchKernelGGL((norm_conv_kernel<T, BLOCK, NP, TAPS, 1>), grid, block, 0, s, a, runs, run);
+  else hipLaunchKernelGGL((norm_conv_kernel<T, BLOCK, NP, TAPS, NB>), grid, block, 0, s, a, runs, run);
+}
+
 template <typename T, int BLOCK, int NP>
 void launch_norm_conv_taps(const e2h_norm_conv_args &a, int runs, int run, hipStream_t s) {
-  const dim3 grid(static_cast<unsigned>(a.batch * runs)), block(BLOCK);
-  if (!a.conv)
-    hipLaunchKernelGGL((norm_conv_kernel<T, BLOCK, NP, 0>), grid, block, 0, s, a, runs, run);
-  else if (a.taps <= 4)
-    hipLaunchKernelGGL((norm_conv_kernel<T, BLOCK, NP, 4>), grid, block, 0, s, a, runs, run);
-  else
-    hipLaunchKernelGGL((norm_conv_kernel<T, BLOCK, NP, 8>), grid, block, 0, s, a, runs, run);
+  if (!a.conv) launch_norm_conv_rows<T, BLOCK, NP, 0>(a, runs, run, s);
+  else if (a.taps <= 4) launch_norm_conv_rows<T, BLOCK, NP, 4>(a, runs, run, s);
+  else launch_norm_conv_rows<T, BLOCK, NP, 8>(a, runs, run, s);
 }
 
 template <typename T>
 void launch_norm_conv(const e2h_norm_conv_args &a, int runs, int run, hipStream_t s) {
   if (a.width <= 1024) launch_norm_conv_taps<T, 256, 1>(a, runs, run, s);
-  else if (a.width <= 2048) launch_norm_conv_taps<T, 256, 2>(a, runs, run, s);
+  else if (a.width <= 2048) launch_norm_conv_taps<T, 512, 1>(a, runs, run, s);
+  else if (a.width <= 4096 && a.conv) launch_norm_conv_taps<T, 1024, 1>(a, runs, run, s);
   else if (a.width <= 4096) launch_norm_conv_taps<T, 512, 2>(a, runs, run, s);
-  else if (a.width <= 8192) launch_norm_conv_taps<T, 1024, 2>(a, runs, run, s);
+  else if (a.width <= 8192) launch_norm_conv_taps<T, 512, 4>(a, runs, run, s);
   else launch_norm_conv_taps<T, 1024, 4>(a, runs, run, s);
 }
 
@@ -285,9 +312,6 @@ extern "C" int e2h_seq_set_option(const char *name, int value) {
   } else if (!strcmp(name, "attention_decode_waves")) {
     if (value != 0 && value != 4 && value != 8) return E2H_ERR_BAD_OPTION;
     o.attention_decode_waves = value;
-  } else if (!strcmp(name, "attention_query_tiles")) {
-    if (value < 0 || value > 2) return E2H_ERR_BAD_OPTION;
-    o.attention_query_tiles = value;
   } else {
     return E2H_ERR_BAD_OPTION;
   }
@@ -298,19 +322,19 @@ extern "C" int e2h_seq_norm_conv(const e2h_norm_conv_args *a, void *stream) {
   if (!a || !a->x || (a->delta && !a->delta_weight)) return E2H_ERR_NULL_POINTER;
   if (!a->out && !a->x_out) return E2H_ERR_NULL_POINTER;
   if (a->conv && (!a->input_pos || (a->taps > 1 && (!a->tail_in || !a->tail_out)))) return E2H_ERR_NULL_POINTER;
-  if (a->batch < 1 || a->seqlen < 1 || a->width < 4 || a->width % 4 != 0 || a->width > 16384 || a->seqlen > INT32_MAX / 2)
+  if (a->batch < 1 || a->seqlen < 1 || a->width < 4 || a->width % 4 != 0 || a->width > 16384 || a->seqlen > INT32_MAX / 4)
     return E2H_ERR_BAD_SHAPE;
   if (a->dtype != E2H_SEQ_BF16 && a->dtype != E2H_SEQ_F32) return E2H_ERR_BAD_SHAPE;
   if (a->conv && (a->taps < 1 || a->taps > 8)) return E2H_ERR_BAD_SHAPE;
   if (a->seqlen > 1 && a->conv && ((a->taps > 1 && a->tail_in == a->tail_out) || (a->delta && a->x == a->x_out && a->taps > 1))) return E2H_ERR_BAD_SHAPE;
   if (!aligned16(a->x) || !aligned16(a->delta) || !aligned16(a->delta_weight) || !aligned16(a->x_out) || !aligned16(a->norm_weight) ||
-      !aligned16(a->tail_in) || !aligned16(a->tail_out) || !aligned16(a->out))
+      !aligned16(a->conv) || !aligned16(a->tail_in) || !aligned16(a->tail_out) || !aligned16(a->out))
     return E2H_ERR_MISALIGNED;
   // enough workgroups to fill the chip first, then longer runs so that fewer tokens are normalised twice
   int run = seq_options().norm_run;
   if (!run) {
-    run = static_cast<int>(a->batch * a->seqlen / 1024);
-    run = run < 1 ? 1 : run > 16 ? 16 : run;
+    run = static_cast<int>(a->batch * a->seqlen / (a->conv ? 256 : 1024));
+    run = run < 1 ? 1 : run > 32 ? 32 : run;
   }
   const int64_t runs = (a->seqlen + run - 1) / run;
   if (a->batch * runs > INT32_MAX) return E2H_ERR_BAD_SHAPE;

@@ -222,7 +222,8 @@ def load_reward_model(checkpoint_path, device, precision=torch.bfloat16, use_tp:
     its `main` runs afterwards (:171-178): the checkpoint is a bfloat16 language-model state dict (quantized files are
     rejected, as there), loaded memory-mapped into the backbone built on the meta device; the `output` projection becomes
     the zero-initialised two-row score head (a fine-tuned head is loaded over it by the caller); the model moves to
-    `device` in `precision`; with `on_the_fly_8bit_quantization` every linear, head included, is then quantized to int8
+    `device` in `precision` (a folder with config.json gives the registered model's backbone instead); with
+    `on_the_fly_8bit_quantization` every linear, head included, is then quantized to int8
     per channel on the device by `WeightOnlyInt8QuantHandler.convert_for_runtime_on_the_fly`."""
     from pathlib import Path
 
@@ -232,6 +233,17 @@ def load_reward_model(checkpoint_path, device, precision=torch.bfloat16, use_tp:
     if use_tp:
         raise NotImplementedError("load_reward_model: tensor parallelism is outside this one-GPU build")
     checkpoint_path = Path(checkpoint_path)
+    if checkpoint_path.is_dir():
+        backbone = load_folder(checkpoint_path, device, precision)
+        apply_reward_modeling_head(backbone)
+        backbone.logit_softcap = None
+        with torch.device("meta"):
+            model = RewardModel(backbone.config)
+        model.backbone = backbone
+        model = model.eval()
+        if on_the_fly_8bit_quantization:
+            model = WeightOnlyInt8QuantHandler(model).convert_for_runtime_on_the_fly().to(device=device).eval()
+        return model
     if "int8" in str(checkpoint_path):
         raise NotImplementedError("int8 quantization cannot be used for reward model!")
     if "int4" in str(checkpoint_path):

@@ -1,0 +1,96 @@
+"""Prefill and decode throughput of the Refatar decoder on random weights at layer sizes of real models, beside the
+Llama-family Transformer of equal width, depth, heads and parameter count per layer (bench.py --refatar)."""
+
+import time
+
+import torch
+
+from . import generate
+from .model import ModelArgs, random_quantized_transformer
+from .refatar import Refatar
+
+# layers alternate between the two mixers; the comparison's gated feed-forward has 2/3 of the hidden size (three matrices)
+SIZES = {
+    "1b": dict(width=2048, ff=8192, heads=16, kv_heads=4, dim=128, recurrent_heads=16, recurrent_dim=128, delta_kv=8, window=1024, keep=4,
+               side=128, layers=8, vocab=32000),
+    "7b": dict(width=4096, ff=16384, heads=32, kv_heads=8, dim=128, recurrent_heads=32, recurrent_dim=128, delta_kv=16, window=2048, keep=4,
+               side=256, layers=8, vocab=32000),
+}
+
+
+def refatar_config(s):
+    r, d = s["recurrent_heads"], s["recurrent_dim"]
+    parallel = {"type": "parallel", "mlp": {"kind": "dense", "ff": s["ff"]}, "mixer": {
+        "left": {"heads": s["heads"], "kv_heads": s["kv_heads"], "dim": s["dim"], "vdim": s["dim"], "scale": s["dim"] ** -0.5,
+                 "mask": {"size": s["window"], "keep_first": s["keep"]}},
+        "right": {"heads": r, "dim": d, "vdim": d}, "left_scale": 0.7, "right_scale": 0.7}}
+    delta = {"type": "delta", "mlp": {"kind": "dense", "ff": s["ff"]},
+             "mixer": {"heads": r, "kv_heads": s["delta_kv"], "dim": d, "vdim": d, "conv": 4}}
+    return {"architecture": "Refatar", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "canon": {"taps": 4},
+            "token_side": {"dim": s["side"]}, "logit_softcap": 30.0, "layers": [parallel if i % 2 == 0 else delta for i in range(s["layers"])]}
+
+
+def random_refatar(config, device):
+    with torch.device("meta"):
+        model = Refatar.from_config(config)
+    return model.init_random_(device=device)
+
+
+def closest_model(s, device):
+    ff = (s["ff"] * 2 // 3 + 255) // 256 * 256
+    cfg = ModelArgs(block_size=32768, vocab_size=s["vocab"], n_layer=s["layers"], n_head=s["heads"], n_local_heads=s["kv_heads"], dim=s["width"],
+                    intermediate_size=ff)
+    return random_quantized_transformer(cfg, "bf16", device=device)
+
+
+def _timed(fn, reps):
+    fn()
+    torch.cuda.synchronize()
+    t0 = time.time()
+    for _ in range(reps):
+        fn()
+    torch.cuda.synchronize()
+    return (time.time() - t0) / reps
+
+
+@torch.no_grad()
+def measure(model, prompts, decodes, device, reps=3, steps=32, graph=True):
+    """{"prefill": tokens/s per (batch, length), "decode": tokens/s and us per step per (batch, context)}."""
+    out = {"prefill": {}, "decode": {}}
+    vocab = model.config.vocab_size
+    model.setup_caches(max([b for b, _ in prompts] + [b for b, _ in decodes]), max([t for _, t in prompts] + [t + steps + 1 for _, t in decodes]))
+    for b, t in prompts:
+        tokens = torch.randint(0, vocab, (b, t), device=device)
+        pos = torch.arange(t, device=device)
+        sec = _timed(lambda: model(tokens, pos, greedy_token=True), reps)
+        out["prefill"][f"{b}x{t}"] = {"tok_s": round(b * t / sec), "ms": round(sec * 1e3, 2)}
+    for b, t in decodes:
+        cur = torch.zeros((b, 1), dtype=torch.int64, device=device)
+        pos = torch.tensor([t], device=device)
+        if graph:
+            stepper = generate.GraphedDecodeStep(model, b, device)
+            fn = lambda: stepper.step(cur, pos)  # noqa: E731
+        else:
+            fn = lambda: generate.decode_one_token(model, cur, pos)  # noqa: E731
+        sec = _timed(fn, steps)
+        out["decode"][f"{b}@{t}"] = {"tok_s": round(b / sec), "us_per_step": round(sec * 1e6, 1)}
+    return out
+
+
+def parameters(model):
+    return sum(p.numel() for n, p in model.named_parameters() if "embeddings" not in n)
+
+
+def run(size, which, phase, device, steps):
+    s = SIZES[size]
+    prompts = [(1, 2048), (1, 8192), (8, 1024)] if phase in ("both", "prefill") else []
+    decodes = [(1, 4096), (32, 4096)] if phase in ("both", "decode") else []
+    result = {"size": size, "layers": s["layers"], "width": s["width"], "dtype": "bf16", "data": "synthetic, random weights"}
+    for name in ("refatar", "llama"):
+        if which not in ("both", name):
+            continue
+        model = random_refatar(refatar_config(s), device) if name == "refatar" else closest_model(s, device)
+        result[name] = {"parameters": parameters(model), **measure(model, prompts, decodes, device, steps=steps)}
+        del model
+        torch.cuda.empty_cache()
+    return result

@@ -337,6 +337,7 @@ def _staged_block_forward(blk: "TransformerBlock", x: Tensor, delta, input_pos: 
 
 class Transformer(nn.Module):
     returns_greedy_token = True  # forward(..., greedy_token=True) yields the token itself
+    logit_softcap = None         # this family's logits are not capped
 
     def __init__(self, config: ModelArgs) -> None:
         super().__init__()
@@ -455,10 +456,12 @@ class RewardModel(nn.Module):
     """Backbone whose `output` is a small score head; per-token reward = mean over head rows
     (reference models/reward_model.py:69-92: `Linear(dim, 2)` head followed by `.mean(-1)`)."""
 
-    def __init__(self, config: ModelArgs, head_rows: int = 2) -> None:
+    def __init__(self, config, head_rows: int = 2) -> None:
+        """config: ModelArgs, or another registered model's arguments (its class is config.model_class())."""
         super().__init__()
-        self.backbone = Transformer(config)
+        self.backbone = Transformer(config) if isinstance(config, ModelArgs) else config.model_class()(config)
         self.backbone.output = nn.Linear(config.dim, head_rows, bias=False)
+        self.backbone.logit_softcap = None  # scores are not logits
 
     def forward(self, idx: Tensor, eos_pos: Optional[Tensor] = None) -> Tensor:
         input_pos = torch.arange(0, idx.size(-1), device=idx.device)

@@ -32,6 +32,10 @@ class RefatarArgs:
     logit_softcap: Optional[float] = None
     block_size: int = 1 << 20  # positions do not enter any layer's weights; the caches are sized by setup_caches
 
+    @staticmethod
+    def model_class():
+        return Refatar
+
     @classmethod
     def from_config(cls, config: dict) -> "RefatarArgs":
         for i, layer in enumerate(config["layers"]):
@@ -76,13 +80,13 @@ class RefatarLayer(nn.Module):
         layer, w, taps = args.layers[index], args.dim, args.canon_taps
         self.mixer = build_mixer(plan, w, layer, args.norm_eps)
         self.norm1, self.norm1b = _vector(w), _vector(w)
-        self.canon1 = nn.Parameter(torch.zeros((w, taps), dtype=torch.float32), requires_grad=False)
+        self.canon1 = nn.Parameter(torch.zeros((taps, w), dtype=torch.float32), requires_grad=False)
         self.ring1 = plan.add_ring(w, taps, float32=True)
         self.feed_forward = None
         if layer.get("mlp") is not None:
             self.feed_forward = SquaredReluFF(w, layer["mlp"]["ff"])
             self.norm2, self.norm2b = _vector(w), _vector(w)
-            self.canon2 = nn.Parameter(torch.zeros((w, taps), dtype=torch.float32), requires_grad=False)
+            self.canon2 = nn.Parameter(torch.zeros((taps, w), dtype=torch.float32), requires_grad=False)
             self.ring2 = plan.add_ring(w, taps, float32=True)
         self.side_gate = nn.Linear(w, args.side_dim, bias=False)
         self.side_proj = nn.Linear(args.side_dim, w, bias=False)
@@ -97,7 +101,8 @@ class RefatarLayer(nn.Module):
             sd["feed_forward.up.weight"] = get(prefix + ".mlp.up").to(linear_dtype)
             sd["feed_forward.down.weight"] = get(prefix + ".mlp.down").to(linear_dtype)
         for n in names:
-            sd[n] = get(f"{prefix}.{n}").float()
+            t = get(f"{prefix}.{n}").float()
+            sd[n] = t.t().contiguous() if n.startswith("canon") else t  # stored [width, taps]; the kernel reads tap by tap
         sd["side_gate.weight"] = get(prefix + ".side.gate").to(linear_dtype)
         sd["side_proj.weight"] = get(prefix + ".side.proj").to(linear_dtype)
         sd["side_norm"] = get(prefix + ".side.norm").float()
@@ -133,6 +138,35 @@ class Refatar(nn.Module):
         for i, layer in enumerate(self.layers):
             sd.update({f"layers.{i}.{k}": v for k, v in layer.from_checkpoint(get, f"l{i}", linear_dtype).items()})
         return sd
+
+    def init_random_(self, seed: int = 1234, std: float = 0.02, dtype=torch.bfloat16, device=None) -> "Refatar":
+        """Random weights in place (also of a model built on the meta device): linears and embeddings N(0, std) in `dtype`,
+        convolution weights small, gate constants in their usual ranges, norms at one."""
+        device = device if device is not None else self.tok_embeddings.weight.device
+        gen = torch.Generator(device=device).manual_seed(seed)
+        rand = lambda p: torch.rand(p.shape, generator=gen, device=device)  # noqa: E731
+        randn = lambda p: torch.randn(p.shape, generator=gen, device=device)  # noqa: E731
+        state = {}
+        for name, p in self.state_dict().items():
+            leaf = name.rsplit(".", 1)[-1]
+            if leaf == "weight":
+                state[name] = (randn(p) * std).to(dtype)
+            elif leaf in ("canon1", "canon2", "conv"):
+                state[name] = randn(p) * 0.2
+            elif leaf == "lower":
+                state[name] = rand(p) * 0.5
+            elif leaf == "f_bias":
+                state[name] = rand(p) * 6
+            elif leaf == "dt_bias":
+                state[name] = rand(p) - 3.5
+            elif leaf == "a_log":
+                state[name] = rand(p) * -3
+            elif leaf == "side_norm" or ".branches." in name and leaf == "norm":
+                state[name] = torch.ones(p.shape, device=device)  # weights stored as they are; the others are offsets from one
+            else:
+                state[name] = torch.zeros(p.shape, device=device)
+        self.load_state_dict(state, assign=True)
+        return self.eval().requires_grad_(False)
 
     @property
     def dtype(self):

@@ -60,9 +60,8 @@ def _check_tail(tails, batch, taps, channels, dtype, what):
 
 def norm_conv(x, batch, seqlen, eps, dtype, delta=None, delta_weight=None, delta_offset=0.0, norm_weight=None, norm_offset=0.0, conv=None,
               tails=None, input_pos=None, first=None, want_x=True, want_out=True):
-    """x + norm(delta), its norm and the norm's convolution over time (each optional) in one pass; x float32 [rows, width].
-
-    Returns (x_out float32 or x itself when there is no delta, out in `dtype` or None)."""
+    """x + norm(delta), its norm and the norm's convolution over time (each optional) in one pass; x float32 [rows, width],
+    conv float32 [taps, width].  Returns (x_out float32 or x itself when there is no delta, out in `dtype` or None)."""
     _need_gpu(x)
     width = x.shape[-1]
     if x.dtype != torch.float32:
@@ -82,7 +81,7 @@ def norm_conv(x, batch, seqlen, eps, dtype, delta=None, delta_weight=None, delta
             a.x_out = _p(x_out)
     a.norm_weight = _vec(norm_weight, width, "norm_conv norm_weight")
     if conv is not None:
-        taps = conv.shape[-1]
+        taps = conv.shape[0]
         a.taps, a.conv = taps, _vec(conv, width * taps, "norm_conv conv")
         a.input_pos, a.first = _positions(input_pos, first, batch, seqlen, "norm_conv")
         if taps > 1:

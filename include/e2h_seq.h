@@ -36,12 +36,12 @@ extern "C" {
 int e2h_seq_abi_version(void);
 /* Experiment switches (0 = built-in choice): "recurrence_form" 1 = token by token, 2 = chunked; "recurrence_chunk" = tokens a
  * workgroup of the chunked HGRN2 form covers; "norm_run" = tokens a workgroup of the norm kernel covers;
- * "attention_decode_waves" = 4 or 8; "attention_query_tiles" = 1 or 2. */
+ * "attention_decode_waves" = 4 or 8. */
 int e2h_seq_set_option(const char *name, int value);
 
 /* x_out = x + norm(delta); h = norm(x_out); out = h + conv(h), each step optional:
  *   norm(z) = z / sqrt(mean(z^2) + eps) * (offset + weight)
- *   conv(h)[t] = sum_j w[:, j] h[t - taps + 1 + j], zero before the sequence starts.
+ *   conv(h)[t] = sum_j w[j, :] h[t - taps + 1 + j], zero before the sequence starts.
  * delta NULL: x_out = x, not stored.  norm_weight NULL: h = x_out.  conv NULL: out = h.  One of x_out and out may be NULL. */
 typedef struct {
   int32_t dtype; /* of delta and out */
@@ -54,7 +54,7 @@ typedef struct {
   const float *delta_weight; /* [width] */
   float *x_out;              /* [rows, width], different memory from x when seqlen > 1 */
   const float *norm_weight;  /* [width] or NULL */
-  const float *conv;         /* [width, taps] or NULL */
+  const float *conv;         /* [taps, width] or NULL; the last row is the current token's */
   const float *tail_in;      /* [batch, taps, width] */
   float *tail_out;
   void *out;                 /* [rows, width] */

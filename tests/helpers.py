@@ -1,5 +1,8 @@
-"""Shared test helpers: seeded inputs (CPU generator, so every machine sees the same values) and
-torch <-> numpy conversions for bfloat16."""
+"""Shared test helpers: seeded inputs (CPU generator, so every machine sees the same values),
+torch <-> numpy conversions for bfloat16, and checkpoint folders with random weights."""
+
+import json
+import struct
 
 import numpy as np
 import torch
@@ -41,3 +44,97 @@ def weight_with_edge_rows(n, k, g, std=0.02, seed=SEED):
         w[5, 1:g:2] = -0.25
         w[6, :k] = torch.linspace(-1, 1, k).to(torch.bfloat16)  # ramp: many .5 rounding ties
     return w
+
+
+def write_safetensors(path, tensors):
+    names = {torch.bfloat16: "BF16", torch.float32: "F32", torch.int32: "I32"}
+    header, blobs, at = {}, [], 0
+    for name, t in tensors.items():
+        raw = t.contiguous().view(torch.uint8).numpy().tobytes() if t.dim() else bytes(t.view(1).view(torch.uint8).tolist())
+        header[name] = {"dtype": names[t.dtype], "shape": list(t.shape), "data_offsets": [at, at + len(raw)]}
+        blobs.append(raw)
+        at += len(raw)
+    text = json.dumps(header).encode()
+    path.write_bytes(struct.pack("<Q", len(text)) + text + b"".join(blobs))
+
+
+def refatar_parallel(heads=4, kv_heads=2, dim=24, vdim=40, size=9, keep=3, scale=0.3, r_heads=3, r_dim=20, r_vdim=36, left=0.7, right=1.3, ff=88):
+    return {"type": "parallel", "mlp": None if ff is None else {"kind": "dense", "ff": ff},
+            "mixer": {"left": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, "mask": {"size": size, "keep_first": keep}},
+                      "right": {"heads": r_heads, "dim": r_dim, "vdim": r_vdim}, "left_scale": left, "right_scale": right}}
+
+
+def refatar_delta(heads=4, kv_heads=2, dim=24, vdim=20, conv=4, ff=72):
+    return {"type": "delta", "mlp": None if ff is None else {"kind": "dense", "ff": ff},
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}}
+
+
+def refatar_config(layers, vocab=97, width=104, taps=4, side=12, cap=11.0, eps=1e-5):
+    return {"architecture": "Refatar", "vocab": vocab, "width": width, "canon": {"taps": taps}, "norm": {"eps": eps}, "token_side": {"dim": side},
+            "logit_softcap": cap, "layers": layers}
+
+
+def refatar_weights(config, seed=SEED):
+    """Random bfloat16 checkpoint tensors at scales at which every mechanism moves the logits."""
+    g = gen(seed)
+    w, eps, taps, side = config["width"], 0.3, config["canon"]["taps"], config["token_side"]["dim"]
+    out = {}
+
+    def randn(name, *shape, std=1.0, mean=0.0):
+        out[name] = (torch.randn(shape, generator=g) * std + mean).to(torch.bfloat16)
+
+    def lin(name, n, k):
+        randn(name, n, k, std=k ** -0.5)
+
+    randn("embed", config["vocab"], w)
+    randn("side.embed", config["vocab"], side * len(config["layers"]))
+    for i, layer in enumerate(config["layers"]):
+        p, m = f"l{i}", layer["mixer"]
+        subs = ["1"] if layer["mlp"] is None else ["1", "2"]
+        for s in subs:
+            randn(f"{p}.norm{s}", w, std=eps)
+            randn(f"{p}.norm{s}b", w, std=eps)
+            randn(f"{p}.canon{s}", w, taps, std=0.4)
+        if layer["type"] == "parallel":
+            a, r = m["left"], m["right"]
+            for n, rows in (("q", a["heads"] * a["dim"]), ("k", a["kv_heads"] * a["dim"]), ("v", a["kv_heads"] * a["vdim"])):
+                lin(f"{p}.mix.left.{n}", rows, w)
+                randn(f"{p}.mix.left.{n}.b", rows, std=0.5)
+            lin(f"{p}.mix.left.g", a["heads"] * a["vdim"], w)
+            lin(f"{p}.mix.left.o", w, a["heads"] * a["vdim"])
+            rd = r["heads"] * r["dim"]
+            lin(f"{p}.mix.right.q", rd, w)
+            lin(f"{p}.mix.right.f", rd, w)
+            randn(f"{p}.mix.right.f.b", rd, std=2.0, mean=3.0)
+            out[f"{p}.mix.right.lower"] = torch.rand((rd,), generator=g).mul(0.9).to(torch.bfloat16)
+            lin(f"{p}.mix.right.v", r["heads"] * r["vdim"], w)
+            randn(f"{p}.mix.right.norm", r["vdim"], std=0.2, mean=1.0)
+            lin(f"{p}.mix.right.o", w, r["heads"] * r["vdim"])
+        else:
+            qk, hv = m["kv_heads"] * m["dim"], m["heads"] * m["vdim"]
+            for n, rows in (("q", qk), ("k", qk), ("v", hv)):
+                lin(f"{p}.mix.{n}", rows, w)
+                randn(f"{p}.mix.{n}.conv", rows, m["conv"], std=0.7)
+            lin(f"{p}.mix.b", m["heads"], w)
+            lin(f"{p}.mix.a", m["heads"], w)
+            out[f"{p}.mix.A_log"] = torch.rand((m["heads"],), generator=g).mul(-4).to(torch.bfloat16)
+            randn(f"{p}.mix.dt_bias", m["heads"], std=0.5, mean=-2.0)
+            randn(f"{p}.mix.norm", m["vdim"], std=0.2, mean=1.0)
+            lin(f"{p}.mix.g", hv, w)
+            lin(f"{p}.mix.o", w, hv)
+        if layer["mlp"] is not None:
+            lin(f"{p}.mlp.up", layer["mlp"]["ff"], w)
+            lin(f"{p}.mlp.down", w, layer["mlp"]["ff"])
+        lin(f"{p}.side.gate", side, w)
+        lin(f"{p}.side.proj", w, side)
+        randn(f"{p}.side.norm", w, std=0.2, mean=0.5)
+    randn("final.norm", w, std=eps)
+    lin("head", config["vocab"], w)
+    out["head"] = out["head"] * 3
+    return out
+
+
+def write_checkpoint_folder(folder, config, weights):
+    (folder / "config.json").write_text(json.dumps(config))
+    write_safetensors(folder / "model.safetensors", weights)
+    return folder

@@ -1,0 +1,626 @@
+"""The Refatar decoder on the GPU against the plain implementation in oracle/refatar_oracle.py: every mechanism alone, whole models
+in float32 and bfloat16, prompts against token-by-token decoding and against portions, sequences side by side, reused rows, and
+generation through the package's own entry points."""
+
+import io
+import json
+
+import numpy as np
+import pytest
+import torch
+
+from easy_to_hard_amd import _lib, generate, seq_ops
+from easy_to_hard_amd.state import KVCache
+from oracle import refatar_oracle as ro
+from tests import helpers as hp
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+BOTH = pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16], ids=["f32", "bf16"])
+
+
+@pytest.fixture(autouse=True)
+def _default_options():
+    yield
+    for name in ("recurrence_form", "recurrence_chunk", "norm_run", "attention_decode_waves"):
+        _lib.set_seq_option(name, 0)
+
+
+def rel(got, want):
+    got, want = np.asarray(got, dtype=np.float64), np.asarray(want, dtype=np.float64)
+    return np.abs(got - want).max() / max(np.abs(want).max(), 1e-30)
+
+
+def f64(t):
+    return t.detach().double().cpu().numpy()
+
+
+def positions(start, n):
+    return torch.arange(start, start + n, device=DEV)
+
+
+def randn(*shape, seed=0, std=1.0, dtype=torch.float32):
+    """values that bfloat16 holds exactly, so that both precisions see the same inputs"""
+    g = torch.Generator().manual_seed(seed)
+    return (torch.randn(shape, generator=g) * std).to(torch.bfloat16).to(dtype).to(DEV)
+
+
+# ---- norm, residual, input convolution -----------------------------------------------------------------------------------------
+
+@BOTH
+@pytest.mark.parametrize("width,taps,run", [(64, 4, 0), (100, 3, 2), (1028, 2, 5), (2048, 1, 0), (2056, 4, 3), (4100, 6, 2), (64, 8, 1)])
+def test_norm_conv_over_portions(dtype, width, taps, run):
+    t, eps = 23, 1e-4
+    x, d = randn(t, width, seed=1), randn(t, width, seed=2, dtype=dtype)
+    wd, wn, wc = randn(width, seed=3, std=0.3), randn(width, seed=4, std=0.3), randn(width, taps, seed=5, std=0.5)
+    x_ref = f64(x) + ro.zero_centred_rms_norm(f64(d), f64(wd), eps)
+    want = ro.canon(ro.zero_centred_rms_norm(x_ref, f64(wn), eps), f64(wc))
+    conv = wc.t().contiguous()
+    _lib.set_seq_option("norm_run", run)
+    live, nxt = torch.full((2, taps, width), 7.0, device=DEV), torch.full((2, taps, width), 9.0, device=DEV)
+    at, outs, xs = 0, [], []
+    for n in (1, 2, 1, 11, 3, 5):  # old contents of the rings must not matter at position 0
+        xo, y = seq_ops.norm_conv(x[at: at + n].clone(), 1, n, eps, dtype, delta=d[at: at + n].clone(), delta_weight=wd, delta_offset=1.0,
+                                  norm_weight=wn, norm_offset=1.0, conv=conv, tails=(live, live if n == 1 else nxt), input_pos=positions(at, n))
+        if n > 1:
+            live.copy_(nxt)
+        xs.append(xo)
+        outs.append(y)
+        at += n
+    assert at == t
+    assert rel(f64(torch.cat(xs)), x_ref) < 2e-6
+    assert rel(f64(torch.cat(outs)), want) < (3e-6 if dtype == torch.float32 else 6e-3)
+
+
+@BOTH
+def test_norm_conv_parts_and_padding(dtype):
+    b, t, width, taps, eps = 3, 9, 72, 3, 1e-5
+    x, d = randn(b * t, width, seed=1), randn(b * t, width, seed=2, dtype=dtype)
+    w, wn, wc = randn(width, seed=3, std=0.3), randn(width, seed=4, std=0.3), randn(width, taps, seed=5)
+    xo, y = seq_ops.norm_conv(x, b, t, eps, dtype, delta=d, delta_weight=w)     # plain weight, no second norm: y is the new x
+    want = f64(x) + ro.rms(f64(d), eps) * f64(w)
+    assert rel(f64(xo), want) < 2e-6 and rel(f64(y), want) < (2e-6 if dtype == torch.float32 else 4e-3)
+    xo, y = seq_ops.norm_conv(x, b, t, eps, dtype, norm_weight=wn, norm_offset=1.0)
+    assert xo is x and rel(f64(y), ro.zero_centred_rms_norm(f64(x), f64(wn), eps)) < (2e-6 if dtype == torch.float32 else 4e-3)
+    first = torch.tensor([0, 4, 8], device=DEV)
+    tails = (torch.full((b, taps, width), 5.0, device=DEV), torch.zeros((b, taps, width), device=DEV))
+    _, y = seq_ops.norm_conv(x, b, t, eps, dtype, norm_weight=wn, norm_offset=1.0, conv=wc.t().contiguous(), tails=tails, input_pos=positions(0, t),
+                             first=first)
+    for i, f in enumerate(first.tolist()):
+        h = ro.zero_centred_rms_norm(f64(x).reshape(b, t, width)[i, f:], f64(wn), eps)
+        assert rel(f64(y).reshape(b, t, width)[i, f:], ro.canon(h, f64(wc))) < (3e-6 if dtype == torch.float32 else 6e-3)
+
+
+@BOTH
+def test_elementwise_steps(dtype):
+    x = randn(5, 203, std=3.0, dtype=dtype)
+    tol = 3e-6 if dtype == torch.float32 else 5e-3
+    assert rel(f64(seq_ops.square_relu_(x.clone())), np.square(np.maximum(f64(x), 0))) < tol
+    assert rel(f64(seq_ops.softcap_(x.clone(), 2.5)), ro.softcap(f64(x), 2.5)) < tol
+    table, tok = randn(11, 60, seed=1, dtype=dtype), torch.tensor([3, 0, 10, 10, 7], device=DEV)
+    gate = randn(5, 20, seed=2, dtype=dtype, std=2.0)
+    want = ro.gelu_tanh(f64(gate)) * f64(table)[tok.cpu().numpy(), 40:60]
+    assert rel(f64(seq_ops.gelu_gate_rows(gate, table, tok, 40)), want) < tol
+
+
+# ---- windowed attention --------------------------------------------------------------------------------------------------------
+
+def run_attention(q, k, v, gate, dtype, scale, window, keep, portions, biases=(None, None, None), first=None, cache=None, out_scale=1.0):
+    """q, k, v, gate [B, T, heads, size] -> output [B, T, H, Dv] through the kernel, portion by portion."""
+    b, t, h, d = q.shape
+    g, dv = k.shape[2], v.shape[3]
+    cache = cache if cache is not None else KVCache(b, t + 3, g, d, dtype, DEV, dv)
+    pad = lambda n: (n + 7) // 8 * 8  # noqa: E731
+    offs, at = [], 0
+    for n in (h * d, g * d, g * dv, h * dv):
+        offs.append(at)
+        at = pad(at + n)
+    outs, pos = [], 0
+    for n in portions:
+        proj = torch.full((b, n, at), 100.0, dtype=dtype, device=DEV)
+        for src, o in zip((q, k, v, gate), offs):
+            if src is not None:
+                proj[:, :, o: o + src.shape[2] * src.shape[3]] = src[:, pos: pos + n].reshape(b, n, -1)
+        out = torch.zeros((b * n, h * dv + 8), dtype=dtype, device=DEV)
+        o4 = (*offs[:3], offs[3] if gate is not None else -1)
+        seq_ops.window_attention(proj.view(b * n, at), b, n, h, g, d, dv, o4, biases, cache, positions(pos, n), first, window, keep, scale, out, 8,
+                                 out_scale)
+        outs.append(out[:, 8:].reshape(b, n, h, dv))
+        pos += n
+    return torch.cat(outs, dim=1)
+
+
+SHAPES = [(4, 2, 32, 32), (3, 1, 20, 12), (5, 5, 48, 72), (8, 1, 64, 128), (6, 3, 128, 40), (2, 1, 136, 200), (20, 1, 16, 16)]
+
+
+@BOTH
+@pytest.mark.parametrize("h,g,d,dv", SHAPES)
+def test_window_attention_shapes(dtype, h, g, d, dv):
+    t, window, keep, scale = 150, 37, 5, 1.4 / d ** 0.5
+    q, k, v, gate = (randn(1, t, n, s, seed=i, dtype=dtype) for i, (n, s) in enumerate(((h, d), (g, d), (g, dv), (h, dv))))
+    bias = tuple(randn(n, seed=10 + i, std=0.5) for i, n in enumerate((h * d, g * d, g * dv)))
+    want = ro.window_attention(f64(q)[0] + f64(bias[0]).reshape(h, d), f64(k)[0] + f64(bias[1]).reshape(g, d), f64(v)[0] + f64(bias[2]).reshape(g, dv),
+                               scale, window, keep) * ro.sigmoid(f64(gate)[0]) * 0.6
+    tol = 5e-6 if dtype == torch.float32 else 1.5e-2
+    whole = run_attention(q, k, v, gate, dtype, scale, window, keep, [t], bias, out_scale=0.6)
+    assert rel(f64(whole)[0], want) < tol
+    mixed = run_attention(q, k, v, gate, dtype, scale, window, keep, [100, 2, 3, 1, 1, 13] + [1] * 30, bias, out_scale=0.6)
+    assert rel(f64(mixed)[0], want) < tol
+
+
+@BOTH
+@pytest.mark.parametrize("window,keep", [(1, 0), (1, 3), (6, 0), (16, 1), (33, 20), (64, 64), (500, 2), (0, 0)])
+def test_window_edges_with_one_key_that_stands_out(dtype, window, keep):
+    """One key scores far above all others: the output is its value wherever it is visible and has no trace of it elsewhere.
+    The key is put just inside and just outside the window and the kept first tokens, in prompts and in decoding."""
+    t, h, g, d = 131, 2, 1, 32
+    size = window if window > 0 else 10 ** 9
+    last = t - 1
+    places = {last - size + 1, last - size, keep - 1, keep, 0, last, last - 1, 63, 64}
+    for j in sorted(p for p in places if 0 <= p < t):
+        q = torch.zeros((1, t, h, d), dtype=dtype, device=DEV)
+        q[..., 0] = 1.0
+        k, v = randn(1, t, g, d, seed=j, std=0.1, dtype=dtype), randn(1, t, g, d, seed=j + 1, std=0.1, dtype=dtype)
+        k[0, j, 0, 0] = 40.0
+        v[0, j] += 16.0
+        want = ro.window_attention(f64(q)[0], f64(k)[0], f64(v)[0], 1.0, size, keep)
+        for portions in ([t], [60, 2, 40] + [1] * 29):
+            got = f64(run_attention(q, k, v, None, dtype, 1.0, window, keep, portions))[0]
+            seen = np.array([ro.window_visible(i, j, size, keep) for i in range(t)])
+            assert (np.abs(got[seen, :, :] - 16.0) < 1.0).all(), (j, portions)
+            assert (np.abs(got[~seen, :, :]) < 1.0).all(), (j, portions)
+            assert rel(got, want) < (1e-5 if dtype == torch.float32 else 1e-2)
+
+
+@BOTH
+def test_attention_of_padded_and_shorter_sequences_side_by_side(dtype):
+    b, t, h, g, d, dv, window, keep = 3, 90, 4, 2, 32, 48, 11, 4
+    q, k, v = (randn(b, t, n, s, seed=i, dtype=dtype) for i, (n, s) in enumerate(((h, d), (g, d), (g, dv))))
+    first = torch.tensor([0, 17, 70], device=DEV)
+    got = f64(run_attention(q, k, v, None, dtype, 0.2, window, keep, [80, 2] + [1] * 8, first=first))
+    for i, f in enumerate(first.tolist()):
+        want = ro.window_attention(f64(q)[i, f:], f64(k)[i, f:], f64(v)[i, f:], 0.2, window, keep)
+        assert rel(got[i, f:], want) < (5e-6 if dtype == torch.float32 else 1.5e-2)
+
+
+def test_attention_ignores_what_an_earlier_sequence_left_in_the_cache():
+    t, d = 40, 32
+    cache = KVCache(1, 64, 1, d, torch.bfloat16, DEV)
+    cache.k_cache.fill_(30.0)
+    cache.v_cache.fill_(1e4)
+    q, k, v = (randn(1, t, 1, d, seed=i, dtype=torch.bfloat16) for i in range(3))
+    got = f64(run_attention(q, k, v, None, torch.bfloat16, 0.2, 64, 2, [30] + [1] * 10, cache=cache))[0]
+    assert rel(got, ro.window_attention(f64(q)[0], f64(k)[0], f64(v)[0], 0.2, 64, 2)) < 1.5e-2
+
+
+@pytest.mark.parametrize("waves", [4, 8])
+def test_decode_attention_over_many_keys_with_either_wave_count(waves):
+    """600 keys: several tiles per wave, and the far keys carry most of the weight."""
+    _lib.set_seq_option("attention_decode_waves", waves)
+    t, h, g, d = 601, 4, 2, 64
+    q, k, v = (randn(1, t, n, d, seed=i, dtype=torch.bfloat16) for i, n in enumerate((h, g, g)))
+    k[0, 5:40] += 0.5 * q[0, -1, 0]
+    want = ro.window_attention(f64(q)[0], f64(k)[0], f64(v)[0], 0.3, 580, 30)
+    got = f64(run_attention(q, k, v, None, torch.bfloat16, 0.3, 580, 30, [600, 1]))[0]
+    assert rel(got[-1], want[-1]) < 1e-2
+
+
+# ---- HGRN2 -----------------------------------------------------------------------------------------------------------------------
+
+def run_hgrn2(q, f, v, fb, low, nw, eps, dtype, portions, first=None, state=None, out_scale=1.0):
+    b, t, h, d = q.shape
+    dv = v.shape[3]
+    state = state if state is not None else torch.full((b, h, d, dv), 3.0, device=DEV)  # stale contents: position 0 starts empty
+    outs, pos = [], 0
+    cols = (0, (h * d + 7) // 8 * 8, 2 * ((h * d + 7) // 8 * 8))
+    ld = (cols[2] + h * dv + 7) // 8 * 8
+    for n in portions:
+        proj = torch.full((b, n, ld), 50.0, dtype=dtype, device=DEV)
+        for src, c in zip((q, f, v), cols):
+            proj[:, :, c: c + src.shape[2] * src.shape[3]] = src[:, pos: pos + n].reshape(b, n, -1)
+        out = torch.zeros((b * n, h * dv + 4), dtype=dtype, device=DEV)
+        seq_ops.hgrn2(proj.view(b * n, ld), b, n, h, d, dv, cols, fb, low, nw, eps, state, positions(pos, n), first, out, 4, out_scale)
+        outs.append(out[:, 4:].reshape(b, n, h, dv))
+        pos += n
+    return torch.cat(outs, dim=1), state
+
+
+def want_hgrn2(q, f, v, fb, low, nw, eps):
+    h, d = q.shape[1:]
+    lo = f64(low).reshape(h, d)
+    gate = lo + (1 - lo) * ro.sigmoid(f64(f) + f64(fb).reshape(h, d))
+    o, s = ro.hgrn2_recurrence(ro.silu(f64(q)), gate, f64(v))
+    return ro.rms(o, eps) * f64(nw), s
+
+
+@BOTH
+@pytest.mark.parametrize("form", [0, 1, 2])
+@pytest.mark.parametrize("h,d,dv,t", [(2, 16, 16, 3), (3, 20, 36, 70), (2, 64, 64, 33), (2, 72, 128, 65), (1, 128, 100, 130), (1, 200, 24, 40),
+                                      (1, 144, 256, 21), (1, 32, 132, 50), (2, 18, 8, 40), (1, 256, 256, 18)])
+def test_hgrn2_shapes(dtype, form, h, d, dv, t):
+    _lib.set_seq_option("recurrence_form", form)
+    eps = 1e-5
+    q, f, v = randn(1, t, h, d, seed=1, dtype=dtype), randn(1, t, h, d, seed=2, dtype=dtype, std=2.0), randn(1, t, h, dv, seed=3, dtype=dtype)
+    fb, low, nw = randn(h * d, seed=4, std=2.0), randn(h * d, seed=5).abs().clamp(max=0.9), randn(dv, seed=6) + 1
+    low[::3] = 0.0
+    want, s = want_hgrn2(q[0], f[0], v[0], fb, low, nw, eps)
+    for portions in ([t], [max(1, t - 20)] + [2] * ((t - max(1, t - 20)) // 2) + [1] * ((t - max(1, t - 20)) % 2)):
+        got, state = run_hgrn2(q, f, v, fb, low, nw, eps, dtype, portions, out_scale=0.5)
+        assert rel(f64(got)[0], 0.5 * want) < (2e-5 if dtype == torch.float32 else 6e-3), portions
+        assert rel(f64(state)[0], s) < 1e-5
+    assert rel(f64(run_hgrn2(q, f, v, fb, low, nw, eps, dtype, [1] * t, out_scale=0.5)[0])[0], 0.5 * want) < (2e-5 if dtype == torch.float32 else 6e-3)
+
+
+@pytest.mark.parametrize("form", [1, 2])
+@pytest.mark.parametrize("chunk", [64, 128])
+def test_hgrn2_gates_at_their_ends(form, chunk):
+    """Gates that forget everything next to gates that forget nothing, within one block and across blocks: what a channel with
+    f = 1 wrote 300 tokens ago is still there, a channel with f = 0 holds the last token only."""
+    _lib.set_seq_option("recurrence_form", form)
+    _lib.set_seq_option("recurrence_chunk", chunk)
+    t, h, d, dv = 330, 1, 16, 16
+    q, v = randn(1, t, h, d, seed=1).abs() + 0.5, randn(1, t, h, dv, seed=3)
+    f = torch.zeros((1, t, h, d), device=DEV)
+    f[..., 0] = -60.0                      # f = 0
+    f[..., 1] = 60.0                       # f = 1: nothing is written
+    f[..., 2] = 9.0                        # f = 1 - 1e-4
+    f[0, :, 0, 3] = torch.where(torch.arange(t, device=DEV) % 7 == 3, -60.0, 20.0)
+    f[0, 20, 0, 4:8] = -30.0
+    f[..., 8:] = 12.0
+    f[0, 5, 0, 8:] = -20.0                 # one early write that stays
+    v[0, 5] = 50.0
+    fb, low, nw = torch.zeros(h * d, device=DEV), torch.zeros(h * d, device=DEV), torch.ones(dv, device=DEV)
+    low[9] = 0.5
+    low[10] = 1.0                          # lower bound one: never writes
+    want, s = want_hgrn2(q[0], f[0], v[0], fb, low, nw, 1e-6)
+    got, state = run_hgrn2(q, f, v, fb, low, nw, 1e-6, torch.float32, [200, 100, 30])
+    assert torch.isfinite(got).all()
+    out_err, state_err = rel(f64(got)[0], want), rel(f64(state)[0], s)
+    assert out_err < 2e-5 and state_err < 1e-5
+    assert want[-1].mean() > 0.5           # the early write dominates the last read-out, so losing it would show
+
+
+@BOTH
+@pytest.mark.parametrize("form", [1, 2])
+def test_hgrn2_batches_padding_and_reused_rows(dtype, form):
+    _lib.set_seq_option("recurrence_form", form)
+    b, t, h, d, dv, eps = 3, 80, 2, 24, 20, 1e-5
+    q, f, v = (randn(b, t, h, s, seed=i, dtype=dtype) for i, s in enumerate((d, d, dv)))
+    fb, low, nw = randn(h * d, seed=4), randn(h * d, seed=5).abs().clamp(max=0.9), randn(dv, seed=6) + 1
+    first = torch.tensor([0, 33, 79], device=DEV)
+    got, state = run_hgrn2(q, f, v, fb, low, nw, eps, dtype, [50, 30], first=first)
+    for i, s0 in enumerate(first.tolist()):
+        want, s = want_hgrn2(q[i, s0:], f[i, s0:], v[i, s0:], fb, low, nw, eps)
+        assert rel(f64(got)[i, s0:], want) < (2e-5 if dtype == torch.float32 else 6e-3) and rel(f64(state)[i], s) < 1e-5
+    again, _ = run_hgrn2(q[:1], f[:1], v[:1], fb, low, nw, eps, dtype, [80], state=state)  # row 0 starts over on used state
+    assert rel(f64(again)[0], f64(got)[0]) < (2e-5 if dtype == torch.float32 else 6e-3)
+
+
+# ---- gated delta rule --------------------------------------------------------------------------------------------------------------
+
+def delta_case(b, t, heads, kvh, d, dv, taps, dtype, seed=0, decay=1.0):
+    x = {n: randn(b, t, w, seed=seed + i, dtype=dtype) for i, (n, w) in enumerate((("q", kvh * d), ("k", kvh * d), ("v", heads * dv), ("b", heads),
+                                                                                  ("a", heads), ("g", heads * dv)))}
+    c = {n: randn(w, taps, seed=seed + 10 + i, std=0.7) for i, (n, w) in enumerate((("q", kvh * d), ("k", kvh * d), ("v", heads * dv)))}
+    p = {"a_log": randn(heads, seed=seed + 20) - 1.5 * decay, "dt": randn(heads, seed=seed + 21) - decay, "norm": randn(dv, seed=seed + 22, std=0.2) + 1}
+    return x, c, p
+
+
+def run_delta(x, c, p, heads, kvh, d, dv, taps, eps, dtype, portions, first=None, state=None, rings=None):
+    b = x["q"].shape[0]
+    ch = 2 * kvh * d + heads * dv
+    state = state if state is not None else torch.full((b, heads, d, dv), 3.0, device=DEV)
+    live, nxt = rings if rings is not None else (torch.full((b, taps, ch), 9.0, dtype=dtype, device=DEV), torch.full((b, taps, ch), 8.0, dtype=dtype, device=DEV))
+    conv = torch.cat([c["q"], c["k"], c["v"]])
+    offs, at = [], 0
+    for n in "qkvbag":
+        offs.append(at)
+        at = (at + x[n].shape[2] + 7) // 8 * 8
+    outs, pos = [], 0
+    for n in portions:
+        proj = torch.full((b, n, at), 30.0, dtype=dtype, device=DEV)
+        for name, o in zip("qkvbag", offs):
+            proj[:, :, o: o + x[name].shape[2]] = x[name][:, pos: pos + n]
+        out = torch.zeros((b * n, heads * dv + 4), dtype=dtype, device=DEV)
+        seq_ops.gated_delta(proj.view(b * n, at), b, n, heads, kvh, d, dv, offs, conv, (live, live if n == 1 else nxt), p["a_log"], p["dt"], p["norm"], eps,
+                            state, positions(pos, n), first, out, 4)
+        if n > 1:
+            live.copy_(nxt)
+        outs.append(out[:, 4:].reshape(b, n, heads, dv))
+        pos += n
+    return torch.cat(outs, dim=1), state
+
+
+def want_delta(x, c, p, heads, kvh, d, dv, eps, i=0, start=0):
+    y = {n: ro.silu(ro.causal_conv(f64(x[n])[i, start:], f64(c[n]))) for n in "qkv"}
+    t = y["q"].shape[0]
+    q, k = ro.unit(y["q"].reshape(t, kvh, d)) * d ** -0.5, ro.unit(y["k"].reshape(t, kvh, d))
+    of = np.arange(heads) // (heads // kvh)
+    beta = ro.sigmoid(f64(x["b"])[i, start:])
+    g = np.exp(-np.exp(f64(p["a_log"])) * ro.softplus(f64(x["a"])[i, start:] + f64(p["dt"])))
+    o, s = ro.delta_recurrence(q[:, of], k[:, of], y["v"].reshape(t, heads, dv), g, beta)
+    return ro.rms(o, eps) * f64(p["norm"]) * ro.silu(f64(x["g"])[i, start:].reshape(t, heads, dv)), s
+
+
+@BOTH
+@pytest.mark.parametrize("form", [0, 1, 2])
+@pytest.mark.parametrize("heads,kvh,d,dv,taps,t", [(2, 2, 16, 16, 4, 5), (4, 2, 24, 20, 4, 70), (6, 2, 64, 40, 3, 64), (2, 1, 128, 72, 2, 65), (3, 3, 20, 12, 1, 129),
+                                                   (2, 1, 68, 128, 4, 130), (1, 1, 160, 48, 4, 80), (2, 1, 30, 8, 5, 60), (1, 1, 256, 256, 4, 70),
+                                                   (2, 2, 32, 24, 6, 40)])
+def test_delta_shapes(dtype, form, heads, kvh, d, dv, taps, t):
+    _lib.set_seq_option("recurrence_form", form)
+    eps = 1e-5
+    x, c, p = delta_case(1, t, heads, kvh, d, dv, taps, dtype)
+    want, s = want_delta(x, c, p, heads, kvh, d, dv, eps)
+    tol, stol = (4e-5, 2e-5) if dtype == torch.float32 else (8e-3, 2e-5)
+    for portions in ([t], [2, 1, t - 10, 3, 2, 2] if t > 12 else [2, t - 2]):
+        got, state = run_delta(x, c, p, heads, kvh, d, dv, taps, eps, dtype, portions)
+        assert rel(f64(got)[0], want) < tol and rel(f64(state)[0], s) < stol, portions
+    got, state = run_delta(x, c, p, heads, kvh, d, dv, taps, eps, dtype, [1] * t)
+    assert rel(f64(got)[0], want) < tol and rel(f64(state)[0], s) < stol
+
+
+@pytest.mark.parametrize("form", [1, 2])
+def test_delta_keeps_a_far_write_and_corrects_repeated_keys(form):
+    """Decay close to one and an early large value: it is read 250 tokens later.  Half the tokens repeat one key, which makes
+    the corrections inside a chunk as large as the values."""
+    _lib.set_seq_option("recurrence_form", form)
+    heads, kvh, d, dv, taps, t = 2, 1, 16, 16, 2, 260
+    x, c, p = delta_case(1, t, heads, kvh, d, dv, taps, torch.float32)
+    p["a_log"].fill_(-8.0)
+    c["k"].zero_()
+    c["k"][:, -1] = 1.0
+    same = torch.arange(t, device=DEV) % 2 == 1
+    x["k"][0, same] = 0.0
+    x["k"][0, same, :3] = 4.0
+    x["b"].fill_(4.0)
+    x["k"][0, 6] = 0.0
+    x["k"][0, 6, 9] = 6.0
+    x["k"][0, 7:, 9] = 0.0                    # nobody else touches that channel's key
+    x["v"][0, 6] = 90.0
+    c["v"] = c["v"].abs() + 0.4
+    x["q"][0, -1] = 0.0
+    x["q"][0, -2] = 0.0
+    x["q"][0, -1, 9] = 6.0
+    c["q"].zero_()
+    c["q"][:, -1] = 1.0
+    want, s = want_delta(x, c, p, heads, kvh, d, dv, 1e-6)
+    got, state = run_delta(x, c, p, heads, kvh, d, dv, taps, 1e-6, torch.float32, [130, 100, 30])
+    out_err, state_err, held = rel(f64(got)[0], want), rel(f64(state)[0], s), float(np.abs(s[:, 9]).min())
+    assert out_err < 1e-4 and state_err < 5e-5
+    assert held > 20                         # the far write is what the state holds there
+
+
+@BOTH
+@pytest.mark.parametrize("form", [1, 2])
+def test_delta_batches_padding_and_reused_rows(dtype, form):
+    _lib.set_seq_option("recurrence_form", form)
+    b, t, heads, kvh, d, dv, taps, eps = 3, 90, 4, 2, 24, 20, 4, 1e-5
+    x, c, p = delta_case(b, t, heads, kvh, d, dv, taps, dtype)
+    first = torch.tensor([0, 41, 89], device=DEV)
+    got, state = run_delta(x, c, p, heads, kvh, d, dv, taps, eps, dtype, [60, 1, 27, 2], first=first)
+    tol = 4e-5 if dtype == torch.float32 else 8e-3
+    for i, s0 in enumerate(first.tolist()):
+        want, s = want_delta(x, c, p, heads, kvh, d, dv, eps, i, s0)
+        assert rel(f64(got)[i, s0:], want) < tol and rel(f64(state)[i], s) < 2e-5
+    one = {n: v[:1].contiguous() for n, v in x.items()}
+    again, _ = run_delta(one, c, p, heads, kvh, d, dv, taps, eps, dtype, [3, 1, 86], state=state)
+    assert rel(f64(again)[0], f64(got)[0]) < tol
+
+
+# ---- whole models ------------------------------------------------------------------------------------------------------------------
+
+CONFIGS = {
+    "mixed": hp.refatar_config([hp.refatar_parallel(), hp.refatar_delta(), hp.refatar_parallel(heads=2, kv_heads=1, dim=32, vdim=16, size=30, keep=0, ff=None)]),
+    "delta-first": hp.refatar_config([hp.refatar_delta(heads=3, kv_heads=1, dim=40, vdim=28, conv=3), hp.refatar_delta(heads=2, kv_heads=2, conv=1, ff=None),
+                                      hp.refatar_parallel(heads=3, kv_heads=3, dim=16, vdim=48, size=1, keep=6, r_heads=1, r_dim=64, r_vdim=12)],
+                                     vocab=61, width=72, taps=2, side=5, cap=4.0),
+    "parallel": hp.refatar_config([hp.refatar_parallel(heads=6, kv_heads=1, dim=12, vdim=20, size=17, keep=2, r_heads=4, r_dim=16, r_vdim=16),
+                                   hp.refatar_parallel(left=1.0, right=0.25)], vocab=130, width=136, taps=5, side=16, cap=30.0),
+}
+
+
+def load(tmp_path, name, dtype):
+    cfg = CONFIGS[name]
+    w = hp.refatar_weights(cfg)
+    hp.write_checkpoint_folder(tmp_path, cfg, w)
+    return generate.load_model(tmp_path, DEV, dtype), cfg, {n: t.float().numpy() for n, t in w.items()}
+
+
+def tokens_for(cfg, n, seed=3):
+    return torch.randint(0, cfg["vocab"], (n,), generator=torch.Generator().manual_seed(seed))
+
+
+def feed(model, rows, portions, left_pad=None):
+    rows = torch.as_tensor(rows, device=DEV)
+    at, outs = 0, []
+    for n in portions:
+        outs.append(generate.extend(model, rows[:, at: at + n], at, left_pad).float())
+        at += n
+    return torch.cat(outs, dim=1)
+
+
+def rms_error(got, want):
+    d = np.asarray(got, np.float64) - want
+    d -= d.mean(-1, keepdims=True)
+    return np.sqrt((d ** 2).mean(-1)).max() / want.std()
+
+
+PORTIONS = [[150], [1] * 150, [2] * 75, [100] + [1] * 50, [3, 2, 40, 1, 25, 1, 1, 64, 2, 11]]
+
+
+@BOTH
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_model_equals_the_plain_implementation_for_every_cut(tmp_path, name, dtype):
+    model, cfg, w = load(tmp_path, name, dtype)
+    toks = tokens_for(cfg, 150)
+    want, _ = ro.forward(cfg, w, toks.numpy())
+    model.setup_caches(1, 160)
+    tol = 2e-5 if dtype == torch.float32 else 6e-2
+    for portions in PORTIONS:
+        got = feed(model, toks[None], portions)[0].cpu().numpy()
+        assert rms_error(got, want) < tol, portions
+        assert (np.abs(got) <= cfg["logit_softcap"] + 1e-6).all()
+
+
+@BOTH
+def test_unequal_sequences_side_by_side_equal_each_alone(tmp_path, dtype):
+    model, cfg, w = load(tmp_path, "mixed", dtype)
+    model.setup_caches(4, 128)
+    lengths, total = [90, 57, 3, 88], 90
+    rows, pad = torch.zeros((4, total), dtype=torch.int64), torch.tensor([total - n for n in lengths], device=DEV)
+    for i, n in enumerate(lengths):
+        rows[i, total - n:] = tokens_for(cfg, n, seed=10 + i)
+    got = feed(model, rows, [70, 2, 1, 16, 1], pad).cpu().numpy()
+    for i, n in enumerate(lengths):
+        want, _ = ro.forward(cfg, w, rows[i, total - n:].numpy())
+        assert rms_error(got[i, total - n:], want) < (2e-5 if dtype == torch.float32 else 6e-2), i
+
+
+def test_a_row_is_reused_by_shorter_and_longer_sequences(tmp_path):
+    model, cfg, w = load(tmp_path, "mixed", torch.float32)
+    model.setup_caches(2, 200)
+    for i, n in enumerate((120, 2, 1, 70, 200)):
+        toks = tokens_for(cfg, n, seed=20 + i)
+        want, _ = ro.forward(cfg, w, toks.numpy())
+        got = feed(model, toks[None], [n] if i % 2 else [n // 2, n - n // 2] if n > 1 else [1])[0].cpu().numpy()
+        assert rms_error(got, want) < 2e-5, n
+    both = torch.stack([tokens_for(cfg, 50, seed=30), tokens_for(cfg, 50, seed=31)])
+    got = feed(model, both, [20, 30]).cpu().numpy()   # a call with more rows after calls with one
+    for i in range(2):
+        assert rms_error(got[i], ro.forward(cfg, w, both[i].numpy())[0]) < 2e-5
+
+
+def test_a_pass_without_state_equals_the_cached_one_and_leaves_the_state_alone(tmp_path):
+    model, cfg, w = load(tmp_path, "mixed", torch.float32)
+    model.setup_caches(1, 80)
+    toks = tokens_for(cfg, 60)
+    feed(model, toks[None], [40])
+    free = model(toks[None].to(DEV), fully_causal=True)
+    rest = generate.extend(model, toks[None, 40:].to(DEV), 40)
+    want, _ = ro.forward(cfg, w, toks.numpy())
+    assert rms_error(free[0].cpu().numpy(), want) < 2e-5 and rms_error(rest[0].cpu().numpy(), want[40:]) < 2e-5
+
+
+@BOTH
+def test_greedy_generation_follows_the_plain_implementation(tmp_path, dtype):
+    """generate() with the graph-replayed step: every token is the plain implementation's arg-max on the same prefix wherever its
+    lead exceeds the rounding noise; the graph's steps equal eager steps."""
+    model, cfg, w = load(tmp_path, "mixed", dtype)
+    prompt = torch.stack([tokens_for(cfg, 40, seed=40 + i) for i in range(2)]).to(DEV)
+    seq = generate.generate(model, prompt, 90)
+    eager = generate.generate(model, prompt, 90, use_graph=False)
+    assert torch.equal(seq, eager)
+    noise, checked = (1e-3, 0) if dtype == torch.float32 else (0.5, 0)
+    for i in range(2):
+        logits, _ = ro.forward(cfg, w, seq[i].cpu().numpy())
+        for t in range(39, 129):
+            top = np.sort(logits[t])[-2:]
+            if top[1] - top[0] > noise:
+                checked += 1
+                assert int(seq[i, t + 1]) == int(logits[t].argmax()), (i, t)
+    assert checked > 60
+
+
+def test_graph_replays_equal_eager_steps_between_other_work(tmp_path):
+    model, cfg, _ = load(tmp_path, "mixed", torch.bfloat16)
+    model.setup_caches(3, 96)
+    rows = torch.stack([tokens_for(cfg, 60, seed=50 + i) for i in range(3)]).to(DEV)
+    stepper = generate.GraphedDecodeStep(model, 3, DEV)
+    want = generate.extend(model, rows, 0)[:, 29:].argmax(-1)
+    generate.extend(model, rows[:, :30], 0)
+    for t in range(30, 60):
+        got = stepper.step(rows[:, t: t + 1], torch.tensor([t], device=DEV)).clone()
+        torch.randn(1000, 1000, device=DEV).sum().item()  # eager work and a synchronisation between replays
+        logits = want[:, t - 29]
+        assert (got[:, 0] == logits).float().mean() >= 2 / 3  # portions round differently in bfloat16; ties may flip
+    generate.extend(model, rows[:, :30], 0)
+    for t in range(30, 60):
+        a = generate.decode_one_token(model, rows[:, t: t + 1], torch.tensor([t], device=DEV))
+    generate.extend(model, rows[:, :30], 0)
+    for t in range(30, 60):
+        b = stepper.step(rows[:, t: t + 1], torch.tensor([t], device=DEV))
+    assert torch.equal(a, b)
+
+
+def test_left_padded_generation_equals_each_sequence_alone(tmp_path):
+    model, cfg, _ = load(tmp_path, "delta-first", torch.float32)
+    a, b = tokens_for(cfg, 30, seed=60), tokens_for(cfg, 12, seed=61)
+    rows = torch.zeros((2, 30), dtype=torch.int64)
+    rows[0], rows[1, 18:] = a, b
+    both = generate.generate(model, rows.to(DEV), 40, left_pad_mask_pos=torch.tensor([0, 18], device=DEV))
+    assert torch.equal(both[0], generate.generate(model, a[None].to(DEV), 40)[0])
+    assert torch.equal(both[1, 18:], generate.generate(model, b[None].to(DEV), 40)[0])
+
+
+def test_sampling_through_the_generation_path(tmp_path):
+    model, cfg, _ = load(tmp_path, "parallel", torch.bfloat16)
+    prompt = tokens_for(cfg, 20)[None].to(DEV)
+    seq = generate.generate(model, prompt, 30, temperature=0.8, top_k=5)
+    logits = generate.extend(model, seq[:, :-1], 0).float()[0]
+    for t in range(19, 49):  # every sampled token is among the five most likely (one more for a tie at the cut)
+        assert (logits[t] > logits[t, seq[0, t + 1]]).sum() <= 6
+
+
+def test_trace_replay_writes_the_wanted_rows(tmp_path, monkeypatch, capsys):
+    from easy_to_hard_amd import trace
+
+    cfg = CONFIGS["mixed"]
+    w = hp.refatar_weights(cfg)
+    (tmp_path / "model").mkdir()
+    (tmp_path / "out").mkdir()
+    hp.write_checkpoint_folder(tmp_path / "model", cfg, w)
+    a, b = tokens_for(cfg, 50, seed=70).tolist(), tokens_for(cfg, 7, seed=71).tolist()
+    steps = [{"entries": [{"id": "x", "tokens": a[:33], "want": [0, 32]}], "end": []}, {"entries": [{"id": "x", "tokens": a[33:35], "want": []}], "end": []},
+             {"entries": [{"id": "x", "tokens": a[35:], "want": [14]}], "end": ["x"]}, {"entries": [{"id": "y", "tokens": b, "want": [6, 1]}], "end": ["y"]}]
+    text = "".join(json.dumps({"step": i, **s}) + "\n" for i, s in enumerate(steps))
+    monkeypatch.setattr("sys.stdin", io.StringIO(text))
+    assert trace.main(["--model", str(tmp_path / "model"), "--dtype", "float32", "--out", str(tmp_path / "out"), "--max-tokens", "50"]) == 0
+    assert [line for line in capsys.readouterr().out.splitlines() if line.startswith("done")] == [f"done {i}" for i in range(4)]
+    weights = {n: t.float().numpy() for n, t in w.items()}
+    la, lb = ro.forward(cfg, weights, a)[0], ro.forward(cfg, weights, b)[0]
+    read = lambda i: np.fromfile(tmp_path / "out" / f"{i}.f32", "<f4").reshape(-1, cfg["vocab"])  # noqa: E731
+    assert rms_error(read(0), la[[0, 32]]) < 2e-5 and rms_error(read(2), la[[49]]) < 2e-5 and rms_error(read(3), lb[[6, 1]]) < 2e-5
+    assert not (tmp_path / "out" / "1.f32").exists()
+
+
+# ---- quantized linears and scoring ---------------------------------------------------------------------------------------------------
+
+def test_int8_and_int4_linears_under_this_model(tmp_path):
+    import easy_to_hard_amd as e2h
+
+    cfg = hp.refatar_config([hp.refatar_parallel(heads=4, kv_heads=2, dim=32, vdim=32, r_heads=4, r_dim=32, r_vdim=32, ff=256),
+                             hp.refatar_delta(heads=4, kv_heads=2, dim=32, vdim=32, ff=256)], vocab=128, width=256, side=16)
+    hp.write_checkpoint_folder(tmp_path, cfg, hp.refatar_weights(cfg))
+    toks = tokens_for(cfg, 70)[None].to(DEV)
+    base = generate.load_model(tmp_path, DEV)
+    base.setup_caches(1, 80)
+    want = feed(base, toks, [70])[0].cpu().numpy()
+    int8 = e2h.WeightOnlyInt8QuantHandler(generate.load_model(tmp_path, DEV)).convert_for_runtime_on_the_fly().to(DEV)
+    int8.setup_caches(1, 80)
+    got = feed(int8, toks, [60] + [1] * 10)[0].cpu().numpy()
+    assert np.sqrt(((got - want) ** 2).mean()) / want.std() < 0.1
+    model = generate.load_model(tmp_path, DEV)
+    handler = e2h.WeightOnlyInt4QuantHandler(model, groupsize=32)
+    state = handler.create_quantized_state_dict()
+    model = handler.convert_for_runtime()
+    model.load_state_dict(state, assign=True)
+    model = model.to(DEV)
+    model.setup_caches(1, 80)
+    got = feed(model, toks, [60] + [1] * 10)[0].cpu().numpy()
+    assert np.isfinite(got).all() and np.corrcoef(got.ravel(), want.ravel())[0, 1] > 0.7
+
+
+def test_scoring_with_a_reward_head(tmp_path):
+    cfg = CONFIGS["mixed"]
+    w = hp.refatar_weights(cfg)
+    hp.write_checkpoint_folder(tmp_path, cfg, w)
+    model = generate.load_reward_model(tmp_path, DEV, torch.float32)
+    head = torch.randn((2, cfg["width"]), generator=torch.Generator().manual_seed(0))
+    model.backbone.output.weight.data.copy_(head)
+    toks = tokens_for(cfg, 40)
+    got = generate.model_score(model, toks[None].to(DEV))[0].cpu().numpy()
+    weights = {n: t.float().numpy() for n, t in w.items()}
+    weights["head"] = head.numpy()
+    linear = ro.forward({**cfg, "logit_softcap": 1e12}, weights, toks.numpy())[0]
+    assert rel(got, linear.mean(-1)) < 1e-4

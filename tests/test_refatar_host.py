@@ -1,0 +1,289 @@
+"""CPU checks of the Refatar decoder's surroundings: the oracle's mechanisms against independent formulas, the configuration and
+checkpoint reader, the fused weight layout, the state plan, and the C ABI of libe2h_seq.so (no kernel is launched)."""
+
+import ctypes
+import re
+from pathlib import Path
+
+import numpy as np
+import pytest
+import torch
+
+from easy_to_hard_amd import _lib, generate, registry
+from easy_to_hard_amd.checkpoint import SafetensorsFile
+from easy_to_hard_amd.model import ModelArgs, RewardModel, Transformer
+from easy_to_hard_amd.refatar import Refatar, RefatarArgs
+from easy_to_hard_amd.state import ConvRings, KVCache, SequenceState, StatePlan
+from oracle import refatar_oracle as ro
+from tests import helpers as hp
+
+ROOT = Path(__file__).resolve().parents[1]
+
+
+# ---- the oracle ------------------------------------------------------------------------------------------------------------
+
+def test_oracle_window_visibility_by_hand():
+    seen = [j for j in range(12) if ro.window_visible(10, j, 3, 2)]
+    assert seen == [0, 1, 8, 9, 10]
+    assert [j for j in range(4) if ro.window_visible(0, j, 1, 5)] == [0]
+    assert [j for j in range(12) if ro.window_visible(6, j, 1, 0)] == [6]
+
+
+def test_oracle_attention_equals_masked_softmax():
+    rng = np.random.default_rng(0)
+    t, h, g, d, dv, size, keep = 17, 6, 2, 5, 7, 4, 3
+    q, k, v = rng.normal(size=(t, h, d)), rng.normal(size=(t, g, d)), rng.normal(size=(t, g, dv))
+    out = ro.window_attention(q, k, v, 0.4, size, keep)
+    i, j = np.arange(t)[:, None], np.arange(t)[None, :]
+    mask = (j <= i) & ((i - j < size) | (j < keep))
+    for a in range(h):
+        s = np.where(mask, 0.4 * q[:, a] @ k[:, a // 3].T, -np.inf)
+        p = np.exp(s - s.max(1, keepdims=True))
+        np.testing.assert_allclose(out[:, a], (p / p.sum(1, keepdims=True)) @ v[:, a // 3], atol=1e-12)
+
+
+def test_oracle_convolution_equals_numpy_convolve():
+    rng = np.random.default_rng(1)
+    x, w = rng.normal(size=(20, 3)), rng.normal(size=(3, 4))
+    y = ro.causal_conv(x, w)
+    for c in range(3):
+        np.testing.assert_allclose(y[:, c], np.convolve(x[:, c], w[c, ::-1])[:20], atol=1e-12)
+
+
+def test_oracle_hgrn2_equals_the_sum_over_earlier_tokens():
+    rng = np.random.default_rng(2)
+    t, h, d, dv = 9, 2, 4, 3
+    q, f, v = rng.normal(size=(t, h, d)), rng.uniform(0.1, 1, size=(t, h, d)), rng.normal(size=(t, h, dv))
+    o, _ = ro.hgrn2_recurrence(q, f, v)
+    for i in range(t):
+        want = sum(((q[i] * (1 - f[s]) * np.prod(f[s + 1: i + 1], axis=0)).sum(-1, keepdims=True)) * v[s] for s in range(i + 1))
+        np.testing.assert_allclose(o[i], want, atol=1e-12)
+
+
+def test_oracle_delta_rule_overwrites_a_key():
+    """beta 1 and decay 1: reading a unit key right after it was written returns exactly its value, whatever was there."""
+    rng = np.random.default_rng(3)
+    t, h, d, dv = 6, 1, 5, 4
+    k = np.repeat(ro.unit(rng.normal(size=(1, h, d))), t, axis=0) * np.sqrt(1 + 1e-6)
+    k /= np.linalg.norm(k, axis=-1, keepdims=True)
+    v = rng.normal(size=(t, h, dv))
+    o, _ = ro.delta_recurrence(k, k, v, np.ones((t, h)), np.ones((t, h)))
+    np.testing.assert_allclose(o, v, atol=1e-12)
+
+
+def test_oracle_delta_rule_equals_the_matrix_form():
+    rng = np.random.default_rng(4)
+    t, d, dv = 7, 4, 3
+    q, k, v = rng.normal(size=(t, 1, d)), ro.unit(rng.normal(size=(t, 1, d))), rng.normal(size=(t, 1, dv))
+    g, b = rng.uniform(0.5, 1, size=(t, 1)), rng.uniform(0, 1, size=(t, 1))
+    o, _ = ro.delta_recurrence(q, k, v, g, b)
+    s = np.zeros((d, dv))
+    for i in range(t):  # S = (I - beta k k^T) g S + beta k v^T
+        kk = k[i, 0][:, None]
+        s = (np.eye(d) - b[i, 0] * kk @ kk.T) @ (g[i, 0] * s) + b[i, 0] * kk @ v[i]
+        np.testing.assert_allclose(o[i, 0], s.T @ q[i, 0], atol=1e-12)
+
+
+def test_oracle_scalar_functions():
+    z = np.array([-30.0, -2.0, 0.0, 0.7, 40.0])
+    t = torch.from_numpy(z)
+    np.testing.assert_allclose(ro.sigmoid(z), torch.sigmoid(t).numpy(), rtol=1e-12)
+    np.testing.assert_allclose(ro.silu(z), torch.nn.functional.silu(t).numpy(), rtol=1e-12)
+    np.testing.assert_allclose(ro.softplus(z), np.logaddexp(0, z), rtol=1e-12)
+    np.testing.assert_allclose(ro.gelu_tanh(z), torch.nn.functional.gelu(t, approximate="tanh").numpy(), atol=1e-12)
+
+
+# ---- configuration, checkpoint, weight layout -----------------------------------------------------------------------------------
+
+def test_registry_and_configuration():
+    cfg = hp.refatar_config([hp.refatar_parallel(), hp.refatar_delta(ff=None)])
+    assert registry.model_class(cfg) is Refatar
+    args = RefatarArgs.from_config(cfg)
+    assert (args.vocab_size, args.dim, args.canon_taps, args.side_dim, args.logit_softcap) == (97, 104, 4, 12, 11.0)
+    with pytest.raises(ValueError, match="unknown architecture"):
+        registry.model_class({"architecture": "Nothing"})
+    bad = hp.refatar_config([dict(hp.refatar_delta(), type="other")])
+    with pytest.raises(ValueError, match="unknown mixer"):
+        RefatarArgs.from_config(bad)
+    model = registry.model_from_config(cfg)
+    assert model.layers[1].feed_forward is None and not hasattr(model.layers[1], "norm2")
+    assert model.returns_greedy_token and Transformer.returns_greedy_token
+
+
+def test_safetensors_reader_round_trip(tmp_path):
+    tensors = {"a": hp.randn_bf16((3, 5)), "b": torch.arange(7, dtype=torch.int32), "c": torch.randn(2, 2, 2)}
+    hp.write_safetensors(tmp_path / "x.safetensors", tensors)
+    f = SafetensorsFile(tmp_path / "x.safetensors")
+    assert set(f.keys()) == set(tensors)
+    for n, t in tensors.items():
+        assert f.get(n).dtype == t.dtype and torch.equal(f.get(n), t)
+    with pytest.raises(KeyError):
+        f.get("missing")
+    st = pytest.importorskip("safetensors.torch")
+    st.save_file(tensors, str(tmp_path / "y.safetensors"))
+    g = SafetensorsFile(tmp_path / "y.safetensors")
+    assert all(torch.equal(g.get(n), t) for n, t in tensors.items())
+
+
+def test_fused_projections_hold_the_checkpoint_rows_and_zeros_between():
+    cfg = hp.refatar_config([hp.refatar_parallel(heads=3, kv_heads=1, dim=20, vdim=12), hp.refatar_delta(heads=3, kv_heads=3)])
+    w = hp.refatar_weights(cfg)
+    model = Refatar.from_config(cfg)
+    sd = model.state_dict_from_checkpoint(w.__getitem__)
+    assert {k: tuple(v.shape) for k, v in sd.items()} == {k: tuple(v.shape) for k, v in model.state_dict().items()}
+    for i, layer in enumerate(model.layers):
+        rows = sd[f"layers.{i}.mixer.in_proj.weight"].clone()
+        for b, name in zip(layer.mixer.branches, layer.mixer.names):
+            for (proj, n), col in zip(b.projections, b.columns):
+                assert col % 8 == 0
+                assert torch.equal(rows[col: col + n], w[f"l{i}.mix.{name + '.' if name else ''}{proj}"])
+                rows[col: col + n] = 0
+        assert not rows.any()
+    assert torch.equal(sd["layers.0.mixer.out_proj.weight"], torch.cat([w["l0.mix.left.o"], w["l0.mix.right.o"]], dim=1))
+    assert sd["layers.0.canon1"].shape == (4, 104) and torch.equal(sd["layers.0.canon1"], w["l0.canon1"].float().t())
+    assert sd["layers.1.mixer.branches.0.conv"].shape == (2 * 3 * 24 + 3 * 20, 4)
+    assert all(v.dtype == torch.float32 for k, v in sd.items() if not k.endswith("weight"))
+
+
+def test_loader_names_the_tensor_whose_shape_does_not_fit(tmp_path):
+    cfg = hp.refatar_config([hp.refatar_delta()])
+    w = hp.refatar_weights(cfg)
+    w["l0.mlp.up"] = w["l0.mlp.up"][:-8]
+    hp.write_checkpoint_folder(tmp_path, cfg, w)
+    with pytest.raises(ValueError, match="feed_forward.up.weight"):
+        generate.load_model(tmp_path, "cpu")
+    w["l0.mix.k"] = w["l0.mix.k"][:-1]
+    hp.write_checkpoint_folder(tmp_path, cfg, w)
+    with pytest.raises(ValueError, match="l0.mix.k"):
+        generate.load_model(tmp_path, "cpu")
+
+
+def test_linears_and_vectors_load_in_their_own_precision(tmp_path):
+    cfg = hp.refatar_config([hp.refatar_parallel()])
+    hp.write_checkpoint_folder(tmp_path, cfg, hp.refatar_weights(cfg))
+    for precision in (torch.bfloat16, torch.float32):
+        model = generate.load_model(tmp_path, "cpu", precision)
+        assert model.layers[0].mixer.in_proj.weight.dtype == precision and model.dtype == precision
+        assert model.layers[0].norm1.dtype == torch.float32 and model.norm.dtype == torch.float32
+
+
+def test_reward_model_takes_either_family():
+    llama = RewardModel(ModelArgs.from_name("tiny-test"))
+    assert isinstance(llama.backbone, Transformer)
+    reward = RewardModel(RefatarArgs.from_config(hp.refatar_config([hp.refatar_delta()])))
+    assert isinstance(reward.backbone, Refatar) and reward.backbone.output.out_features == 2 and reward.backbone.logit_softcap is None
+
+
+# ---- state -----------------------------------------------------------------------------------------------------------------------
+
+def test_state_plan_allocates_what_the_layers_asked_for():
+    cfg = hp.refatar_config([hp.refatar_parallel(), hp.refatar_delta(), hp.refatar_parallel(ff=None)])
+    model = Refatar.from_config(cfg)
+    st = SequenceState(model.plan, 3, 40, torch.bfloat16, "cpu")
+    assert len(st.kv) == 2 and tuple(st.kv[0].k_cache.shape) == (3, 2, 40, 24) and tuple(st.kv[0].v_cache.shape) == (3, 2, 40, 40)
+    assert [tuple(r.s.shape) for r in st.recurrent] == [(3, 3, 20, 36), (3, 4, 24, 20), (3, 3, 20, 36)]
+    assert all(r.s.dtype == torch.float32 for r in st.recurrent)
+    assert len(st.rings_f32.shapes) == 5 and len(st.rings.shapes) == 1 and st.rings.live.dtype == torch.bfloat16
+    assert isinstance(st.kv[0], KVCache)
+
+
+def test_conv_rings_commit_only_the_rows_of_the_call():
+    rings = ConvRings(3, [(4, 3), (8, 2)], torch.float32)
+    live, nxt = rings.site(0, 5)
+    assert live.data_ptr() != nxt.data_ptr() and rings.site(0, 1)[1].data_ptr() == live.data_ptr()
+    nxt.fill_(1.0)
+    rings.site(1, 5)[1].fill_(2.0)
+    rings.commit(2, 5)
+    assert live[:2].eq(1).all() and live[2].eq(0).all() and rings.site(1, 5)[0][:2].eq(2).all()
+    rings.commit(3, 5)
+    assert live.eq(1).all()
+
+
+def test_state_plan_shares_nothing_between_sites():
+    plan = StatePlan()
+    a, b = plan.add_ring(4, 3, True), plan.add_ring(5, 3, True)
+    st = SequenceState(plan, 2, 8, torch.float32, "cpu")
+    st.rings_f32.site(a, 1)[0].fill_(7)
+    assert st.rings_f32.site(b, 1)[0].eq(0).all()
+
+
+# ---- C ABI -----------------------------------------------------------------------------------------------------------------------
+
+def _header():
+    text = (ROOT / "include" / "e2h_seq.h").read_text()
+    return re.sub(r"/\*.*?\*/", "", text, flags=re.S)
+
+
+def test_seq_library_exports_every_declared_symbol():
+    lib = _lib.load_seq()
+    declared = sorted(set(re.findall(r"\b(e2h_seq_[a-z0-9_]+)\s*\(", _header())))
+    assert declared == sorted(_lib.SEQ_EXPORTED_SYMBOLS)
+    assert all(hasattr(lib, n) for n in declared) and lib.e2h_seq_abi_version() == 1
+
+
+@pytest.mark.parametrize("c_name,py", [("e2h_norm_conv_args", _lib.NormConvArgs), ("e2h_window_attention_args", _lib.WindowAttentionArgs),
+                                       ("e2h_hgrn2_args", _lib.Hgrn2Args), ("e2h_delta_args", _lib.DeltaArgs)])
+def test_argument_structs_mirror_the_header(c_name, py):
+    body = re.search(r"typedef struct \{([^}]*)\} " + c_name + ";", _header()).group(1)
+    fields = []
+    for decl in body.split(";"):
+        decl = decl.strip()
+        if not decl:
+            continue
+        base = re.match(r"(const\s+)?(\w+)", decl).group(2)
+        for item in decl[re.match(r"(const\s+)?\w+", decl).end():].split(","):
+            item = item.strip()
+            kind = ctypes.c_void_p if "*" in item else {"int32_t": ctypes.c_int32, "int64_t": ctypes.c_int64, "float": ctypes.c_float}[base]
+            fields.append((item.replace("*", "").strip(), kind))
+    assert fields == py._fields_
+
+
+def test_argument_validation_returns_codes_without_launching():
+    lib = _lib.load_seq()
+    p = 4096  # never dereferenced: validation fails first
+    assert lib.e2h_seq_set_option(b"no_such_option", 1) == -8
+    assert lib.e2h_seq_set_option(b"recurrence_form", 3) == -8
+    assert lib.e2h_seq_square_relu(0, None, p, 8, None) == -1
+    assert lib.e2h_seq_square_relu(5, p, p, 8, None) == -2
+    assert lib.e2h_seq_softcap(0, p, p, 8, 0.0, None) == -2
+    assert lib.e2h_seq_softcap(0, p + 2, p, 8, 1.0, None) == -5
+    assert lib.e2h_seq_gelu_gate_rows(0, p, p, p, p, 2, 8, 8, 1, 4, None) == -2   # column range past the table's rows
+
+    n = _lib.NormConvArgs(dtype=0, batch=1, seqlen=2, width=8, eps=1e-6, x=p, norm_weight=p, out=p)
+    n.width = 6
+    assert lib.e2h_seq_norm_conv(ctypes.byref(n), None) == -2
+    n.width, n.taps, n.conv, n.input_pos, n.tail_in, n.tail_out = 8, 3, p, p, p, p
+    assert lib.e2h_seq_norm_conv(ctypes.byref(n), None) == -2                      # several tokens need a second ring
+    n.tail_out = p + 4096
+    n.taps = 9
+    assert lib.e2h_seq_norm_conv(ctypes.byref(n), None) == -2
+    n.x = None
+    assert lib.e2h_seq_norm_conv(ctypes.byref(n), None) == -1
+
+    a = _lib.WindowAttentionArgs(dtype=0, batch=1, seqlen=1, heads=4, kv_heads=3, dim=8, vdim=8, cache_len=16, proj=p, ld=96, q_off=0, k_off=32,
+                                 v_off=56, g_off=-1, k_cache=p, v_cache=p, input_pos=p, scale=1.0, out_scale=1.0, out=p, ld_out=32)
+    assert lib.e2h_seq_window_attention(ctypes.byref(a), None) == -2               # heads not a multiple of kv_heads
+    a.kv_heads, a.dim = 2, 300
+    assert lib.e2h_seq_window_attention(ctypes.byref(a), None) == -2
+    a.dim, a.ld_out = 8, 31
+    assert lib.e2h_seq_window_attention(ctypes.byref(a), None) == -2               # output does not fit its rows
+
+    r = _lib.Hgrn2Args(dtype=0, eps=1e-6, batch=1, seqlen=1, heads=2, dim=8, vdim=6, proj=p, ld=64, q_off=0, f_off=16, v_off=32, f_bias=p, lower=p,
+                       norm_weight=p, state=p, input_pos=p, out=p, ld_out=12)
+    assert lib.e2h_seq_hgrn2(ctypes.byref(r), None) == -2                          # vdim % 4
+    r.vdim, r.seqlen, r.ld_out = 8, 4096, 16
+    need = lib.e2h_seq_hgrn2_scratch_bytes(ctypes.byref(r))
+    assert need > 0
+    assert lib.e2h_seq_hgrn2(ctypes.byref(r), None) == -1                          # no scratch
+    r.scratch, r.scratch_bytes = p, need - 1
+    assert lib.e2h_seq_hgrn2(ctypes.byref(r), None) == -9
+
+    d = _lib.DeltaArgs(dtype=0, taps=4, batch=1, seqlen=3, heads=2, kv_heads=2, dim=8, vdim=8, proj=p, ld=96, q_off=0, k_off=16, v_off=32, b_off=48,
+                       a_off=56, g_off=64, conv=p, tail_in=p, tail_out=p, a_log=p, dt_bias=p, norm_weight=p, state=p, input_pos=p, out=p, ld_out=16)
+    assert lib.e2h_seq_delta(ctypes.byref(d), None) == -2                          # the same ring for several tokens
+    d.tail_out = p + 4096
+    assert lib.e2h_seq_delta(ctypes.byref(d), None) == -1                          # no scratch
+    d.g_off = 90
+    assert lib.e2h_seq_delta(ctypes.byref(d), None) == -2
+    with pytest.raises(RuntimeError, match="unsupported shape"):
+        _lib.check_seq(-2, "x")
