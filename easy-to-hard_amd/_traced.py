@@ -9,13 +9,14 @@ eager execution they call the wrapper directly, which spares the hot loop the di
 RoPE launches write are declared as mutated arguments.
 """
 
-from typing import NamedTuple, Optional, Tuple
+from typing import List, NamedTuple, Optional, Tuple
 
 import torch
 from torch import Tensor
 
 from . import _lib
 from . import ops as _ops
+from . import seq_ops as _seq
 
 _registered = {}
 
@@ -426,6 +427,120 @@ def int4_staged_partial_slices(rows, lin):
     return s if s > 0 else 0
 
 
+# ---- layers with per-sequence state (seq_ops.py) -----------------------------------------------------------------------------
+#
+# The caches, states, convolution rings and output buffers these kernels write are mutated arguments; a single-token step hands
+# the same ring in for reading and for writing, and the kernel never reads the slot it writes.
+
+_norm_conv_eager = _seq.norm_conv
+_window_attention_eager, _hgrn2_eager, _gated_delta_eager = _seq.window_attention, _seq.hgrn2, _seq.gated_delta
+_square_relu_eager, _softcap_eager, _gelu_gate_eager = _seq.square_relu_, _seq.softcap_, _seq.gelu_gate_rows
+
+
+def _seq_norm_conv(x: Tensor, batch: int, seqlen: int, eps: float, dtype: torch.dtype, delta: Optional[Tensor], delta_weight: Optional[Tensor],
+                   delta_offset: float, norm_weight: Optional[Tensor], norm_offset: float, conv: Optional[Tensor], tail_in: Optional[Tensor],
+                   tail_out: Optional[Tensor], input_pos: Optional[Tensor], first: Optional[Tensor], want_x: bool, want_out: bool) -> Tuple[Tensor, Tensor]:
+    x_out, out = _norm_conv_eager(x, batch, seqlen, eps, dtype, delta, delta_weight, delta_offset, norm_weight, norm_offset, conv,
+                                  None if tail_in is None else (tail_in, tail_out), input_pos, first, want_x, want_out)
+    return (x_out if delta is not None and want_x else x.new_empty((0,))), (out if want_out else x.new_empty((0,), dtype=dtype))
+
+
+def _seq_square_relu(x: Tensor) -> None:
+    _square_relu_eager(x)
+
+
+def _seq_softcap(x: Tensor, cap: float) -> None:
+    _softcap_eager(x, cap)
+
+
+def _seq_gelu_gate(gate: Tensor, table: Tensor, tokens: Tensor, column: int) -> Tensor:
+    return _gelu_gate_eager(gate, table, tokens, column)
+
+
+class _CachePair(NamedTuple):
+    k_cache: Tensor
+    v_cache: Tensor
+
+
+def _seq_window_attention(proj: Tensor, batch: int, seqlen: int, heads: int, kv_heads: int, dim: int, vdim: int, offsets: List[int],
+                          q_bias: Optional[Tensor], k_bias: Optional[Tensor], v_bias: Optional[Tensor], k_cache: Tensor, v_cache: Tensor,
+                          input_pos: Tensor, first: Optional[Tensor], window: int, keep_first: int, scale: float, out: Tensor, out_off: int,
+                          out_scale: float) -> None:
+    _window_attention_eager(proj, batch, seqlen, heads, kv_heads, dim, vdim, offsets, (q_bias, k_bias, v_bias), _CachePair(k_cache, v_cache), input_pos,
+                            first, window, keep_first, scale, out, out_off, out_scale)
+
+
+def _seq_hgrn2(proj: Tensor, batch: int, seqlen: int, heads: int, dim: int, vdim: int, offsets: List[int], f_bias: Tensor, lower: Tensor,
+               norm_weight: Tensor, eps: float, state: Tensor, input_pos: Tensor, first: Optional[Tensor], out: Tensor, out_off: int,
+               out_scale: float) -> None:
+    _hgrn2_eager(proj, batch, seqlen, heads, dim, vdim, offsets, f_bias, lower, norm_weight, eps, state, input_pos, first, out, out_off, out_scale)
+
+
+def _seq_gated_delta(proj: Tensor, batch: int, seqlen: int, heads: int, kv_heads: int, dim: int, vdim: int, offsets: List[int], conv: Tensor,
+                     tail_in: Tensor, tail_out: Tensor, a_log: Tensor, dt_bias: Tensor, norm_weight: Tensor, eps: float, state: Tensor,
+                     input_pos: Tensor, first: Optional[Tensor], out: Tensor, out_off: int, out_scale: float) -> None:
+    _gated_delta_eager(proj, batch, seqlen, heads, kv_heads, dim, vdim, offsets, conv, (tail_in, tail_out), a_log, dt_bias, norm_weight, eps, state,
+                       input_pos, first, out, out_off, out_scale)
+
+
+def _nothing(*args):
+    return None
+
+
+_norm_conv_op = _register(
+    "seq_norm_conv", _seq_norm_conv,
+    lambda x, batch, seqlen, eps, dtype, delta, dw, do, nw, no, conv, ti, to, pos, first, want_x, want_out: (
+        torch.empty_like(x) if delta is not None and want_x else x.new_empty((0,)),
+        x.new_empty(x.shape, dtype=dtype) if want_out else x.new_empty((0,), dtype=dtype)),
+    mutates=("tail_out",))
+_square_relu_op = _register("seq_square_relu", _seq_square_relu, _nothing, mutates=("x",))
+_softcap_op = _register("seq_softcap", _seq_softcap, _nothing, mutates=("x",))
+_gelu_gate_op = _register("seq_gelu_gate_rows", _seq_gelu_gate, lambda gate, table, tokens, column: torch.empty_like(gate))
+_window_attention_op = _register("seq_window_attention", _seq_window_attention, _nothing, mutates=("k_cache", "v_cache", "out"))
+_hgrn2_op = _register("seq_hgrn2", _seq_hgrn2, _nothing, mutates=("state", "out"))
+_gated_delta_op = _register("seq_gated_delta", _seq_gated_delta, _nothing, mutates=("tail_out", "state", "out"))
+
+
+def norm_conv(x, batch, seqlen, eps, dtype, delta=None, delta_weight=None, delta_offset=0.0, norm_weight=None, norm_offset=0.0, conv=None, tails=None,
+              input_pos=None, first=None, want_x=True, want_out=True):
+    ti, to = tails if tails is not None else (None, None)
+    x_out, out = _norm_conv_op(x, batch, seqlen, eps, dtype, delta, delta_weight, delta_offset, norm_weight, norm_offset, conv, ti, to, input_pos, first,
+                               want_x, want_out)
+    return (x_out if delta is not None and want_x else x), (out if want_out else None)
+
+
+def square_relu_(x):
+    _square_relu_op(x)
+    return x
+
+
+def softcap_(x, cap):
+    _softcap_op(x, cap)
+    return x
+
+
+def gelu_gate_rows(gate, table, tokens, column):
+    return _gelu_gate_op(gate, table, tokens, column)
+
+
+def window_attention(proj, batch, seqlen, heads, kv_heads, dim, vdim, offsets, biases, cache, input_pos, first, window, keep_first, scale, out, out_off,
+                     out_scale=1.0):
+    _window_attention_op(proj, batch, seqlen, heads, kv_heads, dim, vdim, list(offsets), *biases, cache.k_cache, cache.v_cache, input_pos, first, window,
+                         keep_first, scale, out, out_off, out_scale)
+
+
+def hgrn2(proj, batch, seqlen, heads, dim, vdim, offsets, f_bias, lower, norm_weight, eps, state, input_pos, first, out, out_off, out_scale=1.0):
+    _hgrn2_op(proj, batch, seqlen, heads, dim, vdim, list(offsets), f_bias, lower, norm_weight, eps, state, input_pos, first, out, out_off, out_scale)
+
+
+def gated_delta(proj, batch, seqlen, heads, kv_heads, dim, vdim, offsets, conv, tails, a_log, dt_bias, norm_weight, eps, state, input_pos, first, out,
+                out_off, out_scale=1.0):
+    _gated_delta_op(proj, batch, seqlen, heads, kv_heads, dim, vdim, list(offsets), conv, *tails, a_log, dt_bias, norm_weight, eps, state, input_pos,
+                    first, out, out_off, out_scale)
+
+
+_SEQ_REBOUND = ("norm_conv", "square_relu_", "softcap_", "gelu_gate_rows", "window_attention", "hgrn2", "gated_delta")
+
 _REBOUND = (
     "rmsnorm", "add_rmsnorm", "silu_mul", "rope_kv_write", "rope_kv_write_seq", "decode_attention", "argmax_rows", "int4_mm_silu_gate",
     "int4_mm_rope_kv", "int4_mm_partials", "int8_mm_silu_gate", "int8_mm_rope_kv", "int8_mm_partials", "ScaledPartials",
@@ -436,6 +551,8 @@ _REBOUND = (
 
 
 def install():
-    """Rebind the public names of ops.py to the dispatchers above (done once, when the package is imported)."""
+    """Rebind the public names of ops.py and seq_ops.py to the dispatchers above (done once, when the package is imported)."""
     for name in _REBOUND:
         setattr(_ops, name, globals()[name])
+    for name in _SEQ_REBOUND:
+        setattr(_seq, name, globals()[name])

@@ -270,3 +270,47 @@ def model_score(reward_model, prompt: Tensor, max_seq_len: Optional[int] = None)
     bsz, t = prompt.shape
     reward_model.backbone.setup_caches(max_batch_size=bsz, max_seq_length=max_seq_len or t, kv_cache=False)
     return reward_model(prompt)
+
+
+def main(argv=None) -> int:
+    """Generate from token ids: python -m easy_to_hard_amd.generate --checkpoint_path DIR_OR_FILE --tokens 1,2,3 [--tokens 4,5]
+    (the reference's inference_generate.py without its tokenizer and data set; prompts of unequal length are padded on the left)."""
+    import argparse
+    import sys
+
+    ap = argparse.ArgumentParser(prog="generate", description="Generate token ids from token ids.")
+    ap.add_argument("--checkpoint_path", required=True, help="a folder with config.json and model.safetensors, or a .pth file of the Llama family")
+    ap.add_argument("--model_name", default=None, help="Llama family: architecture name when the file's folder does not give it")
+    ap.add_argument("--tokens", action="append", required=True, metavar="ID,ID,...", help="one prompt; repeat for a batch")
+    ap.add_argument("--max_new_tokens", type=int, default=32)
+    ap.add_argument("--temperature", type=float, default=None, help="sample at this temperature (default: greedy)")
+    ap.add_argument("--top_k", type=int, default=None)
+    ap.add_argument("--on_the_fly_8bit_quantization", action="store_true", help="quantize every linear to int8 per channel after loading")
+    args = ap.parse_args(argv)
+    if not torch.cuda.is_available():
+        print("generate: no GPU", file=sys.stderr)
+        return 2
+    device = "cuda:0"
+    prompts = [[int(v) for v in text.split(",") if v.strip()] for text in args.tokens]
+    if any(not p for p in prompts):
+        ap.error("--tokens: an empty prompt")
+    model = load_model(args.checkpoint_path, device, torch.bfloat16, model_name=args.model_name)
+    if args.on_the_fly_8bit_quantization:
+        from .quantize import WeightOnlyInt8QuantHandler
+
+        model = WeightOnlyInt8QuantHandler(model).convert_for_runtime_on_the_fly().to(device=device).eval()
+    longest = max(map(len, prompts))
+    rows = torch.zeros((len(prompts), longest), dtype=torch.int64, device=device)
+    for i, p in enumerate(prompts):
+        rows[i, longest - len(p):] = torch.tensor(p, device=device)
+    pad = None if all(len(p) == longest for p in prompts) else torch.tensor([longest - len(p) for p in prompts], device=device)
+    seq = generate(model, rows, args.max_new_tokens, left_pad_mask_pos=pad, temperature=args.temperature, top_k=args.top_k)
+    for row in seq[:, longest:].tolist():
+        print(",".join(map(str, row)))
+    return 0
+
+
+if __name__ == "__main__":
+    import sys
+
+    sys.exit(main())

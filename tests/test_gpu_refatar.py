@@ -543,6 +543,26 @@ def test_graph_replays_equal_eager_steps_between_other_work(tmp_path):
     assert torch.equal(a, b)
 
 
+def test_decode_step_under_fullgraph_compile_equals_the_graphed_step(tmp_path):
+    model, cfg, _ = load(tmp_path, "mixed", torch.bfloat16)
+    model.setup_caches(2, 96)
+    rows = torch.stack([tokens_for(cfg, 50, seed=90 + i) for i in range(2)]).to(DEV)
+    stepper = generate.GraphedDecodeStep(model, 2, DEV)
+    torch._dynamo.reset()
+    compiled = torch.compile(model, backend="aot_eager", fullgraph=True)
+
+    def decode(step):
+        generate.extend(model, rows[:, :40], 0)
+        return torch.cat([step(rows[:, t: t + 1], torch.tensor([t], device=DEV)) for t in range(40, 50)], dim=1)
+
+    with torch.no_grad():
+        graphed = decode(lambda tok, pos: stepper.step(tok, pos).clone())
+        traced = decode(lambda tok, pos: torch.argmax(compiled(tok, pos)[:, -1].float(), -1, keepdim=True))
+        assert torch.equal(graphed, traced)
+        prompt = compiled(rows[:, :40], torch.arange(40, device=DEV))
+        assert torch.equal(prompt, generate.extend(model, rows[:, :40], 0))
+
+
 def test_left_padded_generation_equals_each_sequence_alone(tmp_path):
     model, cfg, _ = load(tmp_path, "delta-first", torch.float32)
     a, b = tokens_for(cfg, 30, seed=60), tokens_for(cfg, 12, seed=61)
@@ -560,6 +580,18 @@ def test_sampling_through_the_generation_path(tmp_path):
     logits = generate.extend(model, seq[:, :-1], 0).float()[0]
     for t in range(19, 49):  # every sampled token is among the five most likely (one more for a tie at the cut)
         assert (logits[t] > logits[t, seq[0, t + 1]]).sum() <= 6
+
+
+def test_generate_command_line(tmp_path, capsys):
+    model, cfg, _ = load(tmp_path, "mixed", torch.bfloat16)
+    a, b = tokens_for(cfg, 9, seed=80), tokens_for(cfg, 5, seed=81)
+    text = lambda t: ",".join(map(str, t.tolist()))  # noqa: E731
+    assert generate.main(["--checkpoint_path", str(tmp_path), "--tokens", text(a), "--tokens", text(b), "--max_new_tokens", "12"]) == 0
+    lines = [[int(v) for v in line.split(",")] for line in capsys.readouterr().out.split()]
+    rows = torch.zeros((2, 9), dtype=torch.int64)
+    rows[0], rows[1, 4:] = a, b
+    want = generate.generate(model, rows.to(DEV), 12, left_pad_mask_pos=torch.tensor([0, 4], device=DEV))[:, 9:]
+    assert lines == want.tolist()
 
 
 def test_trace_replay_writes_the_wanted_rows(tmp_path, monkeypatch, capsys):
