@@ -47,6 +47,10 @@ __device__ __forceinline__ void store4(bf16_t *p, f32x4_t v) {
   *reinterpret_cast<u32x2_t *>(p) = u32x2_t{pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3])};
 }
 
+// state that one launch reads or writes exactly once: streamed past the caches
+__device__ __forceinline__ f32x4_t load4_stream(const float *p) { return __builtin_nontemporal_load(reinterpret_cast<const f32x4_t *>(p)); }
+__device__ __forceinline__ void store4_stream(float *p, f32x4_t v) { __builtin_nontemporal_store(v, reinterpret_cast<f32x4_t *>(p)); }
+
 __device__ __forceinline__ float wave_add(float v) {
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) v += __shfl_xor(v, off);

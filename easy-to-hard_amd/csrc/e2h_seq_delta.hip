@@ -232,7 +232,7 @@ __global__ __launch_bounds__(BLOCK) void delta_tokens_kernel(const e2h_delta_arg
   for (int i = 0; i < RPT; ++i) {
     const int r = rg + RG * i;
     s[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    if (pos0 > 0 && col_ok && r < D) s[i] = load4(st + static_cast<size_t>(r) * DV + cg * 4);
+    if (pos0 > 0 && col_ok && r < D) s[i] = load4_stream(st + static_cast<size_t>(r) * DV + cg * 4);
   }
   const T *proj = static_cast<const T *>(a.proj);
   for (int t = 0; t < seqlen; ++t) {
@@ -242,24 +242,43 @@ __global__ __launch_bounds__(BLOCK) void delta_tokens_kernel(const e2h_delta_arg
       const int channels = 2 * kvh * D + H * DV;
       float qs = 0.f, ks = 0.f;
       const bool owner = h % (H / kvh) == 0;  // of the shared query/key head's ring slot; nobody reads that slot in this call
-      T *slot = static_cast<T *>(a.tail_out) + (static_cast<size_t>(b) * a.taps + (pos0 > 0 ? pos0 % a.taps : 0)) * channels;
-      for (int i = threadIdx.x; i < D; i += BLOCK) {
-        const int qc = hk * D + i, kc = (kvh + hk) * D + i;
-        const float q = conv_silu<T>(a, row, b, 0, pos0, first, a.q_off + qc, qc, channels);
-        const float k = conv_silu<T>(a, row, b, 0, pos0, first, a.k_off + hk * D + i, kc, channels);
-        sh_q[i] = q;
-        sh_k[i] = k;
-        qs = __builtin_fmaf(q, q, qs);
-        ks = __builtin_fmaf(k, k, ks);
-        if (owner && a.taps > 1) {
-          slot[qc] = proj[row * a.ld + a.q_off + qc];
-          slot[kc] = proj[row * a.ld + a.k_off + hk * D + i];
-        }
+      const uint32_t taps = static_cast<uint32_t>(a.taps), at = static_cast<uint32_t>(pos0 > 0 ? pos0 : 0);
+      T *slot = static_cast<T *>(a.tail_out) + (static_cast<size_t>(b) * a.taps + at % taps) * channels;
+      size_t kept[3];  // ring rows of the three tokens before this one
+      bool there[3];
+#pragma unroll
+      for (int j = 0; j < 3; ++j) {
+        const int64_t pos = pos0 - 3 + j;
+        there[j] = taps > 3u - j && pos >= first && pos >= 0;
+        kept[j] = (static_cast<size_t>(b) * a.taps + (there[j] ? static_cast<uint32_t>(pos) % taps : 0u)) * channels;
       }
-      for (int i = threadIdx.x; i < DV; i += BLOCK) {
-        const int vc = h * DV + i, ch = 2 * kvh * D + vc;
-        sh_v[i] = conv_silu<T>(a, row, b, 0, pos0, first, a.v_off + vc, ch, channels);
-        if (a.taps > 1) slot[ch] = proj[row * a.ld + a.v_off + vc];
+      for (int i = threadIdx.x; i < 2 * D + DV; i += BLOCK) {  // channels of q, k, v
+        const bool is_q = i < D, is_k = !is_q && i < 2 * D;
+        const int d = is_q ? i : is_k ? i - D : i - 2 * D;
+        const int ch = is_q ? hk * D + d : is_k ? (kvh + hk) * D + d : 2 * kvh * D + h * DV + d;
+        const int64_t c0 = is_q ? a.q_off + hk * D + d : is_k ? a.k_off + hk * D + d : a.v_off + static_cast<int64_t>(h) * DV + d;
+        float y;
+        if (taps <= 4) {  // everything in flight at once
+          const T now = proj[row * a.ld + c0];
+          const T *tail = static_cast<const T *>(a.tail_in);
+          T x[3];
+          float w[4];
+#pragma unroll
+          for (int j = 0; j < 3; ++j) x[j] = *(there[j] ? tail + kept[j] + ch : proj + row * a.ld + c0);
+#pragma unroll
+          for (int j = 0; j < 4; ++j) w[j] = a.conv[static_cast<size_t>(ch) * taps + (j + taps >= 4u ? j + taps - 4u : 0u)];
+          y = w[3] * to_f32(now);
+#pragma unroll
+          for (int j = 0; j < 3; ++j) y = __builtin_fmaf(w[j], there[j] ? to_f32(x[j]) : 0.f, y);
+          y = silu_f32(y);
+          if (taps > 1 && (owner || !(is_q || is_k))) slot[ch] = now;
+        } else {
+          y = conv_silu<T>(a, row, b, 0, pos0, first, c0, ch, channels);
+          if (owner || !(is_q || is_k)) slot[ch] = proj[row * a.ld + c0];
+        }
+        if (is_q) qs = __builtin_fmaf(y, y, qs);
+        if (is_k) ks = __builtin_fmaf(y, y, ks);
+        (is_q ? sh_q : is_k ? sh_k : sh_v)[d] = y;
       }
       qs = wave_add(qs);
       ks = wave_add(ks);
@@ -348,7 +367,7 @@ __global__ __launch_bounds__(BLOCK) void delta_tokens_kernel(const e2h_delta_arg
 #pragma unroll
   for (int i = 0; i < RPT; ++i) {
     const int r = rg + RG * i;
-    if (col_ok && r < D) store4(st + static_cast<size_t>(r) * DV + cg * 4, s[i]);
+    if (col_ok && r < D) store4_stream(st + static_cast<size_t>(r) * DV + cg * 4, s[i]);
   }
 }
 
@@ -461,25 +480,25 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(const e2h_delta_args a
   }
 }
 
-// What one wave of the scan reads of a chunk: its 16 token rows of k, q, T and the decayed q k^T, its values and, in wave 0, the
-// decays.  None of it depends on the state, so it is fetched a chunk ahead.
+// What one wave of the scan reads of a chunk: its 16 token rows of k, T and v, or of q and the decayed q k^T.  None of it
+// depends on the state, so it is fetched a chunk ahead.
 template <int DT>
 struct ChunkRows {
-  f32x4_t k[DT], q[DT], t[4], p[4], v;
+  f32x4_t rows[DT], square[4], v;
   float log_g;
 };
 
-// step 2: DT = head dimension in tiles of 16.  Four waves; wave w owns the token rows 16 w .. 16 w + 15 of every chunk and the
-// state's row tiles w, w + 4, ...  The state is kept twice: in accumulators by its owner, and in LDS, transposed, as the B
-// operand of everybody's read-outs.  The keys go through LDS once to be read transposed in the state update.
+// step 2: DT = head dimension in tiles of 16.  Eight waves: wave w < 4 owns the token rows 16 w .. 16 w + 15 on the writing side
+// (k, T, v: what u is made of), wave w + 4 the same rows on the reading side (q and the outputs); the state's row tiles w, w + 8
+// are wave w's.  The state is kept twice: in accumulators by its owner, and in LDS, transposed, as the B operand of
+// everybody's read-outs.  The keys go through LDS once to be read transposed in the state update.
 // WHOLE: the head dimension fills its tiles, so no load needs a mask (rows past the end are read from the last token: their beta is
 // 0, which keeps them out of u, and their outputs are not stored).
 template <int DT, bool WHOLE>
-__global__ __launch_bounds__(256, 1) void delta_scan_kernel(const e2h_delta_args a, Prepared p, ChunkScratch cs, int v_blocks) {
-  constexpr int DP = DT * 16, OWN = DT / 4, kRow = DP + 4, kTok = 20;
-  constexpr bool kAhead = DT <= 8;  // wider heads leave no registers for the next chunk
-  __shared__ __attribute__((aligned(16))) float st[16 * kRow];                       // state, [value column][row]
-  __shared__ __attribute__((aligned(16))) float sk[kChunk * kRow];                   // keys, [token][channel]
+__global__ __launch_bounds__(512) void delta_scan_kernel(const e2h_delta_args a, Prepared p, ChunkScratch cs, int v_blocks) {
+  constexpr int DP = DT * 16, OWN = (DT + 7) / 8, kRow = DP + 4, kTok = 20;
+  __shared__ __attribute__((aligned(16))) float st[16 * kRow];                         // state, [value column][row]
+  __shared__ __attribute__((aligned(16))) float sk[kChunk * kRow];                     // keys, [token][channel]
   __shared__ __attribute__((aligned(16))) float sx[kChunk * kTok], su[kChunk * kTok];  // [token][value column]
   __shared__ float sg[2][kChunk];
   const int D = static_cast<int>(a.dim), DV = static_cast<int>(a.vdim), H = static_cast<int>(a.heads), kvh = static_cast<int>(a.kv_heads);
@@ -497,6 +516,8 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(const e2h_delta_args
   }
   const int b = bh / H, h = bh % H, hk = h / (H / kvh);
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), c = threadIdx.x & 15, b4 = (threadIdx.x & 63) >> 4;
+  const bool reader = wave >= 4;
+  const int block = wave & 3;  // of 16 tokens
   const int col = vb * 16 + c;
   const bool col_ok = col < DV;
   float *state = a.state + static_cast<size_t>(bh) * D * DV;
@@ -504,42 +525,37 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(const e2h_delta_args
   f32x4_t s[OWN];
 #pragma unroll
   for (int i = 0; i < OWN; ++i) {
-    const int dt = wave + 4 * i;
+    const int dt = wave + 8 * i;
     s[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int d = dt * 16 + 4 * b4 + r;
       if (carried && d < D && col_ok) s[i][r] = state[static_cast<size_t>(d) * DV + col];
     }
-    store4(st + c * kRow + dt * 16 + 4 * b4, s[i]);
+    if (dt < DT) store4(st + c * kRow + dt * 16 + 4 * b4, s[i]);
   }
   const size_t stride = static_cast<size_t>(kvh) * D;
-  const int tr = 16 * wave + c;
+  const int tr = 16 * block + c;
   const size_t seq0 = static_cast<size_t>(b) * seqlen;
-  const float *squares_t = cs.t + static_cast<size_t>(bh) * cs.chunks * kChunk * kChunk, *squares_p = cs.p + static_cast<size_t>(bh) * cs.chunks * kChunk * kChunk;
+  const float *squares = (reader ? cs.p : cs.t) + static_cast<size_t>(bh) * cs.chunks * kChunk * kChunk;
+  const float *vectors = reader ? p.q : p.k;
 
   auto fetch = [&](int chunk, ChunkRows<DT> &x) {
     const size_t row0 = seq0 + static_cast<size_t>(chunk) * kChunk;
     const int live = seqlen - chunk * kChunk < kChunk ? seqlen - chunk * kChunk : kChunk;
-    const float *kb = p.k + (row0 * kvh + hk) * D, *qb = p.q + (row0 * kvh + hk) * D;
-    const float *tt = squares_t + static_cast<size_t>(chunk) * kChunk * kChunk, *pt = squares_p + static_cast<size_t>(chunk) * kChunk * kChunk;
-    const size_t mine = (tr < live ? tr : live - 1) * stride;
+    const float *mine = vectors + ((row0 + (tr < live ? tr : live - 1)) * kvh + hk) * D;
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
-      const int d = dt * 16 + 4 * b4;
-      x.k[dt] = WHOLE ? load4(kb + mine + d) : row4(kb + mine, true, d, D);
-      x.q[dt] = WHOLE ? load4(qb + mine + d) : row4(qb + mine, true, d, D);
-    }
+    for (int dt = 0; dt < DT; ++dt) x.rows[dt] = WHOLE ? load4(mine + dt * 16 + 4 * b4) : row4(mine, true, dt * 16 + 4 * b4, D);
+    const float *sq = squares + static_cast<size_t>(chunk) * kChunk * kChunk + tr * kChunk + 4 * b4;
 #pragma unroll
     for (int j = 0; j < 4; ++j)
-      if (j <= wave) {
-        x.t[j] = load4(tt + tr * kChunk + 16 * j + 4 * b4);
-        x.p[j] = load4(pt + tr * kChunk + 16 * j + 4 * b4);
-      }
+      if (j <= block) x.square[j] = load4(sq + 16 * j);
+    if (!reader) {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = 16 * wave + 4 * b4 + r;
-      x.v[r] = p.v[((row0 + (t < live ? t : live - 1)) * H + h) * DV + (col_ok ? col : 0)];
+      for (int r = 0; r < 4; ++r) {
+        const int t = 16 * block + 4 * b4 + r;
+        x.v[r] = p.v[((row0 + (t < live ? t : live - 1)) * H + h) * DV + (col_ok ? col : 0)];
+      }
     }
     if (wave == 0) x.log_g = p.log_g[(row0 + (static_cast<int>(threadIdx.x) < live ? threadIdx.x : live - 1)) * H + h];
   };
@@ -547,9 +563,10 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(const e2h_delta_args
   ChunkRows<DT> cur, next;
   fetch(0, cur);
   for (int chunk = 0; chunk < cs.chunks; ++chunk) {
+    const int live = seqlen - chunk * kChunk < kChunk ? seqlen - chunk * kChunk : kChunk;
     float *g = sg[chunk & 1];
     if (wave == 0) {
-      float x = static_cast<int>(threadIdx.x) < seqlen - chunk * kChunk ? cur.log_g : 0.f;
+      float x = static_cast<int>(threadIdx.x) < live ? cur.log_g : 0.f;
 #pragma unroll
       for (int off = 1; off < 64; off <<= 1) {
         const float up = __shfl_up(x, off);
@@ -557,50 +574,49 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(const e2h_delta_args
       }
       g[threadIdx.x] = x * kLog2e;
     }
+    if (!reader) {
 #pragma unroll
-    for (int dt = 0; dt < DT; ++dt) store4(sk + tr * kRow + dt * 16 + 4 * b4, cur.k[dt]);
-    if (kAhead && chunk + 1 < cs.chunks) fetch(chunk + 1, next);
-    lds_barrier();  // state, keys and decays of this chunk are in LDS; the loads above stay in flight
-    f32x4_t ks = {0.f, 0.f, 0.f, 0.f}, qs = ks;
-#pragma unroll
-    for (int dt = 0; dt < DT; ++dt) {
-      const f32x4_t sb = load4(st + c * kRow + dt * 16 + 4 * b4);
-      ks = mfma4(cur.k[dt], sb, ks);
-      qs = mfma4(cur.q[dt], sb, qs);
+      for (int dt = 0; dt < DT; ++dt) store4(sk + tr * kRow + dt * 16 + 4 * b4, cur.rows[dt]);
     }
-    f32x4_t gt;
+    if (chunk + 1 < cs.chunks) fetch(chunk + 1, next);
+    lds_barrier();  // state, keys and decays of this chunk are in LDS; the loads above stay in flight
+    f32x4_t y = {0.f, 0.f, 0.f, 0.f}, gt;  // S0^T k or S0^T q, decayed to each token
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) y = mfma4(cur.rows[dt], load4(st + c * kRow + dt * 16 + 4 * b4), y);
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      gt[r] = __builtin_amdgcn_exp2f(g[16 * wave + 4 * b4 + r]);
-      sx[(16 * wave + 4 * b4 + r) * kTok + c] = cur.v[r] - gt[r] * ks[r];
+      gt[r] = __builtin_amdgcn_exp2f(g[16 * block + 4 * b4 + r]);
+      y[r] *= gt[r];
+      if (!reader) sx[(16 * block + 4 * b4 + r) * kTok + c] = cur.v[r] - y[r];
     }
     lds_barrier();
-    f32x4_t u = {0.f, 0.f, 0.f, 0.f};
+    if (!reader) {
+      f32x4_t u = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      if (j > wave) break;
-      f32x4_t x;
+      for (int j = 0; j < 4; ++j) {
+        if (j > block) break;
+        f32x4_t x;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) x[r] = sx[(16 * j + 4 * b4 + r) * kTok + c];
-      u = mfma4(cur.t[j], x, u);
+        for (int r = 0; r < 4; ++r) x[r] = sx[(16 * j + 4 * b4 + r) * kTok + c];
+        u = mfma4(cur.square[j], x, u);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) su[(16 * block + 4 * b4 + r) * kTok + c] = u[r];
     }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) su[(16 * wave + 4 * b4 + r) * kTok + c] = u[r];
     lds_barrier();
-    f32x4_t o, ub[4];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) o[r] = gt[r] * qs[r];
+    f32x4_t ub[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) ub[j][r] = su[(16 * j + 4 * b4 + r) * kTok + c];
-      if (j <= wave) o = mfma4(cur.p[j], ub[j], o);
+      if (reader && j <= block) y = mfma4(cur.square[j], ub[j], y);
     }
-    const int live = seqlen - chunk * kChunk < kChunk ? seqlen - chunk * kChunk : kChunk;
+    if (reader) {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {  // over the values this workgroup has read
-      const int t = 16 * wave + 4 * b4 + r;
-      if (t < live && col_ok) p.v[((seq0 + static_cast<size_t>(chunk) * kChunk + t) * H + h) * DV + col] = o[r];
+      for (int r = 0; r < 4; ++r) {  // over the values this workgroup has read
+        const int t = 16 * block + 4 * b4 + r;
+        if (t < live && col_ok) p.v[((seq0 + static_cast<size_t>(chunk) * kChunk + t) * H + h) * DV + col] = y[r];
+      }
     }
     const float g_end = g[kChunk - 1], dec = __builtin_amdgcn_exp2f(g_end);
 #pragma unroll
@@ -609,26 +625,26 @@ __global__ __launch_bounds__(256, 1) void delta_scan_kernel(const e2h_delta_args
       for (int r = 0; r < 4; ++r) ub[j][r] *= __builtin_amdgcn_exp2f(g_end - g[16 * j + 4 * b4 + r]);
 #pragma unroll
     for (int i = 0; i < OWN; ++i) {
+      if (wave + 8 * i >= DT) break;
 #pragma unroll
       for (int r = 0; r < 4; ++r) s[i][r] *= dec;
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         f32x4_t kt;
 #pragma unroll
-        for (int r = 0; r < 4; ++r) kt[r] = sk[(16 * j + 4 * b4 + r) * kRow + (wave + 4 * i) * 16 + c];
+        for (int r = 0; r < 4; ++r) kt[r] = sk[(16 * j + 4 * b4 + r) * kRow + (wave + 8 * i) * 16 + c];
         s[i] = mfma4(kt, ub[j], s[i]);
       }
-      store4(st + c * kRow + (wave + 4 * i) * 16 + 4 * b4, s[i]);
+      store4(st + c * kRow + (wave + 8 * i) * 16 + 4 * b4, s[i]);
     }
     lds_barrier();  // the keys have been read; the next chunk's take their place
-    if (kAhead) cur = next;
-    else if (chunk + 1 < cs.chunks) fetch(chunk + 1, cur);
+    cur = next;
   }
 #pragma unroll
   for (int i = 0; i < OWN; ++i)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      const int d = (wave + 4 * i) * 16 + 4 * b4 + r;
+      const int d = (wave + 8 * i) * 16 + 4 * b4 + r;
       if (d < D && col_ok) state[static_cast<size_t>(d) * DV + col] = s[i][r];
     }
 }
@@ -673,7 +689,7 @@ bool use_chunks(const e2h_delta_args &a) {
 template <int DT>
 void launch_scan(const e2h_delta_args &a, const Prepared &p, const ChunkScratch &cs, hipStream_t s) {
   const int v_blocks = static_cast<int>((a.vdim + 15) / 16);
-  const dim3 grid(static_cast<unsigned>(a.batch * a.heads * v_blocks)), block(256);
+  const dim3 grid(static_cast<unsigned>(a.batch * a.heads * v_blocks)), block(512);
   if (a.dim == DT * 16) hipLaunchKernelGGL((delta_scan_kernel<DT, true>), grid, block, 0, s, a, p, cs, v_blocks);
   else hipLaunchKernelGGL((delta_scan_kernel<DT, false>), grid, block, 0, s, a, p, cs, v_blocks);
 }

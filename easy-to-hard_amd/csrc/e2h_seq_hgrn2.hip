@@ -46,7 +46,7 @@ __global__ __launch_bounds__(BLOCK) void hgrn2_tokens_kernel(const e2h_hgrn2_arg
   for (int i = 0; i < RPT; ++i) {
     const int r = rg + RG * i;
     s[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    if (pos0 > 0 && col_ok && r < D) s[i] = load4(st + static_cast<size_t>(r) * DV + cg * 4);
+    if (pos0 > 0 && col_ok && r < D) s[i] = load4_stream(st + static_cast<size_t>(r) * DV + cg * 4);
   }
   const T *proj = static_cast<const T *>(a.proj);
   for (int t = 0; t < seqlen; ++t) {
@@ -96,7 +96,7 @@ __global__ __launch_bounds__(BLOCK) void hgrn2_tokens_kernel(const e2h_hgrn2_arg
 #pragma unroll
   for (int i = 0; i < RPT; ++i) {
     const int r = rg + RG * i;
-    if (col_ok && r < D) store4(st + static_cast<size_t>(r) * DV + cg * 4, s[i]);
+    if (col_ok && r < D) store4_stream(st + static_cast<size_t>(r) * DV + cg * 4, s[i]);
   }
 }
 
