@@ -1,5 +1,5 @@
 """Prefill and decode throughput of the Refatar decoder on random weights at layer sizes of real models, beside the
-Llama-family Transformer of equal width, depth, heads and parameter count per layer (bench.py --refatar)."""
+Llama-family Transformer of equal width, depth, attention heads and parameter count (bench.py --refatar)."""
 
 import time
 
@@ -9,7 +9,7 @@ from . import generate
 from .model import ModelArgs, random_quantized_transformer
 from .refatar import Refatar
 
-# layers alternate between the two mixers; the comparison's gated feed-forward has 2/3 of the hidden size (three matrices)
+# layers alternate between the two mixers
 SIZES = {
     "1b": dict(width=2048, ff=8192, heads=16, kv_heads=4, dim=128, recurrent_heads=16, recurrent_dim=128, delta_kv=8, window=1024, keep=4,
                side=128, layers=8, vocab=32000),
@@ -37,9 +37,13 @@ def random_refatar(config, device):
 
 
 def closest_model(s, device):
-    ff = (s["ff"] * 2 // 3 + 255) // 256 * 256
-    cfg = ModelArgs(block_size=32768, vocab_size=s["vocab"], n_layer=s["layers"], n_head=s["heads"], n_local_heads=s["kv_heads"], dim=s["width"],
-                    intermediate_size=ff)
+    """Llama-family model of the same width, depth and attention heads whose feed-forward makes up the same parameter count."""
+    with torch.device("meta"):
+        total = parameters(Refatar.from_config(refatar_config(s)))
+    w, n = s["width"], s["layers"]
+    rest = total - s["vocab"] * w - n * (w * w * 2 + 2 * w * s["kv_heads"] * s["dim"])
+    ff = round(rest / (n * 3 * w * 256)) * 256
+    cfg = ModelArgs(block_size=32768, vocab_size=s["vocab"], n_layer=n, n_head=s["heads"], n_local_heads=s["kv_heads"], dim=w, intermediate_size=ff)
     return random_quantized_transformer(cfg, "bf16", device=device)
 
 

@@ -53,9 +53,10 @@ def build_mixer(plan: StatePlan, width: int, layer: dict, eps: float) -> TokenMi
     if layer["type"] == "delta":
         return TokenMixer(width, [GatedDelta(plan, width, m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["conv"], eps)], [""])
     left, right = m["left"], m["right"]
+    mask = left.get("mask") or {}
     return TokenMixer(width, [
-        WindowAttention(plan, width, left["heads"], left["kv_heads"], left["dim"], left["vdim"], left["scale"], left["mask"]["size"],
-                        left["mask"]["keep_first"], m["left_scale"]),
+        WindowAttention(plan, width, left["heads"], left["kv_heads"], left["dim"], left["vdim"], left["scale"], mask.get("size", 0),
+                        mask.get("keep_first", 0), m["left_scale"]),
         HGRN2(plan, width, right["heads"], right["dim"], right["vdim"], eps, m["right_scale"]),
     ], ["left", "right"])
 
